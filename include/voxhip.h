@@ -357,7 +357,8 @@ int vox_lm_prefill(vox_lm* m, void* stream, const vox_lm_io* io, const int32_t* 
  * A decoder whose layers mix tokens with a linear recurrence (HGRN2, mLSTM, a real-gated diagonal unit behind a short
  * convolution, a matrix state with token shift and per-channel decay, retention, the gated delta rule) or with attention
  * over a paged cache (a sliding window that also keeps one mean key / value per block of older tokens, plain causal
- * attention with normed q / k / v, or attention over a cached low-rank latent); two mixers may run side by side on the
+ * attention with normed q / k / v, attention over a cached low-rank latent, or attention whose key weights are independent
+ * sigmoids inside position chunks); two mixers may run side by side on the
  * same input; a layer's outputs may carry a layer scale; a contiguous range of layers may run several times with the
  * same weights (every run owns its cache or state).  A layer is sequential (x += mixer(norm1 x); x += ff(norm2 x)) or
  * parallel (x += mixer(norm1 x) + ff(norm2 x)); the feed-forward is dense or a routed mixture of experts.  Residual
@@ -366,13 +367,14 @@ int vox_lm_prefill(vox_lm* m, void* stream, const vox_lm_io* io, const int32_t* 
  * (prompt portions next to single decoded tokens); rows of a request are contiguous and ascending in position.      */
 typedef struct vox_hybrid vox_hybrid;
 enum { VOX_MIXER_HGRN2 = 0, VOX_MIXER_POOLED_WINDOW_ATTN = 1, VOX_MIXER_MLSTM = 2, VOX_MIXER_RGLRU = 3, VOX_MIXER_CAUSAL_ATTN = 4,
-       VOX_MIXER_SHIFT_DECAY = 5, VOX_MIXER_LATENT_ATTN = 6, VOX_MIXER_RETENTION = 7, VOX_MIXER_DELTA = 8 };
+       VOX_MIXER_SHIFT_DECAY = 5, VOX_MIXER_LATENT_ATTN = 6, VOX_MIXER_RETENTION = 7, VOX_MIXER_DELTA = 8,
+       VOX_MIXER_SIGMOID_ATTN = 9 };
 enum { VOX_HYBRID_BF16 = 0, VOX_HYBRID_F32 = 1 };
 enum { VOX_NORM_LAYER = 0 /* weight-only layer norm */, VOX_NORM_RMS_GROUPS = 1 /* RMS norm over norm_groups equal slices */ };
 /* sequential: x += mixer(norm1 x); x += ff(norm2 x).  parallel: x += mixer(norm1 x) + ff(norm2 x).  parallel, one norm:
  * x += mixer(n) + ff(n) with n = norm1 x (norm2 is not used) */
 enum { VOX_BLOCK_SEQUENTIAL = 0, VOX_BLOCK_PARALLEL = 1, VOX_BLOCK_PARALLEL_ONE_NORM = 2 };
-enum { VOX_FF_UP_DOWN = 0 /* down(gelu_erf(up h)) */, VOX_FF_GATED = 1 /* down(act(gate h + b) * (up h + b)) + b */ };
+enum { VOX_FF_UP_DOWN = 0 /* down(gelu_erf(up h)), with ff_act VOX_ACT_RELU2 down(max(up h, 0)^2) */, VOX_FF_GATED = 1 /* down(act(gate h + b) * (up h + b)) + b */ };
 enum { VOX_ACT_GELU_TANH = 0, VOX_ACT_SWISH = 1 /* g * sigmoid(alpha g) */, VOX_ACT_RELU2 = 2 /* max(g, 0)^2 */ };
 enum { VOX_EXPERT_GATED = 0 /* down(act(gate h) * (up h + up_offset)), clamped */, VOX_EXPERT_UP_DOWN = 1 /* down(act(up h)) */ };
 enum { VOX_GATE_NONE = 0, VOX_GATE_SIGMOID = 1, VOX_GATE_SILU = 2 };
@@ -397,6 +399,10 @@ typedef struct {
      * router_bias [experts + identity] fp32 or NULL is added to the router logits before the scores are formed. */
     int32_t expert_form, expert_act;
     const float* router_bias;
+    /* groups > 1: the experts form that many equal groups of neighbours; a group's score is its largest choice value, and only experts
+     * of the `keep` best groups can be chosen (identity = 0 then).  weight_scale multiplies the weights (0: as 1). */
+    int32_t groups, keep;
+    float weight_scale;
 } vox_hybrid_moe;
 typedef struct {
     int32_t kind, heads, kv_heads, dim, vdim;
@@ -410,6 +416,7 @@ typedef struct {
      *   mLSTM         q (heads*dim) | k (heads*dim) | v (heads*vdim) | output gate (heads*vdim) | input gate (heads) | forget gate (heads)
      *   RGLRU         gated branch (C) | recurrent branch (C), C = heads*dim channels in `heads` blocks of dim (= vdim)
      *   causal attn   q (heads*dim) | k (kv_heads*dim) | v (kv_heads*vdim)
+     *   sigmoid attn  q (heads*dim) | k (kv_heads*dim) | v (kv_heads*vdim) | output gate (heads*vdim; out_gate only)
      *   shift-decay   r | k | v | g (heads*dim each, dim = vdim) | decay bottleneck (lora); each of the five reads its own token-shift mix */
     const void* w_in;                     /* [n_in, width] engine dtype */
     const float* b_in;                    /* [n_in] fp32 or NULL */
@@ -482,6 +489,28 @@ typedef struct {
     int32_t decay_channels, gate_rank, gate_act;
     const void* w_gate2;
     const float *a_log, *dt_bias;
+    /* sigmoid attention (VOX_MIXER_SIGMOID_ATTN): q and k RMS-normed per head (q_norm, k_norm [dim]).  A position sees the positions
+     * up to itself in its own chunk (chunk > 0: positions with the same p / chunk; 0: all).  z = (q . k) * scale * head_temp[h];
+     * score_cap > 0: z <- cap * tanh(z / cap); z += dist_bias[h][min(distance, dist_n - 1)]; the key's weight is
+     * sigmoid(z + weight_bias[h]), nothing is normalised over the keys.  out_gate: every output column times the sigmoid of its gate. */
+    int32_t chunk, dist_n, out_gate;
+    float score_cap;
+    const float *head_temp, *dist_bias, *weight_bias;    /* [heads], [heads][dist_n], [heads]; each may be NULL */
+    /* latent attention: q_rank 0: the query has no latent, w_in starts with the heads' rows [dim plain | rot_dim rotated] in the place of
+     * the query latent's; no_head_gate: no gate rows and no gate; sinks [heads] or NULL: exp(sinks[h]) joins the softmax denominator;
+     * rot_mag: factor of the rotated vectors (0: as 1). */
+    int32_t no_head_gate;
+    float rot_mag;
+    const float* sinks;
+    /* residual gate (res_gate = width, or 0): a sublayer's result is multiplied column by column with sigmoid(W n + b), n being its
+     * normed input.  The mixer's gate rows follow its own rows in w_in / b_in; the up / down feed-forward's follow the up rows in
+     * w_up / b_up; a routed feed-forward's are w_gate_ff [width, width] and b_gate_ff.  Sequential layers only. */
+    int32_t res_gate;
+    const void* w_gate_ff;
+    const float* b_gate_ff;
+    /* several residual streams (config.streams = s > 0): sublayer i (0 mixer, 1 feed-forward) reads u = sum hc_in[i][a] x_a and
+     * leaves x_b <- sum hc_mix[i][a*s + b] x_a + hc_out[i][b] y, every new stream from the old ones; fp32 */
+    const float *hc_in[2], *hc_out[2], *hc_mix[2];
 } vox_hybrid_layer;
 typedef struct {
     int32_t layer;       /* index into layers */
@@ -507,6 +536,7 @@ typedef struct {
     /* bigram_buckets > 0: x0 += bigram[(prev * bigram_mul_prev + id * bigram_mul_cur) mod buckets], row `buckets` for a sequence's first token */
     int32_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;
     float logit_scale;                    /* logits <- logits * logit_scale (0: as 1) */
+    int32_t streams;                      /* > 0: that many copies of the residual stream, all the embedding at the start; the head reads their sum */
 } vox_hybrid_config;
 typedef struct {
     const vox_hybrid_layer* layers;

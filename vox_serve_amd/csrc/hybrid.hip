@@ -2,8 +2,10 @@
 // unit behind a short convolution, a matrix state with token shift and per-channel decay, retention, the gated delta rule behind
 // short convolutions) or with attention over a paged cache (a sliding window that also keeps one mean key / value per block of
 // older tokens, plain causal attention with normed q / k / v -- optionally behind a short convolution, rotated, with a softmax
-// sink --, or attention over a cached low-rank latent).  Two mixers may run side by side on one input; a layer is sequential or
-// parallel, with an optional layer scale; its feed-forward is dense or a routed mixture of experts.  A contiguous range of layers
+// sink --, attention over a cached low-rank latent, or attention with independent sigmoid weights inside position chunks).  Two mixers
+// may run side by side on one input; a layer is sequential or parallel, with an optional layer scale or a gate on what joins the
+// residual sum, over one residual stream or several that are mixed at every sublayer; its feed-forward is dense or a routed mixture of
+// experts.  A contiguous range of layers
 // may run several times with the same weights; every run owns its cache or recurrent state.
 //
 // Numeric rule of this engine: the residual stream, norms, rotary angles, attention scores / softmax, gates, decays and every
@@ -79,19 +81,55 @@ __device__ __forceinline__ float hb_dot_wave(const T* w, const float* x, int K, 
 }
 // HB_EPI_SOFTCAP: v <- arg * tanh(v / arg) (arg = the product's hb_rowmap::epi_arg)
 // HB_EPI_RESID_SCALED: c += v * col_scale[column] (a layer scale; arg = that column's entry); HB_EPI_SCALE: v <- v * arg
-enum { HB_EPI_STORE = 0, HB_EPI_GELU = 1, HB_EPI_RESID = 2, HB_EPI_TANH = 3, HB_EPI_SOFTCAP = 4, HB_EPI_RESID_SCALED = 5, HB_EPI_SCALE = 6 };
+// HB_EPI_RELU2: the square of relu on columns below arg, the others as they are; HB_EPI_JOIN: hb_join_add (hb_rowmap::join)
+enum { HB_EPI_STORE = 0, HB_EPI_GELU = 1, HB_EPI_RESID = 2, HB_EPI_TANH = 3, HB_EPI_SOFTCAP = 4, HB_EPI_RESID_SCALED = 5, HB_EPI_SCALE = 6,
+       HB_EPI_RELU2 = 7, HB_EPI_JOIN = 8 };
 template <int EPI> __device__ __forceinline__ void hb_epilogue(float* c, float acc, float bias, float arg = 0.f) {
     float v = acc + bias;
     if (EPI == HB_EPI_GELU) v = 0.5f * v * (1.0f + erff(v * 0.70710678118654752440f));
     if (EPI == HB_EPI_TANH) v = tanhf(v);
     if (EPI == HB_EPI_SOFTCAP) v = arg * tanhf(v / arg);
     if (EPI == HB_EPI_SCALE) v = v * arg;
+    if (EPI == HB_EPI_RELU2 && arg != 0.f) { const float r = fmaxf(v, 0.f); v = r * r; }
     if (EPI == HB_EPI_RESID) v = *c + v;
     if (EPI == HB_EPI_RESID_SCALED) v = *c + v * arg;
     *c = v;
 }
 __device__ __forceinline__ float hb_gelu_tanh(float z) {
     return 0.5f * z * (1.0f + tanhf(0.79788456080286535588f * (z + 0.044715f * z * z * z)));
+}
+// How a sublayer's result v joins the residual stream at (row, col): v is multiplied by sigmoid(gate logit) and by a layer scale where
+// they are given; then x += v, or -- several streams -- x_t <- sum_s mix[s*streams + t] x_s + out[t] v for all streams at once, and
+// u = sum_t next[t] x_t, what the next sublayer (or the head: all ones) reads, is left beside them.  Streams of a row lie `sld` apart.
+// One thread owns all streams of a (row, col), so the update is in place.
+#define HB_MAX_STREAMS 8
+struct hb_join {
+    const float* gate;
+    long ldg;
+    const float* scale;
+    int streams, sld;
+    const float *mix, *out, *next;
+    float* u;
+    long ldu;
+};
+__device__ __forceinline__ void hb_join_add(const hb_join& j, float* x, int row, int col, float v) {
+    if (j.gate) v *= hb_sigmoid(j.gate[(size_t)row * j.ldg + col]);
+    if (j.scale) v *= j.scale[col];
+    if (j.streams == 0) { x[col] += v; return; }
+    float xs[HB_MAX_STREAMS];
+#pragma unroll
+    for (int s = 0; s < HB_MAX_STREAMS; ++s) xs[s] = s < j.streams ? x[(size_t)s * j.sld + col] : 0.f;
+    float u = 0.f;
+    for (int t = 0; t < j.streams; ++t) {
+        float nx = 0.f;
+#pragma unroll
+        for (int s = 0; s < HB_MAX_STREAMS; ++s)
+            if (s < j.streams) nx = fmaf(j.mix[s * j.streams + t], xs[s], nx);
+        nx = fmaf(j.out[t], v, nx);
+        x[(size_t)t * j.sld + col] = nx;
+        u = fmaf(j.next[t], nx, u);
+    }
+    j.u[(size_t)row * j.ldu + col] = u;
 }
 // Several products in one launch: product z uses the matrix Wt + z*w_stride, the activations A + z*a_stride, the outputs
 // C + z*c_stride and the bias + z*b_stride (a strided batch: block-diagonal matrices, projections that each read their own input).
@@ -105,13 +143,21 @@ struct hb_rowmap {
     const float* a_scale;
     float epi_arg;
     const float* col_scale;     // HB_EPI_RESID_SCALED: [N] fp32
+    hb_join join;               // HB_EPI_JOIN
 };
-static inline hb_rowmap hb_plain() { return hb_rowmap{nullptr, nullptr, 0, 1, 0, 0, 0, 0, nullptr, 0.f, nullptr}; }
+static inline hb_rowmap hb_plain() { return hb_rowmap{nullptr, nullptr, 0, 1, 0, 0, 0, 0, nullptr, 0.f, nullptr, {}}; }
 template <int EPI> __device__ __forceinline__ float hb_epi_arg(const hb_rowmap& rm, int col) {
+    if (EPI == HB_EPI_RELU2) return col < (int)rm.epi_arg ? 1.0f : 0.0f;
     return EPI == HB_EPI_RESID_SCALED ? rm.col_scale[col] : rm.epi_arg;
+}
+// a product's result at (row, col) of C
+template <int EPI> __device__ __forceinline__ void hb_finish(const hb_rowmap& rm, float* C, long ldc, int row, int col, float acc, float bias) {
+    if (EPI == HB_EPI_JOIN) hb_join_add(rm.join, C + (size_t)row * ldc, row, col, acc + bias);
+    else hb_epilogue<EPI>(C + (size_t)row * ldc + col, acc, bias, hb_epi_arg<EPI>(rm, col));
 }
 
 // ---- embedding gather: x[row] = table[id]; the second half of both residual buffers keeps the embedding output ----------
+// streams > 0: every stream of xa [row][streams][W] is the embedding, u = what the first sublayer reads of them (s_in: its weights).
 // A bigram table (bg.table != NULL) adds row (prev * mul_prev + id * mul_cur) mod buckets, prev being the token before this one in its
 // sequence: the previous row of the request, or what the request's state slot remembers, or nothing at position 0 (row `buckets`).
 // Steps with one row per request (bg.store) also leave the row's id in the slot; other steps do that in k_hb_store_prev, after every
@@ -125,7 +171,7 @@ __device__ __forceinline__ int hb_clamp_id(int id, int vocab) { return id < 0 ? 
 template <typename T>
 __global__ __launch_bounds__(256) void k_hb_embed(const T* table, const int* ids, int id_stride, float* xa, float* xb, int W, int vocab,
                                                   float scale, hb_bigram bg, const int* pos, const int* row_req, const int* req_rows,
-                                                  const int* req_state) {
+                                                  const int* req_state, int streams, const float* s_in, float* u) {
     const int row = blockIdx.x;
     const int id = hb_clamp_id(ids[(size_t)row * id_stride], vocab);
     const T* extra = nullptr;
@@ -143,6 +189,15 @@ __global__ __launch_bounds__(256) void k_hb_embed(const T* table, const int* ids
     for (int i = threadIdx.x; i < W; i += 256) {
         float v = hb_ld(table + (size_t)id * W + i) * scale;
         if (extra) v += hb_ld(extra + i);
+        if (streams > 0) {
+            float t = 0.f;
+            for (int s = 0; s < streams; ++s) {
+                xa[((size_t)row * streams + s) * W + i] = v;
+                t = fmaf(s_in[s], v, t);
+            }
+            u[(size_t)row * W + i] = t;
+            continue;
+        }
         xa[(size_t)row * 2 * W + i] = v;
         xa[(size_t)row * 2 * W + W + i] = v;
         xb[(size_t)row * 2 * W + W + i] = v;
@@ -422,7 +477,7 @@ __global__ __launch_bounds__(256) void k_hb_gemm_bf16(const float* A, long lda, 
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int gm = m0 + (mt0 + i) * 16 + (lane >> 4) * 4 + r;
-                if (gm < M) hb_epilogue<EPI>(C + (size_t)(lst ? lst[gm] : gm) * ldc + gn, acc[i][j][r], b, hb_epi_arg<EPI>(rm, gn));
+                if (gm < M) hb_finish<EPI>(rm, C, ldc, lst ? lst[gm] : gm, gn, acc[i][j][r], b);
             }
         }
 }
@@ -491,7 +546,7 @@ __global__ __launch_bounds__(256) void k_hb_gemm_f32(const float* A, long lda, c
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int gn = n0 + tx * 4 + j;
-            if (gn < N) hb_epilogue<EPI>(C + (size_t)arow[ty * RM + i] * ldc + gn, acc[i][j], bias ? bias[gn] : 0.f, hb_epi_arg<EPI>(rm, gn));
+            if (gn < N) hb_finish<EPI>(rm, C, ldc, arow[ty * RM + i], gn, acc[i][j], bias ? bias[gn] : 0.f);
         }
     }
 }
@@ -565,7 +620,7 @@ __global__ __launch_bounds__(256) void k_hb_gemv(const float* A, long lda, const
 #pragma unroll
         for (int j = 0; j < HB_GEMV_CPW; ++j) {
             const float sum = hb_wave_sum(acc[m][j]);
-            if (m < M && n0 + j < N && lane == 0) hb_epilogue<EPI>(C + (size_t)m * ldc + n0 + j, sum, bias ? bias[n0 + j] : 0.f, hb_epi_arg<EPI>(rm, n0 + j));
+            if (m < M && n0 + j < N && lane == 0) hb_finish<EPI>(rm, C, ldc, m, n0 + j, sum, bias ? bias[n0 + j] : 0.f);
         }
 }
 
@@ -636,7 +691,8 @@ __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, co
 #pragma unroll
     for (int j = 0; j < CPW; ++j) {
         const float sum = hb_wave_sum(acc[j]);
-        if (n0 + j < N && lane == 0) hb_epilogue<EPI>(C + n0 + j, sum, bias ? bias[n0 + j] : 0.f, epi_arg);
+        const float arg = EPI == HB_EPI_RELU2 ? (n0 + j < (int)epi_arg ? 1.0f : 0.0f) : epi_arg;
+        if (n0 + j < N && lane == 0) hb_epilogue<EPI>(C + n0 + j, sum, bias ? bias[n0 + j] : 0.f, arg);
     }
 }
 // true: the fused form was launched (one row, aligned operands); false: the caller normalises and multiplies in two launches
@@ -654,6 +710,7 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
     } while (0)
     if (epi == HB_EPI_GELU) HB_LN(HB_EPI_GELU);
     else if (epi == HB_EPI_SCALE) HB_LN(HB_EPI_SCALE);
+    else if (epi == HB_EPI_RELU2) HB_LN(HB_EPI_RELU2);
     else if (epi != HB_EPI_STORE) return false;
     else HB_LN(HB_EPI_STORE);
 #undef HB_LN
@@ -709,7 +766,7 @@ __global__ __launch_bounds__(512) void k_hb_gemm_rows16(const float* A, long lda
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int row = kb * 4 + r;
-            if (row < M) hb_epilogue<EPI>(C + (size_t)row * ldc + n0 + col, ((((((red[0][row][col] + red[1][row][col]) + red[2][row][col]) + red[3][row][col]) + red[4][row][col]) + red[5][row][col]) + red[6][row][col]) + red[7][row][col], bz, hb_epi_arg<EPI>(rm, n0 + col));
+            if (row < M) hb_finish<EPI>(rm, C, ldc, row, n0 + col, ((((((red[0][row][col] + red[1][row][col]) + red[2][row][col]) + red[3][row][col]) + red[4][row][col]) + red[5][row][col]) + red[6][row][col]) + red[7][row][col], bz);
         }
     }
 }
@@ -773,6 +830,8 @@ int hb_gemm(hipStream_t st, int epi, const float* A, long lda, const T* W, const
     if (epi == HB_EPI_SOFTCAP) return hb_gemm_epi<T, HB_EPI_SOFTCAP>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
     if (epi == HB_EPI_RESID_SCALED) return hb_gemm_epi<T, HB_EPI_RESID_SCALED>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
     if (epi == HB_EPI_SCALE) return hb_gemm_epi<T, HB_EPI_SCALE>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
+    if (epi == HB_EPI_RELU2) return hb_gemm_epi<T, HB_EPI_RELU2>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
+    if (epi == HB_EPI_JOIN) return hb_gemm_epi<T, HB_EPI_JOIN>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
     return hb_gemm_epi<T, HB_EPI_STORE>(st, A, lda, W, bias, C, ldc, M, N, K, rm, nz);
 }
 
@@ -949,12 +1008,14 @@ __global__ __launch_bounds__(64 * HB_SCAN_MAX_WAVES) void k_hb_mlstm_scan(const 
 
 // Rotation of the newer mixers: dims i and i + rot/2 (i < rot/2) of a vector form a pair (u, v) that position p turns by the angle
 // p * inv_freq[i] into (u cos - v sin, v cos + u sin); dims at or beyond rot pass unchanged.  x: the vector, d: the dim asked for.
-__device__ __forceinline__ float hb_rot_half(const float* x, int d, int rot, float p, const float* inv_freq) {
+__device__ __forceinline__ float hb_rot_half(const float* x, int d, int rot, float p, const float* inv_freq, float mag = 1.0f) {
     const float v = x[d];
     if (d >= rot) return v;
     const int half = rot >> 1, i = d < half ? d : d - half;
     float sn, cs;
     sincosf(p * inv_freq[i], &sn, &cs);
+    sn *= mag;
+    cs *= mag;
     return d < half ? v * cs - x[d + half] * sn : v * cs + x[d - half] * sn;
 }
 
@@ -1080,41 +1141,50 @@ __global__ __launch_bounds__(256) void k_hb_retention_carry(float* ws, float* st
 }
 
 // ---- latent attention: what a row leaves in the cache, and its query ----------------------------------------------------------
-// proj row = [query latent (q_rank) | key / value latent (R) | rotated key part (r) | gate (H) | ...].  Block (row, 0): the query latent
-// is RMS-normed with its weight in place.  Block (row, 1): the key / value latent is RMS-normed with its weight into the row's cache
-// entry [R + r] (engine dtype), followed by the rotated key part (hb_rot_half on its first `rot` dims).
+// proj row = [query latent (q_rank), or without one the query itself (q_rank = 0) | key / value latent (R) at kv_off | rotated key part
+// (r) | ...].  Block (row, 0): the key / value latent is RMS-normed with its weight into the row's cache entry [R + r] (engine dtype),
+// followed by the rotated key part (hb_rot_half on its first `rot` dims).  Block (row, 1) with a query latent: it is RMS-normed with its
+// weight in place.  Blocks (row, 1..) without one: the rotated query parts of 8 heads each (what k_hb_latent_qrot does otherwise).
+#define HB_LAT_QROT_HEADS 8
+__device__ __forceinline__ void hb_latent_qrot_head(const float* q, float* qa, const float* inv_freq, float pf, int h, int d, int dim, int R, int r,
+                                                    int rot, float mag) {
+    qa[(size_t)h * (R + r) + R + d] = hb_rot_half(q + (size_t)h * (dim + r) + dim, d, rot, pf, inv_freq, mag);
+}
 template <typename T>
 __global__ __launch_bounds__(256) void k_hb_latent_prep(float* proj, long ldp, T* cache, const float* qn, const float* kn, const float* inv_freq,
-                                                        const int* pos, const int* page, const int* slot, int q_rank, int R, int r, int rot,
-                                                        int ps, float eps) {
+                                                        const int* pos, const int* page, const int* slot, int q_rank, int kv_off, int R, int r,
+                                                        int rot, int ps, float eps, float mag, int H, int dim, int off_qa) {
     __shared__ float red[4];
     const int row = blockIdx.x;
     float* p = proj + (size_t)row * ldp;
-    if (blockIdx.y == 0) {
+    const float pf = (float)pos[row];
+    if (blockIdx.y > 0 && q_rank > 0) {
         float ss = 0.f;
         for (int i = threadIdx.x; i < q_rank; i += 256) ss = fmaf(p[i], p[i], ss);
         const float inv = 1.0f / sqrtf(hb_block_sum256(ss, red) / (float)q_rank + eps);
         for (int i = threadIdx.x; i < q_rank; i += 256) p[i] = p[i] * inv * qn[i];
         return;
     }
-    const float* x = p + q_rank;
+    if (blockIdx.y > 0) {
+        const int h0 = (blockIdx.y - 1) * HB_LAT_QROT_HEADS, nh = H - h0 < HB_LAT_QROT_HEADS ? H - h0 : HB_LAT_QROT_HEADS;
+        for (int i = threadIdx.x; i < nh * r; i += 256) hb_latent_qrot_head(p, p + off_qa, inv_freq, pf, h0 + i / r, i % r, dim, R, r, rot, mag);
+        return;
+    }
+    const float* x = p + kv_off;
     float ss = 0.f;
     for (int i = threadIdx.x; i < R; i += 256) ss = fmaf(x[i], x[i], ss);
     const float inv = 1.0f / sqrtf(hb_block_sum256(ss, red) / (float)R + eps);
     T* dst = cache + ((size_t)page[row] * ps + slot[row]) * (size_t)(R + r);
     for (int i = threadIdx.x; i < R; i += 256) hb_st(dst + i, x[i] * inv * kn[i]);
-    const float pf = (float)pos[row];
-    for (int d = threadIdx.x; d < r; d += 256) hb_st(dst + R + d, hb_rot_half(x + R, d, rot, pf, inv_freq));
+    for (int d = threadIdx.x; d < r; d += 256) hb_st(dst + R + d, hb_rot_half(x + R, d, rot, pf, inv_freq, mag));
 }
 // q row = per head [plain (dim) | rotated (r)]; qa row = per head [query against the latent (R) | rotated part (r)].  The first part
 // of qa is a product of its own (the plain part times the head's key expansion); this fills the second.
 __global__ __launch_bounds__(64) void k_hb_latent_qrot(const float* q, long ldq, float* qa, long ldqa, const float* inv_freq, const int* pos, int dim,
-                                                       int R, int r, int rot) {
+                                                       int R, int r, int rot, float mag) {
     const int row = blockIdx.x, h = blockIdx.y;
-    const float* src = q + (size_t)row * ldq + (size_t)h * (dim + r) + dim;
-    float* dst = qa + (size_t)row * ldqa + (size_t)h * (R + r) + R;
     const float pf = (float)pos[row];
-    for (int d = threadIdx.x; d < r; d += 64) dst[d] = hb_rot_half(src, d, rot, pf, inv_freq);
+    for (int d = threadIdx.x; d < r; d += 64) hb_latent_qrot_head(q + (size_t)row * ldq, qa + (size_t)row * ldqa, inv_freq, pf, h, d, dim, R, r, rot, mag);
 }
 
 // per (row, head): o / rms(o) over vdim, times a weight (per_head_w: indexed over all heads, else shared [vdim]; NULL: none), times
@@ -2003,6 +2073,13 @@ __global__ __launch_bounds__(64) void k_hb_pool_update(const T* cache, float* po
     }
 }
 
+// A softmax sink: exp(value of the head) joins the denominator, a key without a value (v NULL: value 0 for every head).
+struct hb_sink {
+    int on;
+    const float* v;
+};
+__device__ __forceinline__ float hb_sink_of(const hb_sink& s, int h) { return s.v ? s.v[h] : 0.f; }
+
 // One block per (row, kv head).  Keys of a row at position p: the pooled blocks 0 .. nb-1 (nb = floor((p - window + 1) / P), those
 // wholly before the window) and then the tokens max(0, p-window+1) .. p.  The block has SPLIT waves per query head of the group; wave
 // (head, s) takes the 64-key chunks s, s + SPLIT, ... in ascending order: lane = key for the scores, lane = value column for the
@@ -2062,7 +2139,7 @@ template <typename T>
 __global__ __launch_bounds__(1024) __attribute__((amdgpu_waves_per_eu(1, 4))) void k_hb_attn(const float* proj, long ldp, const T* cache, const float* pool, float* out, long ldo, const int* pos,
                           const int* row_req, const int* ptab, int pts, int H, int G, int dim, int vdim, int window, int P, int ps, int ppp,
                           long v_base, float scale, int split, int seg_chunks, float* part, const float* gate, long ldg, float out_scale,
-                          int Gc, long v_ld, int sink) {
+                          int Gc, long v_ld, hb_sink sink) {
     extern __shared__ float sm[];
     const int QG = H / G, NWV = QG * split;
     const int dimp = (dim + 3) & ~3;
@@ -2281,15 +2358,17 @@ __global__ __launch_bounds__(1024) __attribute__((amdgpu_waves_per_eu(1, 4))) vo
     if (lane == 0) { mine[vdim] = m; mine[vdim + 1] = l; }
     __syncthreads();
     if (sp == 0) {
-        // sink: a key of score 0 without a value joins the softmax of the whole row (a segmented launch adds it in the merge)
-        float mm = sink && !part ? 0.f : -INFINITY;
+        // sink: a key without a value joins the softmax of the whole row (a segmented launch adds it in the merge)
+        const bool with_sink = sink.on && !part;
+        const float sk = with_sink ? hb_sink_of(sink, hq) : -INFINITY;
+        float mm = sk;
         for (int s2 = 0; s2 < split; ++s2) mm = fmaxf(mm, mo[(size_t)(s2 * QG + qh) * (vdim + 2) + vdim]);
         float lt = 0.f;
         for (int s2 = 0; s2 < split; ++s2) {
             const float* o2 = mo + (size_t)(s2 * QG + qh) * (vdim + 2);
             lt += o2[vdim + 1] * expf(o2[vdim] - mm);
         }
-        if (sink && !part) lt += expf(-mm);
+        if (with_sink) lt += expf(sk - mm);
         if (part) {
             float* dst = part + ((size_t)(row * H + hq) * gridDim.z + blockIdx.z) * (vdim + 2);
             for (int j = lane; j < vdim; j += 64) {
@@ -2318,7 +2397,7 @@ __global__ __launch_bounds__(1024) __attribute__((amdgpu_waves_per_eu(1, 4))) vo
 // few-row steps: the segments' partial results of a (row, head), merged in segment order; output gate applied here
 __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nseg_grid, float* out, long ldo, const int* pos, int H, int vdim,
                                                       int window, int P, int seg_chunks, const float* gate, long ldg, float out_scale, int chunk,
-                                                      int sink) {
+                                                      hb_sink sink) {
     const int row = blockIdx.x, hq = blockIdx.y, lane = threadIdx.x;
     const int p = pos[row];
     const int first = p - window + 1;
@@ -2326,7 +2405,8 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
     const int nseg = ((total + chunk - 1) / chunk + seg_chunks - 1) / seg_chunks;
     const float* src = part + (size_t)(row * H + hq) * nseg_grid * (vdim + 2);
     // lane s of each 64 segments fetches segment s's maximum and sum; the total is added in segment order
-    float mm = sink ? 0.f : -INFINITY;      // sink: a key of score 0 without a value
+    const float sk = sink.on ? hb_sink_of(sink, hq) : -INFINITY;      // sink: a key without a value
+    float mm = sk;
     for (int s0 = 0; s0 < nseg; s0 += 64) mm = fmaxf(mm, s0 + lane < nseg ? src[(size_t)(s0 + lane) * (vdim + 2) + vdim] : -INFINITY);
     mm = hb_wave_max(mm);
     const float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
@@ -2361,7 +2441,7 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
             }
         }
     }
-    if (sink) lt += expf(-mm);
+    if (sink.on) lt += expf(sk - mm);
 #pragma unroll
     for (int e = 0; e < HB_MAX_VPL; ++e) {
         const int j = lane + e * 64;
@@ -2386,7 +2466,7 @@ template <typename T>
 __global__ __launch_bounds__(hb_lat_tile<T>::NT) void k_hb_latent_attn_rows(const float* qa, long ldq, const T* cache, float* out, long ldo, const int* pos,
                                                              const int* row_req, const int* ptab, int pts, int H, int R, int r, int window,
                                                              int ps, float scale, int cpb, float* part, const float* gate, long ldg,
-                                                             float out_scale, int DP) {
+                                                             float out_scale, int DP, hb_sink sink) {
     constexpr int KT = hb_lat_tile<T>::KT, NT = hb_lat_tile<T>::NT, NS = NT / KT, HPT = HB_LAT_HG / NS, PVH = HB_LAT_HG / (NT / 256);
     extern __shared__ float sm[];
     const int D = R + r, Dq = (D + 3) & ~3;
@@ -2568,10 +2648,16 @@ __global__ __launch_bounds__(hb_lat_tile<T>::NT) void k_hb_latent_attn_rows(cons
                     if (two) dst[2 * ct + 1] = acc[h][1];
                     if (ct == 0) { dst[R] = ml[2 * (hb + h)]; dst[R + 1] = ml[2 * (hb + h) + 1]; }
                 } else {
-                    const float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
+                    float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
+                    float lt = ml[2 * (hb + h) + 1];
+                    if (sink.on) {
+                        const float mh = ml[2 * (hb + h)], sk = hb_sink_of(sink, hq), mm = fmaxf(mh, sk), f = expf(mh - mm);
+                        lt = lt * f + expf(sk - mm);
+                        gmul *= f;
+                    }
                     float* dst = out + (size_t)row * ldo + (size_t)hq * R;
-                    dst[2 * ct] = acc[h][0] / ml[2 * (hb + h) + 1] * gmul;
-                    if (two) dst[2 * ct + 1] = acc[h][1] / ml[2 * (hb + h) + 1] * gmul;
+                    dst[2 * ct] = acc[h][0] / lt * gmul;
+                    if (two) dst[2 * ct + 1] = acc[h][1] / lt * gmul;
                 }
             }
         }
@@ -2614,7 +2700,7 @@ __device__ __forceinline__ hb_f32x4 hb_mfma_bf16(uint4 a, uint4 b, hb_f32x4 c) {
 template <int KS, int CT>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void k_hb_latent_attn_mfma(
     const float* qa, long ldq, const bf16_t* cache, float* out, long ldo, const int* pos, const int* req_rows, int n_req, const int* ptab, int pts,
-    int H, int R, int r, int window, int ps, float scale, const float* gate, long ldg, float out_scale, int ks_n, int ct_n) {
+    int H, int R, int r, int window, int ps, float scale, const float* gate, long ldg, float out_scale, int ks_n, int ct_n, hb_sink sink) {
     extern __shared__ float sm[];
     const int D = R + r, DPK = ks_n * 32 + 8;
     long* tokoff = (long*)sm;                      // [64] where the tile's keys start in the cache
@@ -2766,7 +2852,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     }
     if (!active || col >= hg) return;
     const int hq = h0 + col;
-    const float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
+    float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
+    if (sink.on) {
+        const float sk = hb_sink_of(sink, hq), mm = fmaxf(m, sk), f = expf(m - mm);
+        l = l * f + expf(sk - mm);
+        gmul *= f;
+    }
     float* dst = out + (size_t)row * ldo + (size_t)hq * R;
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct)
@@ -2778,19 +2869,365 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
             }
 }
 
+// ---- attention with independent key weights --------------------------------------------------------------------------------------
+// z = (q . k) * scale * temp[h]; cap > 0: z <- cap * tanh(z / cap); z += dist[h][min(distance, dist_n - 1)]; weight = sigmoid(z + wb[h]).
+// Nothing is normalised over the keys, so partial sums over any split of the keys simply add.  chunk > 0: a position sees the positions
+// up to itself that share its p / chunk.
+struct hb_sig_score {
+    float scale, cap;
+    const float *temp, *dist, *wb;
+    int dist_n, chunk;
+};
+__device__ __forceinline__ int hb_chunk_start(int p, int chunk) { return chunk > 0 ? p / chunk * chunk : 0; }
+__device__ __forceinline__ float hb_sig_weight(const hb_sig_score& sc, int h, float dot, int dist) {
+    float z = dot * (sc.temp ? sc.scale * sc.temp[h] : sc.scale);
+    if (sc.cap > 0.f) z = sc.cap * tanhf(z / sc.cap);
+    if (sc.dist) z += sc.dist[(size_t)h * sc.dist_n + (dist < sc.dist_n ? dist : sc.dist_n - 1)];
+    if (sc.wb) z += sc.wb[h];
+    return hb_sigmoid(z);
+}
+// Steps of few rows (and every step of shapes or dtypes the matrix-core form does not take): block = (row, HPB query heads of one key
+// head, segment of cpb 64-key chunks); wave w takes the segment's chunks w, w + waves, ...: lane = key for the scores of the HPB heads,
+// then lane = value columns (two adjacent ones of each 128 with a bf16 cache and even sizes) for the weighted sums; the waves' sums are
+// added in wave order.  part != NULL: the segment's sums are left there for k_hb_sig_merge; else gate and scale are applied here.
+template <typename T, int HPB>
+__global__ __launch_bounds__(1024) void k_hb_sig_attn_rows(const float* q, long ldq, const T* cache, float* out, long ldo, const int* pos,
+                                                           const int* row_req, const int* ptab, int pts, int H, int G, int dim, int vdim, int ps,
+                                                           long v_base, hb_sig_score sc, int cpb, float* part, const float* gate, long ldg,
+                                                           float out_scale) {
+    extern __shared__ float sm[];
+    const int NW = blockDim.x >> 6, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    const int dimp = (dim + 3) & ~3;
+    long* loc = (long*)sm;                       // [NW][64] cache token of each lane's key
+    float* pw = sm + NW * 128;                   // [NW][64][HPB] weights
+    float* qs = pw + NW * 64 * HPB;              // [HPB][dimp]
+    float* red = qs + HPB * dimp;                // [NW][HPB * vdim]
+    const int row = blockIdx.x, h0 = blockIdx.y * HPB, g = h0 / (H / G), p = pos[row];
+    const int* pt = ptab + (size_t)row_req[row] * pts;
+    const int lo = hb_chunk_start(p, sc.chunk), total = p - lo + 1, nchunks = (total + 63) >> 6;
+    const int c0 = blockIdx.z * cpb, c1 = c0 + cpb < nchunks ? c0 + cpb : nchunks;
+    if (c0 >= nchunks) return;
+    for (int i = tid; i < HPB * dimp; i += blockDim.x) {
+        const int h = i / dimp, d = i - h * dimp;
+        qs[i] = d < dim ? q[(size_t)row * ldq + (size_t)(h0 + h) * dim + d] : 0.f;
+    }
+    __syncthreads();
+    constexpr int VE = 16 / sizeof(T);
+    const bool kvec = (dim % VE == 0) && ((((size_t)cache) & 15) == 0);
+    const bool pair = sizeof(T) == 2 && (vdim % 2 == 0) && (dim % 2 == 0);
+    const size_t kld = (size_t)G * dim, vld = (size_t)G * vdim;
+    float acc[HPB][HB_MAX_VPL];
+#pragma unroll
+    for (int h = 0; h < HPB; ++h)
+#pragma unroll
+        for (int e = 0; e < HB_MAX_VPL; ++e) acc[h][e] = 0.f;
+    long* wloc = loc + wv * 64;
+    float* wpw = pw + wv * 64 * HPB;
+    for (int c = c0 + wv; c < c1; c += NW) {
+        const int base = c * 64, cnt = total - base < 64 ? total - base : 64;
+        const int t = lo + base + (lane < cnt ? lane : cnt - 1);
+        const long tok = (long)pt[t / ps] * ps + t % ps;
+        __builtin_amdgcn_wave_barrier();
+        wloc[lane] = tok;
+        const T* kr = cache + (size_t)tok * kld + (size_t)g * dim;
+        float dot[HPB];
+#pragma unroll
+        for (int h = 0; h < HPB; ++h) dot[h] = 0.f;
+        if (kvec) {
+#pragma unroll 4
+            for (int d = 0; d < dim; d += VE) {
+                const uint4 u = *(const uint4*)(kr + d);
+                float k[VE];
+                if (sizeof(T) == 2) {
+                    k[0] = bflo(u.x); k[1] = bfhi(u.x); k[2] = bflo(u.y); k[3] = bfhi(u.y);
+                    if (VE == 8) { k[VE - 4] = bflo(u.z); k[VE - 3] = bfhi(u.z); k[VE - 2] = bflo(u.w); k[VE - 1] = bfhi(u.w); }
+                } else {
+                    k[0] = __uint_as_float(u.x); k[1] = __uint_as_float(u.y); k[2] = __uint_as_float(u.z); k[3] = __uint_as_float(u.w);
+                }
+#pragma unroll
+                for (int h = 0; h < HPB; ++h)
+#pragma unroll
+                    for (int e = 0; e < VE; ++e) dot[h] = fmaf(qs[h * dimp + d + e], k[e], dot[h]);
+            }
+        } else {
+            for (int d = 0; d < dim; ++d) {
+                const float k = hb_ld(kr + d);
+#pragma unroll
+                for (int h = 0; h < HPB; ++h) dot[h] = fmaf(qs[h * dimp + d], k, dot[h]);
+            }
+        }
+#pragma unroll
+        for (int h = 0; h < HPB; ++h) wpw[lane * HPB + h] = lane < cnt ? hb_sig_weight(sc, h0 + h, dot[h], p - t) : 0.f;
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        if (pair) {
+#pragma unroll
+            for (int cc = 0; cc < HB_MAX_VPL / 2; ++cc) {
+                if (cc * 128 < vdim) {
+                    const int j = cc * 128 + 2 * lane, jj = j < vdim ? j : vdim - 2;
+                    const T* vb = cache + v_base + (size_t)g * vdim + jj;
+                    for (int k0 = 0; k0 < cnt; k0 += 16) {
+                        u32 vv[16];
+#pragma unroll
+                        for (int x = 0; x < 16; ++x) vv[x] = *(const u32*)(vb + (size_t)wloc[k0 + x < cnt ? k0 + x : cnt - 1] * vld);
+#pragma unroll
+                        for (int x = 0; x < 16; ++x)
+#pragma unroll
+                            for (int h = 0; h < HPB; ++h) {
+                                const float w = wpw[(k0 + x) * HPB + h];        // (zero behind the last key)
+                                acc[h][2 * cc] = fmaf(w, bflo(vv[x]), acc[h][2 * cc]);
+                                acc[h][2 * cc + 1] = fmaf(w, bfhi(vv[x]), acc[h][2 * cc + 1]);
+                            }
+                    }
+                }
+            }
+        } else {
+#pragma unroll
+            for (int cc = 0; cc < HB_MAX_VPL; ++cc) {
+                if (cc * 64 < vdim) {
+                    const int j = cc * 64 + lane, jj = j < vdim ? j : vdim - 1;
+                    const T* vb = cache + v_base + (size_t)g * vdim + jj;
+                    for (int k0 = 0; k0 < cnt; k0 += 8) {
+                        float vv[8];
+#pragma unroll
+                        for (int x = 0; x < 8; ++x) vv[x] = hb_ld(vb + (size_t)wloc[k0 + x < cnt ? k0 + x : cnt - 1] * vld);
+#pragma unroll
+                        for (int x = 0; x < 8; ++x)
+#pragma unroll
+                            for (int h = 0; h < HPB; ++h) acc[h][cc] = fmaf(wpw[(k0 + x) * HPB + h], vv[x], acc[h][cc]);
+                    }
+                }
+            }
+        }
+        __builtin_amdgcn_wave_barrier();
+    }
+    float* mine = red + (size_t)wv * HPB * vdim;
+#pragma unroll
+    for (int h = 0; h < HPB; ++h)
+#pragma unroll
+        for (int e = 0; e < HB_MAX_VPL; ++e) {
+            const int j = pair ? (e >> 1) * 128 + 2 * lane + (e & 1) : lane + e * 64;
+            if (j < vdim) mine[h * vdim + j] = acc[h][e];
+        }
+    __syncthreads();
+    for (int i = tid; i < HPB * vdim; i += blockDim.x) {
+        float a = 0.f;
+        for (int w = 0; w < NW; ++w) a += red[(size_t)w * HPB * vdim + i];
+        const int h = h0 + i / vdim, j = i % vdim;
+        if (part) { part[((size_t)(row * H + h) * gridDim.z + blockIdx.z) * vdim + j] = a; continue; }
+        a *= out_scale;
+        if (gate) a *= hb_sigmoid(gate[(size_t)row * ldg + h * vdim + j]);
+        out[(size_t)row * ldo + (size_t)h * vdim + j] = a;
+    }
+}
+// the segments' sums of a (row, head), added in segment order; gate and scale
+__global__ __launch_bounds__(64) void k_hb_sig_merge(const float* part, int nseg_grid, float* out, long ldo, const int* pos, int H, int vdim, int chunk,
+                                                     int cpb, const float* gate, long ldg, float out_scale) {
+    const int row = blockIdx.x, h = blockIdx.y, p = pos[row];
+    const int nchunks = (p - hb_chunk_start(p, chunk) + 64) >> 6, nseg = (nchunks + cpb - 1) / cpb;
+    const float* src = part + (size_t)(row * H + h) * nseg_grid * vdim;
+    for (int j = threadIdx.x; j < vdim; j += 64) {
+        float a = 0.f;
+        for (int s = 0; s < nseg; ++s) a += src[(size_t)s * vdim + j];
+        a *= out_scale;
+        if (gate) a *= hb_sigmoid(gate[(size_t)row * ldg + h * vdim + j]);
+        out[(size_t)row * ldo + (size_t)h * vdim + j] = a;
+    }
+}
+// Steps of many rows, bf16 cache: block = 64 consecutive rows of one request (16 per wave) and one head; tiles of 64 keys in LDS, keys as
+// cached (Kt[key][dim]), values transposed two keys at a time (Vt[column][key]); the next tile's requests are on their way while a tile is
+// multiplied.  Per tile and wave, rows being the 16 columns of both products:
+//   S^T[key][row] = sum_dim Kt[key][dim] Q[row][dim]     v_mfma_f32_16x16x32_bf16, the query in registers as two bf16 parts (hi + lo)
+//   weights of the lane's 16 (key, row) pairs, fp32; masked pairs 0
+//   O^T[col][row] += sum_key Vt[col][key] P[row][key]    the weights as they sit in the lanes (k index laid out to match), hi + lo
+// Row tiles of the launch are found by walking the requests' row counts; blocks beyond the last tile leave.  KS 32-dim steps of the key
+// and CT 16-column tiles of the value at most.
+#define HB_SIG_VLD 76        // keys per row of the transposed value tile (64 + 12: rows 8 bytes aligned, eight rows 16 banks apart)
+#define HB_SIG_DIST_LDS 4096 // distance biases per head that are kept in LDS
+// tanh and the logistic function from the hardware's exponential and reciprocal: absolute error of a few 1e-7
+__device__ __forceinline__ float hb_fast_tanh(float x) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(__expf(2.0f * x) + 1.0f); }
+__device__ __forceinline__ float hb_fast_sigmoid(float x) { return __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
+template <int KS, int CT>
+__global__ __launch_bounds__(256) void k_hb_sig_attn_mfma(const float* q, long ldq, const bf16_t* cache, float* out, long ldo, const int* pos,
+                                                          const int* req_rows, int n_req, const int* ptab, int pts, int H, int G, int dim, int vdim,
+                                                          int ps, long v_base, hb_sig_score sc, const float* gate, long ldg, float out_scale,
+                                                          int ks_n, int ct_n) {
+    extern __shared__ float sm[];
+    const int DPK = ks_n * 32 + 8;
+    const int nbias = sc.dist && sc.dist_n <= HB_SIG_DIST_LDS ? sc.dist_n : 0;
+    bf16_t* Kt = (bf16_t*)sm;                            // [64][DPK]
+    bf16_t* Vt = Kt + 64 * DPK;                          // [ct_n * 16][HB_SIG_VLD]
+    float* sbias = (float*)(Vt + ct_n * 16 * HB_SIG_VLD);   // [nbias]
+    const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, col = lane & 15, g4 = lane >> 4;
+    int t = blockIdx.x, rq = -1, rs = 0, re = 0;
+    for (int r = 0; r < n_req; ++r) {
+        const int a = req_rows[r], b = req_rows[r + 1], nt = (b - a + 63) >> 6;
+        if (t < nt) { rq = r; rs = a + 64 * t; re = b; break; }
+        t -= nt;
+    }
+    if (rq < 0) return;
+    const int h = blockIdx.y, g = h / (H / G);
+    const int nrows = re - rs < 64 ? re - rs : 64;
+    const int w0 = wv * 16, wn = nrows - w0 < 16 ? nrows - w0 : 16;      // the wave's rows: w0 .. w0 + wn - 1 of the tile (wn may be <= 0)
+    const bool active = wn > 0;
+    const bool rowok = col < wn;
+    const int row = rs + (rowok ? w0 + col : 0);
+    const int p = pos[row], lo_r = hb_chunk_start(p, sc.chunk);
+    const int p0 = pos[rs], pl = pos[rs + nrows - 1];
+    const int wp_lo = active ? hb_chunk_start(pos[rs + w0], sc.chunk) : 0, wp_hi = active ? pos[rs + w0 + wn - 1] : -1;
+    const int lo_t = hb_chunk_start(p0, sc.chunk), ntiles = (pl - lo_t + 64) >> 6;
+    const int* pt = ptab + (size_t)rq * pts;
+    const float zmul = sc.temp ? sc.scale * sc.temp[h] : sc.scale, wbias = sc.wb ? sc.wb[h] : 0.f;
+    const float icap = sc.cap > 0.f ? 1.0f / sc.cap : 0.f;
+    for (int i = tid; i < nbias; i += 256) sbias[i] = sc.dist[(size_t)h * sc.dist_n + i];
+    uint4 qh[KS], ql[KS];
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+        float v[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = 0.f;
+        const int d0 = ks * 32 + g4 * 8;
+        if (ks < ks_n && rowok && d0 < dim) {
+            const float* src = q + (size_t)row * ldq + (size_t)h * dim + d0;
+            const float4 a = *(const float4*)src, b = *(const float4*)(src + 4);
+            v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+        }
+        hb_split_bf16x8(v, qh[ks], ql[ks]);
+    }
+    hb_f32x4 oacc[CT];
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) oacc[ct] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
+    // staging: keys -- four threads per key, pieces of 8 dims (tid & 3) + 4k; values -- eight threads per pair of keys, pieces of 8
+    // columns (tid & 7) + 8k of both keys
+    constexpr int NV = (CT * 2 + 7) / 8;
+    uint4 rk[KS], rv0[NV], rv1[NV];
+    const int kj = tid >> 2, kpiece = tid & 3, vj = (tid >> 3) * 2, vpiece = tid & 7, dpie = dim >> 3, vpie = vdim >> 3;
+    auto fetch = [&](int base) {
+        const int cnt = pl - base + 1 < 64 ? pl - base + 1 : 64;
+        const bool kok = kj < cnt;
+        const int tk = base + (kok ? kj : 0);
+        const bf16_t* kp = cache + ((size_t)pt[tk / ps] * ps + tk % ps) * (size_t)(G * dim) + (size_t)g * dim;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) {
+            const int v = kpiece + 4 * k;
+            rk[k] = kok && v < dpie ? *(const uint4*)(kp + v * 8) : make_uint4(0, 0, 0, 0);
+        }
+        const bool ok0 = vj < cnt, ok1 = vj + 1 < cnt;
+        const int t0 = base + (ok0 ? vj : 0), t1 = base + (ok1 ? vj + 1 : 0);
+        const bf16_t* vb = cache + v_base + (size_t)g * vdim;
+        const bf16_t* v0 = vb + ((size_t)pt[t0 / ps] * ps + t0 % ps) * (size_t)(G * vdim);
+        const bf16_t* v1 = vb + ((size_t)pt[t1 / ps] * ps + t1 % ps) * (size_t)(G * vdim);
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int v = vpiece + 8 * k;
+            rv0[k] = ok0 && v < vpie ? *(const uint4*)(v0 + v * 8) : make_uint4(0, 0, 0, 0);
+            rv1[k] = ok1 && v < vpie ? *(const uint4*)(v1 + v * 8) : make_uint4(0, 0, 0, 0);
+        }
+    };
+    fetch(lo_t);
+    for (int c = 0; c < ntiles; ++c) {
+        const int base = lo_t + c * 64;
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < KS; ++k)
+            if (k < ks_n) *(uint4*)(Kt + kj * DPK + (kpiece + 4 * k) * 8) = rk[k];
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int cc = (vpiece + 8 * k) * 8;
+            if (cc < ct_n * 16) {
+                const u32 a[4] = {rv0[k].x, rv0[k].y, rv0[k].z, rv0[k].w}, b[4] = {rv1[k].x, rv1[k].y, rv1[k].z, rv1[k].w};
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    u32* d0 = (u32*)(Vt + (size_t)(cc + 2 * i) * HB_SIG_VLD + vj);
+                    *d0 = (a[i] & 0xffffu) | (b[i] << 16);
+                    u32* d1 = (u32*)(Vt + (size_t)(cc + 2 * i + 1) * HB_SIG_VLD + vj);
+                    *d1 = (a[i] >> 16) | (b[i] & 0xffff0000u);
+                }
+            }
+        }
+        __syncthreads();
+        if (c + 1 < ntiles) fetch(base + 64);
+        if (!active || base > wp_hi || base + 63 < wp_lo) continue;        // (a wave whose rows see no key of the tile)
+        hb_f32x4 st[4];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) st[kt] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            if (ks < ks_n) {
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt) {
+                    const uint4 a = *(const uint4*)(Kt + (size_t)(kt * 16 + col) * DPK + ks * 32 + g4 * 8);
+                    st[kt] = hb_mfma_bf16(a, qh[ks], st[kt]);
+                    st[kt] = hb_mfma_bf16(a, ql[ks], st[kt]);
+                }
+            }
+        }
+        // lane (col, g4) holds the scores of row `col` against keys base + kt*16 + g4*4 + i
+        float pr[4][4];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int key = base + kt * 16 + g4 * 4 + i;
+                float z = st[kt][i] * zmul;
+                if (icap > 0.f) z = sc.cap * hb_fast_tanh(z * icap);
+                if (sc.dist) {
+                    int d = p - key;
+                    d = d < 0 ? 0 : (d < sc.dist_n ? d : sc.dist_n - 1);
+                    z += nbias ? sbias[d] : sc.dist[(size_t)h * sc.dist_n + d];
+                }
+                pr[kt][i] = key >= lo_r && key <= p ? hb_fast_sigmoid(z + wbias) : 0.f;
+            }
+        uint4 ph[2], plo[2];
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            const float v[8] = {pr[2 * kk][0], pr[2 * kk][1], pr[2 * kk][2], pr[2 * kk][3], pr[2 * kk + 1][0], pr[2 * kk + 1][1], pr[2 * kk + 1][2],
+                                pr[2 * kk + 1][3]};
+            hb_split_bf16x8(v, ph[kk], plo[kk]);
+        }
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) {
+            if (ct < ct_n) {
+#pragma unroll
+                for (int kk = 0; kk < 2; ++kk) {
+                    const bf16_t* vr = Vt + (size_t)(ct * 16 + col) * HB_SIG_VLD + kk * 32 + g4 * 4;
+                    const uint2 a0 = *(const uint2*)vr, a1 = *(const uint2*)(vr + 16);
+                    const uint4 a = make_uint4(a0.x, a0.y, a1.x, a1.y);
+                    oacc[ct] = hb_mfma_bf16(a, ph[kk], oacc[ct]);
+                    oacc[ct] = hb_mfma_bf16(a, plo[kk], oacc[ct]);
+                }
+            }
+        }
+    }
+    if (!rowok) return;
+    float* dst = out + (size_t)row * ldo + (size_t)h * vdim;
+    const float* gr = gate ? gate + (size_t)row * ldg + (size_t)h * vdim : nullptr;
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct)
+        if (ct < ct_n)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int cc = ct * 16 + g4 * 4 + i;
+                if (cc < vdim) dst[cc] = oacc[ct][i] * out_scale * (gr ? hb_sigmoid(gr[cc]) : 1.0f);
+            }
+}
+
 // ---- routed feed-forward --------------------------------------------------------------------------------------------------
 // One block per row: router logits z_j = router[j] . h in fp32 (lane-strided sums over four waves and a butterfly: an order fixed by
 // the width, the same for every step shape), then one wave: s = softmax(z) over all nE router outputs, choice = s + correction, the `top` largest choices (first
 // index wins a tie) in descending order; weights = their s / (sum + 1e-20).  sel[row*top + k] = router output index, wgt likewise.
 // sigmoid != 0: s_j = sigmoid(z_j) instead of the softmax; renorm == 0: the weights are the chosen s as they are.
-// bias != NULL: added to the logits before the scores are formed.
+// bias != NULL: added to the logits before the scores are formed.  groups > 1: only experts of the `keep` best groups can be chosen.
+// wscale multiplies the weights.
 __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh, const float* router, const float* corr, int W, int nE, int top,
-                                                       int* sel, float* wgt, int sigmoid, int renorm, const float* bias) {
+                                                       int* sel, float* wgt, int sigmoid, int renorm, const float* bias, int groups, int keep,
+                                                       float wscale) {
     extern __shared__ float sm[];
     float* sc = sm;                    // [nE] logits, then scores
     float* ch = sm + nE;               // [nE] choice values
     int* pick = (int*)(sm + 2 * nE);   // [top]
     float* part = sm + 2 * nE + top;   // [4][nE] the waves' partial logits
+    float* gs = part + 4 * nE;         // [groups] group scores (groups > 1)
     const int row = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const float* x = h + (size_t)row * ldh;
     const bool vec = (W % 4 == 0) && (ldh % 4 == 0) && ((((size_t)h) & 15) == 0) && ((((size_t)router) & 15) == 0);
@@ -2872,6 +3309,27 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
     __builtin_amdgcn_wave_barrier();
+    if (groups > 1 && keep < groups) {
+        // groups of neighbours: a group's score is its largest choice value; `keep` groups stay (the first of equal ones), the experts of
+        // the others cannot be chosen
+        const int per = nE / groups;
+        for (int g = lane; g < groups; g += 64) {
+            float best = -INFINITY;
+            for (int i = 0; i < per; ++i) best = fmaxf(best, ch[g * per + i]);
+            gs[g] = best;
+        }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+        for (int i = lane; i < nE; i += 64) {
+            const int g = i / per;
+            const float mine = gs[g];
+            int ahead = 0;
+            for (int o = 0; o < groups; ++o) ahead += gs[o] > mine || (gs[o] == mine && o < g) ? 1 : 0;
+            if (ahead >= keep) ch[i] = -INFINITY;
+        }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+    }
     // one wave from here on: every lane follows the same picks; lane 0 retires a pick in LDS before the next search reads it
     float wsum = 0.f;
     for (int k = 0; k < top; ++k) {
@@ -2899,7 +3357,7 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
     const float den = wsum + 1e-20f;
     for (int k = lane; k < top; k += 64) {
         sel[(size_t)row * top + k] = pick[k];
-        wgt[(size_t)row * top + k] = renorm ? sc[pick[k]] / den : sc[pick[k]];
+        wgt[(size_t)row * top + k] = (renorm ? sc[pick[k]] / den : sc[pick[k]]) * wscale;
     }
 }
 // Block e lists the entries (row*top + k) routed to expert e, ascending: list[e*cap + 0 .. count[e]).
@@ -2959,15 +3417,28 @@ struct hb_moe_small {
     const float* shared_bias;   // [2 * shared_ff] gate, then up biases of the shared unit, or NULL
     int shared_gelu;            // the shared unit's activation is the tanh form of gelu
     int up_down, relu2;         // units are down(act(up h)): the matrices hold up rows only; act = the square of relu (else swish)
-    const float* out_scale;     // [W] layer scale of what joins the residual sum, or NULL
+    hb_join join;               // how the result joins the residual stream
+    const void* w_res;          // [W, W] rows of the residual gate, one more entry per row of the first launch, or NULL
+    const float* b_res;
+    float* res;                 // [rows][W] its logits
 };
 // gate / up products + activation of every entry: block (column tile, entry); a wave takes gate row n and up row ff + n of the
 // entry's expert and stores g * sigmoid(alpha g) * (u + 1) with the clamps of that expert.  act row of an entry: ld_act floats.
 template <typename T>
 __global__ __launch_bounds__(256) void k_hb_moe_gate_up(const float* h, long ldh, const T* w_gate_up, const T* shared_gate_up, float* act, int W,
                                                         hb_moe_small q) {
-    const int per = q.top + (q.shared_ff > 0 ? 1 : 0);
-    const int entry = blockIdx.y, row = entry / per, slot = entry - row * per, lane = threadIdx.x & 63, n = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int per = q.top + (q.shared_ff > 0 ? 1 : 0), per_y = per + (q.w_res ? 1 : 0);
+    const int row = blockIdx.y / per_y, slot = blockIdx.y - row * per_y, entry = row * per + slot, lane = threadIdx.x & 63, n = blockIdx.x * 4 + (threadIdx.x >> 6);
+    constexpr int CH = sizeof(T) == 2 ? 8 : 4;
+    const float* x = h + (size_t)row * ldh;
+    if (slot == per) {
+        if (n >= W) return;
+        const T* wr = (const T*)q.w_res;
+        const bool rvec = (W % CH == 0) && ((((size_t)wr) & 15) == 0) && (ldh % 4 == 0) && ((((size_t)h) & 15) == 0);
+        const float z = hb_dot_wave<T>(wr + (size_t)n * W, x, W, rvec, lane);
+        if (lane == 0) q.res[(size_t)row * W + n] = z + (q.b_res ? q.b_res[n] : 0.f);
+        return;
+    }
     const T* wg;
     int N;
     float limit, xs = 1.0f;
@@ -2988,8 +3459,6 @@ __global__ __launch_bounds__(256) void k_hb_moe_gate_up(const float* h, long ldh
         gelu = q.shared_gelu;
     }
     if (n >= N) return;
-    constexpr int CH = sizeof(T) == 2 ? 8 : 4;
-    const float* x = h + (size_t)row * ldh;
     const bool vec = (W % CH == 0) && ((((size_t)wg) & 15) == 0) && (ldh % 4 == 0) && ((((size_t)h) & 15) == 0);
     if (q.up_down) {
         const float u1 = hb_dot_wave<T>(wg + (size_t)n * W, x, W, vec, lane, xs);
@@ -3023,12 +3492,12 @@ __global__ __launch_bounds__(256) void k_hb_moe_down_combine(const float* h, lon
         const bool vec = avec && (q.shared_ff % CH == 0) && ((((size_t)shared_down) & 15) == 0);
         acc += hb_dot_wave<T>(shared_down + (size_t)c * q.shared_ff, act + (size_t)(row * per + q.top) * q.ld_act, q.shared_ff, vec, lane);
     }
-    if (lane == 0) x[(size_t)row * ldx + c] += q.out_scale ? acc * q.out_scale[c] : acc;
+    if (lane == 0) hb_join_add(q.join, x + (size_t)row * ldx, row, c, acc);
 }
 // x[row] += sum_k wgt[row*top + k] * (identity output ? h[row] : expert_out[row*top + k]), k ascending
 // (scale_input: an expert's output enters with weight 1, its input was scaled instead)
 __global__ __launch_bounds__(256) void k_hb_moe_combine(float* x, long ldx, const float* h, long ldh, const float* eo, const int* sel,
-                                                        const float* wgt, int top, int experts, int W, int scale_input, const float* out_scale) {
+                                                        const float* wgt, int top, int experts, int W, int scale_input, hb_join join) {
     const int row = blockIdx.x;
     for (int i = threadIdx.x; i < W; i += 256) {
         float acc = 0.f;
@@ -3037,13 +3506,22 @@ __global__ __launch_bounds__(256) void k_hb_moe_combine(float* x, long ldx, cons
             const bool ident = sel[en] >= experts;
             acc = fmaf(scale_input && !ident ? 1.0f : wgt[en], ident ? h[(size_t)row * ldh + i] : eo[en * W + i], acc);
         }
-        x[(size_t)row * ldx + i] += out_scale ? acc * out_scale[i] : acc;
+        hb_join_add(join, x + (size_t)row * ldx, row, i, acc);
     }
 }
 
 __global__ void k_hb_copy_rows(const float* src, long lds_, float* dst, long ldd, int W) {
     const int row = blockIdx.x;
     for (int i = threadIdx.x; i < W; i += blockDim.x) dst[(size_t)row * ldd + i] = src[(size_t)row * lds_ + i];
+}
+// dst[row] = the sum of the row's streams
+__global__ void k_hb_sum_streams(const float* src, int streams, float* dst, long ldd, int W) {
+    const int row = blockIdx.x;
+    for (int i = threadIdx.x; i < W; i += blockDim.x) {
+        float v = 0.f;
+        for (int s = 0; s < streams; ++s) v += src[((size_t)row * streams + s) * W + i];
+        dst[(size_t)row * ldd + i] = v;
+    }
 }
 __global__ void k_hb_logits_bf16(const float* src, bf16_t* dst, long n) {
     const long i = (long)blockIdx.x * 256 + threadIdx.x;
@@ -3098,6 +3576,8 @@ struct vox_hybrid {
     std::vector<vox_hybrid_run> runs;
     vox_hybrid_weights w;
     float *xa = nullptr, *xb = nullptr, *h = nullptr, *h2 = nullptr, *proj = nullptr, *mix = nullptr, *ff = nullptr, *hout = nullptr;
+    float *u = nullptr, *ones = nullptr;    // [max_rows][width]: what the next sublayer reads of several residual streams; [HB_MAX_STREAMS]
+    float *rgate = nullptr;                 // [max_rows][width]: residual gate logits of a routed feed-forward
     float *ff_act = nullptr;                // [max_rows][max gated dense width]: activation output of the gated dense feed-forward
     int max_gated = 0;
     float *shift = nullptr;                 // [5][max_rows][width]: token-shift mixes
@@ -3110,24 +3590,28 @@ struct vox_hybrid {
     size_t attn_ws_bytes = 0;
     int max_in = 0, max_mix = 0, max_ff = 0;
     int max_ne = 0, max_top = 0, max_eff = 0, max_experts = 0;
-    bool any_shift = false;
+    bool any_shift = false, any_rgate = false;
     bool attn_big_lds = false;              // the attention kernel was given the right to more than 64 KB of LDS
     bool lat_big_lds = false;               // the same for the few-row latent attention
 };
 
-static bool hb_is_attn(int kind) { return kind == VOX_MIXER_POOLED_WINDOW_ATTN || kind == VOX_MIXER_CAUSAL_ATTN || kind == VOX_MIXER_LATENT_ATTN; }
+static bool hb_is_attn(int kind) { return kind == VOX_MIXER_POOLED_WINDOW_ATTN || kind == VOX_MIXER_CAUSAL_ATTN || kind == VOX_MIXER_LATENT_ATTN || kind == VOX_MIXER_SIGMOID_ATTN; }
 static inline int hb_up4(int v) { return (v + 3) & ~3; }
 // Where a latent-attention row keeps what it derives from the fused projection [query latent | kv latent | rotated key | gate]:
+// (without a query latent: [q | kv latent | rotated key | gate], the query at column 0), then the residual gate's columns.
 // q = per head [plain | rotated] at off_q, the query against the cached rows (per head [R | r]) at off_qa, the weighted sum of cached
 // latents per head at off_o.  Every part starts on a 16-byte boundary.
 struct hb_latent_layout {
-    int n_in, off_q, off_qa, off_o, n_proj;
+    int n_in, off_kv, off_gate, off_q, off_qa, off_o, n_proj;
 };
 static hb_latent_layout hb_latent(const vox_hybrid_layer& L) {
     hb_latent_layout y;
-    y.n_in = L.q_rank + L.kv_rank + L.rot_dim + L.heads;
-    y.off_q = hb_up4(y.n_in);
-    y.off_qa = y.off_q + hb_up4(L.heads * (L.dim + L.rot_dim));
+    const int dq = L.heads * (L.dim + L.rot_dim);
+    y.off_kv = L.q_rank > 0 ? L.q_rank : dq;
+    y.off_gate = y.off_kv + L.kv_rank + L.rot_dim;
+    y.n_in = y.off_gate + (L.no_head_gate ? 0 : L.heads) + L.res_gate;
+    y.off_q = L.q_rank > 0 ? hb_up4(y.n_in) : 0;
+    y.off_qa = L.q_rank > 0 ? y.off_q + hb_up4(dq) : hb_up4(y.n_in);
     y.off_o = y.off_qa + hb_up4(L.heads * (L.kv_rank + L.rot_dim));
     y.n_proj = y.off_o + hb_up4(L.heads * L.kv_rank);
     return y;
@@ -3149,7 +3633,7 @@ static hb_delta_layout hb_delta(const vox_hybrid_layer& L) {
     y.off_din = y.off_b + L.heads;
     y.ndec = L.decay_channels ? L.heads * L.dim : L.heads;
     y.off_gin = y.off_din + (L.lora > 0 ? L.lora : y.ndec);
-    y.n_in = y.off_gin + (L.gate_rank > 0 ? L.gate_rank : nv);
+    y.n_in = y.off_gin + (L.gate_rank > 0 ? L.gate_rank : nv) + L.res_gate;
     int next = hb_up4(y.n_in);
     y.off_dec = y.off_din;
     if (L.lora > 0) { y.off_dec = next; next += hb_up4(y.ndec); }
@@ -3171,24 +3655,26 @@ struct hb_conv_attn_layout {
 static hb_conv_attn_layout hb_conv_attn_cols(const vox_hybrid_layer& L) {
     const int C = L.heads * L.dim + L.kv_heads * (L.dim + L.vdim);
     hb_conv_attn_layout y;
-    y.off_y = hb_up4(C);
+    y.off_y = hb_up4(C + L.res_gate);
     y.off_qc = y.off_y + hb_up4(C);
     y.off_ss = y.off_qc + hb_up4(L.heads * L.dim);
     y.n_proj = y.off_ss + hb_up4(2 * ((C + 255) / 256));
     return y;
 }
-// rows of the fused input projection
+// rows of the fused input projection, the residual gate's (the last ones) included
 static int hb_layer_in(const vox_hybrid_layer& L) {
+    const int rg = L.res_gate;
     switch (L.kind) {
-        case VOX_MIXER_HGRN2: return 2 * L.heads * L.dim + L.heads * L.vdim;
-        case VOX_MIXER_POOLED_WINDOW_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim) + L.heads;
-        case VOX_MIXER_MLSTM: return 2 * L.heads * L.dim + 2 * L.heads * L.vdim + 2 * L.heads;
+        case VOX_MIXER_HGRN2: return 2 * L.heads * L.dim + L.heads * L.vdim + rg;
+        case VOX_MIXER_POOLED_WINDOW_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim) + L.heads + rg;
+        case VOX_MIXER_MLSTM: return 2 * L.heads * L.dim + 2 * L.heads * L.vdim + 2 * L.heads + rg;
         case VOX_MIXER_RGLRU: return 2 * L.heads * L.dim;
-        case VOX_MIXER_CAUSAL_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim);
+        case VOX_MIXER_CAUSAL_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim) + rg;
         case VOX_MIXER_SHIFT_DECAY: return 4 * L.heads * L.dim + L.lora;
-        case VOX_MIXER_LATENT_ATTN: return L.q_rank + L.kv_rank + L.rot_dim + L.heads;
-        case VOX_MIXER_RETENTION: return 2 * L.heads * L.dim + 2 * L.heads * L.vdim;
+        case VOX_MIXER_LATENT_ATTN: return hb_latent(L).n_in;
+        case VOX_MIXER_RETENTION: return 2 * L.heads * L.dim + 2 * L.heads * L.vdim + rg;
         case VOX_MIXER_DELTA: return L.kv_heads > 0 ? hb_delta(L).n_in : -1;
+        case VOX_MIXER_SIGMOID_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim) + (L.out_gate ? L.heads * L.vdim : 0) + rg;
     }
     return -1;
 }
@@ -3199,6 +3685,7 @@ static int hb_layer_proj(const vox_hybrid_layer& L) {
     if (L.kind == VOX_MIXER_LATENT_ATTN) return hb_latent(L).n_proj;
     if (L.kind == VOX_MIXER_DELTA) return hb_delta(L).n_proj;
     if (hb_conv_attn(L)) return hb_conv_attn_cols(L).n_proj;
+    if (L.kind == VOX_MIXER_SIGMOID_ATTN) return hb_up4(hb_layer_in(L));
     return hb_layer_in(L);
 }
 
@@ -3236,7 +3723,8 @@ static bool hb_try_latent_mfma(vox_hybrid* m, hipStream_t st, const vox_hybrid_i
     do { \
         if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_latent_attn_mfma<KS_, CT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
         hipLaunchKernelGGL((k_hb_latent_attn_mfma<KS_, CT_>), grid, block, lds, st, qa, ldp, cache, o, ldp, io->pos, io->req_rows, n_req, io->page_table, \
-                           io->pt_stride, L.heads, R, r, window, ps, L.scale, gate, ldp, L.out_scale, ks_n, ct_n); \
+                           io->pt_stride, L.heads, R, r, window, ps, L.scale, gate, ldp, L.out_scale, ks_n, ct_n, \
+                           hb_sink{L.sinks ? 1 : 0, L.sinks}); \
     } while (0)
     if (ks_n <= 10 && ct_n <= 16) HB_LM(10, 16);
     else if (ct_n <= 16) HB_LM(18, 16);
@@ -3248,24 +3736,92 @@ static bool hb_try_latent_mfma(vox_hybrid* m, hipStream_t st, const vox_hybrid_i
 static bool hb_try_latent_mfma(vox_hybrid*, hipStream_t, const vox_hybrid_io*, const vox_hybrid_layer&, const float*, const float*, float*, long,
                                const float*, int, int, int, int) { return false; }
 
-// cur += (A . W^T + bias) [* scale column by column]
+// The matrix-core sigmoid attention for steps of many rows over a bf16 cache.  false: the sizes do not fit it (head dims that are no
+// multiple of 8, or above 256).
+static bool hb_try_sig_mfma(hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const bf16_t* cache, const float* q, long ldp,
+                            float* out, long ldo, const hb_sig_score& sc, const float* gate, long v_base, int n, int n_req, int ps) {
+    if ((L.dim & 7) || (L.vdim & 7) || L.dim > 256 || L.vdim > 256 || (ldp & 3) || ((size_t)q & 15) || ((size_t)cache & 15)) return false;
+    const int ks_n = (L.dim + 31) / 32, ct_n = (L.vdim + 15) / 16;
+    const int nbias = sc.dist && sc.dist_n <= HB_SIG_DIST_LDS ? sc.dist_n : 0;
+    const size_t lds = (size_t)64 * (ks_n * 32 + 8) * 2 + (size_t)ct_n * 16 * HB_SIG_VLD * 2 + (size_t)nbias * 4;
+    const dim3 grid((n + 63) / 64 + n_req, L.heads), block(256);
+#define HB_SM(KS_, CT_) \
+    do { \
+        if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_sig_attn_mfma<KS_, CT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        hipLaunchKernelGGL((k_hb_sig_attn_mfma<KS_, CT_>), grid, block, lds, st, q, ldp, cache, out, ldo, io->pos, io->req_rows, n_req, io->page_table, \
+                           io->pt_stride, L.heads, L.kv_heads, L.dim, L.vdim, ps, v_base, sc, gate, ldp, L.out_scale, ks_n, ct_n); \
+    } while (0)
+    if (ks_n <= 4 && ct_n <= 8) HB_SM(4, 8);
+    else HB_SM(8, 16);
+#undef HB_SM
+    return true;
+}
+static bool hb_try_sig_mfma(hipStream_t, const vox_hybrid_io*, const vox_hybrid_layer&, const float*, const float*, long, float*, long,
+                            const hb_sig_score&, const float*, long, int, int, int) { return false; }
+// query heads of one key head that share a block of the few-row sigmoid attention
+static int hb_sig_heads(const vox_hybrid_layer& L) {
+    const int qg = L.heads / L.kv_heads;
+    for (int h = 4; h > 1; --h)
+        if (qg % h == 0) return h;
+    return 1;
+}
+#define HB_SIG_SEG 16     // 64-key chunks per block of the few-row sigmoid attention (one per wave)
+static size_t hb_sig_lds(const vox_hybrid_layer& L, int hpb, int nw) {
+    return (size_t)(nw * 128 + nw * 64 * hpb + hpb * ((L.dim + 3) & ~3) + nw * hpb * L.vdim) * 4;
+}
+template <typename T>
+static int hb_sig_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const T* cache, long ldp, int n, int n_req,
+                            int max_kvlen, long v_base) {
+    const int H = L.heads, G = L.kv_heads, ps = m->cfg.page_size, n_mix = H * L.vdim;
+    const hb_sig_score sc{L.scale, L.score_cap, L.head_temp, L.dist_bias, L.weight_bias, L.dist_n, L.chunk};
+    const float* gate = L.out_gate ? m->proj + H * L.dim + G * (L.dim + L.vdim) : nullptr;
+    const bool few = n <= HB_ATTN_SEG_ROWS;
+    if (!few && hb_try_sig_mfma(st, io, L, cache, m->proj, ldp, m->mix, (long)n_mix, sc, gate, v_base, n, n_req, ps)) return VOX_OK;
+    const int hpb = hb_sig_heads(L);
+    int nw = few ? 16 : 4;
+    while (nw > 1 && hb_sig_lds(L, hpb, nw) > 64 * 1024) nw >>= 1;
+    const int max_keys = L.chunk > 0 && L.chunk < max_kvlen ? L.chunk : max_kvlen, nchunks = (max_keys + 63) / 64;
+    const int cpb = few ? HB_SIG_SEG : nchunks, nseg = (nchunks + cpb - 1) / cpb;
+    if (nseg > 1 && (size_t)n * H * nseg * L.vdim * 4 > m->attn_ws_bytes) return vox_fail(VOX_ERR_INVALID, "hybrid_step: attention workspace");
+    float* part = nseg > 1 ? m->attn_ws : nullptr;
+#define HB_SR(HPB_) \
+    hipLaunchKernelGGL((k_hb_sig_attn_rows<T, HPB_>), dim3(n, H / HPB_, nseg), dim3(64 * nw), hb_sig_lds(L, HPB_, nw), st, m->proj, ldp, cache, m->mix, \
+                       (long)n_mix, io->pos, io->row_req, io->page_table, io->pt_stride, H, G, L.dim, L.vdim, ps, v_base, sc, cpb, part, gate, ldp, \
+                       L.out_scale)
+    if (hpb == 4) HB_SR(4);
+    else if (hpb == 3) HB_SR(3);
+    else if (hpb == 2) HB_SR(2);
+    else HB_SR(1);
+#undef HB_SR
+    if (nseg > 1)
+        hipLaunchKernelGGL(k_hb_sig_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim, L.chunk, cpb, gate, ldp,
+                           L.out_scale);
+    return VOX_OK;
+}
+
+// cur joins (A . W^T + bias)
 template <typename T>
 static int hb_gemm_resid(hipStream_t st, const float* A, long lda, const T* W, const float* bias, float* cur, long ldx, int n, int N, int K,
-                         const float* scale) {
+                         const hb_join& j) {
     hb_rowmap rm = hb_plain();
-    rm.col_scale = scale;
-    return hb_gemm<T>(st, scale ? HB_EPI_RESID_SCALED : HB_EPI_RESID, A, lda, W, bias, cur, ldx, n, N, K, rm);
+    rm.col_scale = j.scale;
+    rm.join = j;
+    const int epi = j.gate || j.streams > 0 ? HB_EPI_JOIN : (j.scale ? HB_EPI_RESID_SCALED : HB_EPI_RESID);
+    return hb_gemm<T>(st, epi, A, lda, W, bias, cur, ldx, n, N, K, rm);
 }
-// One mixer: reads the normed rows (hn != NULL) or norms `cur` itself with L.norm1, adds out_scale * mixer(.) [* ls1] to cur.
+// One mixer: reads the normed rows (hn != NULL) or norms src (rows lds apart) itself with L.norm1; out_scale * mixer(.) joins cur as `jn`
+// says (the layer's residual gate, when it has one, is added to it here: its logits are the last columns of the input projection).
 template <typename T>
 static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, void* cache, float* pool, float* state,
-                    const float* hn, float* cur, long ldx, int n, int n_req, int max_kvlen) {
+                    const float* hn, const float* src, long lds_x, float* cur, long ldx, int n, int n_req, int max_kvlen, hb_join jn) {
     const vox_hybrid_config& c = m->cfg;
     const int W = c.width, ps = c.page_size;
     const int n_in = hb_layer_in(L), n_proj = hb_layer_proj(L), n_mix = L.heads * L.vdim;
+    jn.scale = L.ls1;
+    if (L.res_gate) { jn.gate = m->proj + n_in - L.res_gate; jn.ldg = n_proj; }
     if (L.kind == VOX_MIXER_SHIFT_DECAY) {
         // five token-shift mixes of the normed input, each with its own projection
-        if (!hn) { hb_norm(m, st, n, cur, ldx, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W); hn = m->h; }
+        if (!hn) { hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W); hn = m->h; }
         const int HD = L.heads * L.dim;
         const long per_slot = (long)HD * L.dim + W, rows_stride = (long)c.max_rows * W;
         const T* wi = (const T*)L.w_in;
@@ -3318,10 +3874,10 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         if (!fused_norm)
             hipLaunchKernelGGL(k_hb_head_norm, dim3(n, L.heads), dim3(64), 0, st, m->mix, (long)n_mix, L.head_norm, 1, m->proj, (long)n_proj, 3 * HD,
                                (int)HB_GATE_SILU, L.vdim, c.eps, L.out_scale);
-        return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, L.ls1);
+        return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
     }
-    if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, cur, ldx, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W))) {
-        hb_norm(m, st, n, cur, ldx, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W);
+    if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, src, lds_x, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W))) {
+        hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W);
         hn = m->h;
     }
     if (hn) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hn, W, (const T*)L.w_in, L.b_in, m->proj, n_proj, n, n_in, W));
@@ -3417,15 +3973,19 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         float* q = m->proj + y.off_q;
         float* qa = m->proj + y.off_qa;
         float* o = m->proj + y.off_o;
-        hipLaunchKernelGGL((k_hb_latent_prep<T>), dim3(n, 2), dim3(256), 0, st, m->proj, (long)n_proj, (T*)cache, L.q_lat_norm, L.kv_lat_norm,
-                           L.inv_freq, io->pos, io->page, io->slot, L.q_rank, R, r, L.rot_dims, ps, c.eps);
-        VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, m->proj, n_proj, (const T*)L.w_uq, nullptr, q, n_proj, n, H * dq, L.q_rank));
+        const float mag = L.rot_mag != 0.f ? L.rot_mag : 1.0f;
+        const hb_sink sink{L.sinks ? 1 : 0, L.sinks};
+        const int prep_y = L.q_rank > 0 ? 2 : 1 + (r > 0 ? (H + HB_LAT_QROT_HEADS - 1) / HB_LAT_QROT_HEADS : 0);
+        hipLaunchKernelGGL((k_hb_latent_prep<T>), dim3(n, prep_y), dim3(256), 0, st, m->proj, (long)n_proj, (T*)cache, L.q_lat_norm, L.kv_lat_norm,
+                           L.inv_freq, io->pos, io->page, io->slot, L.q_rank, y.off_kv, R, r, L.rot_dims, ps, c.eps, mag, H, L.dim, y.off_qa);
+        if (L.q_rank > 0)
+            VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, m->proj, n_proj, (const T*)L.w_uq, nullptr, q, n_proj, n, H * dq, L.q_rank));
         // every head's plain query part times its key expansion: the query against the cached latent
         VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, q, n_proj, (const T*)L.w_ukT, nullptr, qa, n_proj, n, R, L.dim,
                            hb_rowmap{nullptr, nullptr, 0, 1, (long)R * L.dim, (long)dq, (long)D, 0, nullptr, 0.f}, H));
-        if (r > 0)
+        if (r > 0 && L.q_rank > 0)
             hipLaunchKernelGGL(k_hb_latent_qrot, dim3(n, H), dim3(64), 0, st, q, (long)n_proj, qa, (long)n_proj, L.inv_freq, io->pos, L.dim, R, r,
-                               L.rot_dims);
+                               L.rot_dims, mag);
         // attention of all heads over one cached head of D key dims whose first R dims are also the value
         const int G = hb_latent_groups(H), QG = H / G;
         const int window = L.window > 0 ? L.window : c.max_seq_len, P = 0x7fffffff;
@@ -3433,7 +3993,7 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         const int nwv2 = QG * split, dimp = (D + 3) & ~3;
         const size_t lds = (size_t)nwv2 * 64 * 8 + (size_t)nwv2 * 64 * 4 + (size_t)QG * dimp * 4 + (size_t)nwv2 * (R + 2) * 4;
         const int max_keys = max_kvlen < window ? max_kvlen : window;
-        const float* gate = m->proj + L.q_rank + D;
+        const float* gate = L.no_head_gate ? nullptr : m->proj + y.off_gate;
         if (n <= HB_ATTN_SEG_ROWS) {
             // few rows: a block per (row, key tiles), all heads against the tile in LDS; the tiles of a row spread over up to
             // HB_LAT_MAX_SEG blocks whose partial results are merged
@@ -3452,10 +4012,10 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
             }
             hipLaunchKernelGGL((k_hb_latent_attn_rows<T>), dim3(n, nseg2), dim3(hb_lat_tile<T>::NT), lds2, st, qa, (long)n_proj, (const T*)cache, o, (long)n_proj,
                                io->pos, io->row_req, io->page_table, io->pt_stride, H, R, r, window, ps, L.scale, cpb,
-                               seg2 ? m->attn_ws : (float*)nullptr, gate, (long)n_proj, L.out_scale, DP);
+                               seg2 ? m->attn_ws : (float*)nullptr, gate, (long)n_proj, L.out_scale, DP, sink);
             if (seg2)
                 hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg2, o, (long)n_proj, io->pos, H, R, window, P, cpb,
-                                   gate, (long)n_proj, L.out_scale, KT, 0);
+                                   gate, (long)n_proj, L.out_scale, KT, sink);
         } else if (hb_try_latent_mfma(m, st, io, L, (const T*)cache, qa, o, (long)n_proj, gate, n, n_req, window, ps)) {
         } else {
         const int nseg = 1;
@@ -3467,10 +4027,10 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         hipLaunchKernelGGL((k_hb_attn<T>), dim3(n, G, segmented ? nseg : 1), dim3(64 * nwv2), lds, st, qa, (long)n_proj, (const T*)cache,
                            (const float*)nullptr, o, (long)n_proj, io->pos, io->row_req, io->page_table, io->pt_stride, H, G, D, R, window, P, ps, 1,
                            0L, L.scale, split, segmented ? HB_ATTN_SEG : 0, segmented ? m->attn_ws : (float*)nullptr, gate, (long)n_proj,
-                           L.out_scale, 1, (long)D, 0);
+                           L.out_scale, 1, (long)D, sink);
         if (segmented)
             hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, o, (long)n_proj, io->pos, H, R, window, P,
-                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, 0);
+                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink);
         }
         // every head's weighted latent times its value expansion
         VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, o, n_proj, (const T*)L.w_uv, nullptr, m->mix, n_mix, n, L.vdim, R,
@@ -3490,6 +4050,13 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         else
             hipLaunchKernelGGL(k_hb_rglru_scan, dim3(n_req, (C + 63) / 64), dim3(64), 0, st, m->proj, (long)n_proj, m->mix, (long)n_mix, L.lam, state,
                                io->req_rows, io->req_state, io->pos, C, bs, L.conv_taps, L.rec_scale, L.out_scale);
+    } else if (L.kind == VOX_MIXER_SIGMOID_ATTN) {
+        const int H = L.heads, G = L.kv_heads;
+        const long v_base = (long)c.max_pages * ps * G * L.dim;
+        hipLaunchKernelGGL((k_hb_attn_prep<T>), dim3(n, H + G), dim3(64), 0, st, m->proj, (long)n_proj, (T*)cache, (const float*)nullptr, io->pos, io->page,
+                           io->slot, H, G, L.dim, L.vdim, 0, ps, v_base, c.eps, (float*)nullptr, io->row_req, io->page_table, io->pt_stride, 1, ps,
+                           hb_qkv_opts{L.q_norm, L.k_norm, 0.f, 1, 0});
+        VOX_TRY(hb_sig_attention<T>(m, st, io, L, (const T*)cache, (long)n_proj, n, n_req, max_kvlen, v_base));
     } else {
         const bool causal = L.kind == VOX_MIXER_CAUSAL_ATTN, conv = hb_conv_attn(L);
         // query heads per block: the whole group of a key / value head, or (groups of more than 16) its largest divisor up to 16
@@ -3507,7 +4074,7 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         const float* qrows = m->proj;
         if (conv) {
             const hb_conv_attn_layout y = hb_conv_attn_cols(L);
-            const int C = n_in;
+            const int C = n_in - L.res_gate;
             const long per_slot = (long)(L.conv_taps - 1) * C;
             hipLaunchKernelGGL(k_hb_attn_conv, dim3(n, (C + 255) / 256), dim3(256), 0, st, m->proj, (long)n_proj, L.conv_w, state, per_slot, io->pos,
                                io->row_req, io->req_rows, io->req_state, H * L.dim, G * L.dim, C, L.conv_taps, y.off_y, y.off_ss);
@@ -3533,7 +4100,7 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         const int nseg = ((max_keys + 63) / 64 + HB_ATTN_SEG - 1) / HB_ATTN_SEG;
         const bool segmented = n <= HB_ATTN_SEG_ROWS && nseg > 1 && (size_t)n * H * nseg * (L.vdim + 2) * 4 <= m->attn_ws_bytes;
         const float* gate = causal ? (const float*)nullptr : m->proj + H * L.dim + G * L.dim + G * L.vdim;      // one logit per query head
-        const int sink = causal && L.sink ? 1 : 0;
+        const hb_sink sink{causal && (L.sink || L.sinks) ? 1 : 0, causal ? L.sinks : nullptr};
         hipLaunchKernelGGL((k_hb_attn<T>), dim3(n, GG, segmented ? nseg : 1), dim3(64 * nwv2), lds, st, qrows, (long)n_proj, (const T*)cache,
                            pool, m->mix, (long)n_mix, io->pos, io->row_req, io->page_table, io->pt_stride, H, GG, L.dim, L.vdim, window,
                            P, ps, ppp, v_base, L.scale, split, segmented ? HB_ATTN_SEG : 0, segmented ? m->attn_ws : (float*)nullptr,
@@ -3542,28 +4109,34 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
             hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim, window, P,
                                HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink);
     }
-    return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, L.ls1);
+    return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
 }
 
 // Routed feed-forward of the normed rows h2, added to cur.  Few rows: one GEMV pair per routed entry; more: the entries are
 // listed per expert and every expert multiplies its own rows in one tile launch.
 template <typename T>
-static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_moe& E, const float* h2, float* cur, long ldx, int n, const float* ls) {
+static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_layer& L, const float* h2, float* cur, long ldx, int n, hb_join jn) {
+    const vox_hybrid_moe& E = *L.moe;
+    jn.scale = L.ls2;
+    if (L.res_gate) { jn.gate = m->rgate; jn.ldg = m->cfg.width; }
     const int W = m->cfg.width, nE = E.experts + E.identity, top = E.top, ne = n * top, ff = E.ff;
     const int up_down = E.expert_form == VOX_EXPERT_UP_DOWN ? 1 : 0, relu2 = E.expert_act == VOX_ACT_RELU2 ? 1 : 0, nf = up_down ? 1 : 2;
-    hipLaunchKernelGGL(k_hb_moe_router, dim3(n), dim3(256), (size_t)(6 * nE + top) * 4, st, h2, (long)W, E.router, E.correction, W, nE, top,
-                       m->moe_sel, m->moe_wgt, E.score_kind == VOX_ROUTER_SIGMOID ? 1 : 0, E.renorm, E.router_bias);
+    hipLaunchKernelGGL(k_hb_moe_router, dim3(n), dim3(256), (size_t)(6 * nE + top + (E.groups > 1 ? E.groups : 0)) * 4, st, h2, (long)W, E.router, E.correction,
+                       W, nE, top, m->moe_sel, m->moe_wgt, E.score_kind == VOX_ROUTER_SIGMOID ? 1 : 0, E.renorm, E.router_bias, E.groups, E.keep,
+                       E.weight_scale != 0.f ? E.weight_scale : 1.0f);
     if (n <= HB_MOE_GEMV_ROWS) {
         const int per = top + (E.shared_ff > 0 ? 1 : 0), maxf = ff > E.shared_ff ? ff : E.shared_ff;
         const hb_moe_small q{m->moe_sel, m->moe_wgt, top, E.experts, ff, E.shared_ff, m->max_eff, E.limit, E.shared_limit, E.act_alpha, E.up_offset,
-                             E.scale_input, nullptr, 0, up_down, relu2, ls};
-        if (maxf > 0 && per > 0 && (E.experts > 0 || E.shared_ff > 0))
-            hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((maxf + 3) / 4, n * per), dim3(256), 0, st, h2, (long)W, (const T*)E.w_gate_up,
+                             E.scale_input, nullptr, 0, up_down, relu2, jn, L.res_gate ? L.w_gate_ff : nullptr, L.b_gate_ff, m->rgate};
+        const int cols = L.res_gate && W > maxf ? W : maxf, per_y = per + (L.res_gate ? 1 : 0);
+        if (cols > 0 && per_y > 0 && (E.experts > 0 || E.shared_ff > 0 || L.res_gate))
+            hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((cols + 3) / 4, n * per_y), dim3(256), 0, st, h2, (long)W, (const T*)E.w_gate_up,
                                (const T*)E.shared_gate_up, m->moe_act, W, q);
         hipLaunchKernelGGL((k_hb_moe_down_combine<T>), dim3((W + 3) / 4, n), dim3(256), 0, st, h2, (long)W, (const T*)E.w_down,
                            (const T*)E.shared_down, m->moe_act, cur, ldx, W, q);
         return VOX_OK;
     }
+    if (L.res_gate) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, W, (const T*)L.w_gate_ff, L.b_gate_ff, m->rgate, W, n, W, W));
     if (E.experts > 0) {
         const int cap = m->cfg.max_rows;
         hipLaunchKernelGGL(k_hb_moe_group, dim3(E.experts), dim3(256), 0, st, m->moe_sel, ne, cap, m->moe_list, m->moe_count);
@@ -3576,13 +4149,13 @@ static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_moe& E, const 
                                             hb_rowmap{m->moe_count, m->moe_list, cap, 1, (long)W * ff, 0, 0, 0}, E.experts));
     }
     hipLaunchKernelGGL(k_hb_moe_combine, dim3(n), dim3(256), 0, st, cur, ldx, h2, (long)W, m->moe_out, m->moe_sel, m->moe_wgt, top, E.experts, W,
-                       E.scale_input, ls);
+                       E.scale_input, jn);
     if (E.shared_ff > 0) {
         const int sf = E.shared_ff;
         VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, W, (const T*)E.shared_gate_up, nullptr, m->ff, nf * sf, n, nf * sf, W));
         hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (sf + 1023) / 1024), dim3(256), 0, st, m->ff, m->moe_act, sf, E.shared_limit, E.act_alpha,
                            (const int*)nullptr, 0, E.up_offset, 0, up_down, relu2);
-        VOX_TRY(hb_gemm_resid<T>(st, m->moe_act, sf, (const T*)E.shared_down, nullptr, cur, ldx, n, W, sf, ls));
+        VOX_TRY(hb_gemm_resid<T>(st, m->moe_act, sf, (const T*)E.shared_down, nullptr, cur, ldx, n, W, sf, jn));
     }
     return VOX_OK;
 }
@@ -3591,11 +4164,12 @@ template <typename T>
 static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const int32_t* ids, int n, int n_req, int n_out, int max_kvlen) {
     const vox_hybrid_config& c = m->cfg;
     const int W = c.width;
-    const long ldx = 2L * W;
+    const int S = c.streams;
+    const long ldx = S > 0 ? (long)S * W : 2L * W;
     const bool bigram = c.bigram_buckets > 0 && m->w.bigram && m->w.prev_token;
     const hb_bigram bg{bigram ? m->w.bigram : nullptr, m->w.prev_token, c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, n == n_req ? 1 : 0};
     hipLaunchKernelGGL((k_hb_embed<T>), dim3(n), dim3(256), 0, st, (const T*)m->w.embedding, ids, 1, m->xa, m->xb, W, c.vocab, c.embed_scale, bg,
-                       io->pos, io->row_req, io->req_rows, io->req_state);
+                       io->pos, io->row_req, io->req_rows, io->req_state, S, S > 0 ? m->layers[m->runs[0].layer].hc_in[0] : nullptr, m->u);
     if (bigram && n != n_req)
         hipLaunchKernelGGL(k_hb_store_prev, dim3((n_req + 63) / 64), dim3(64), 0, st, ids, 1, c.vocab, io->req_rows, io->req_state, m->w.prev_token, n_req);
     float *cur = m->xa, *other = m->xb;
@@ -3607,6 +4181,17 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
             float* t = cur; cur = other; other = t;
         }
         const bool has_ff = L.ff > 0 || L.moe;
+        // what a sublayer reads (src), and how its result joins the stream(s): with several streams each sublayer leaves what the next
+        // one reads in m->u
+        const float* src = S > 0 ? m->u : cur;
+        const long lds_x = S > 0 ? W : ldx;
+        const float* next_in = ri + 1 < c.n_runs ? m->layers[m->runs[ri + 1].layer].hc_in[0] : m->ones;
+        hb_join j1{}, j2{};
+        if (S > 0) {
+            j1 = hb_join{nullptr, 0, nullptr, S, W, L.hc_mix[0], L.hc_out[0], has_ff ? L.hc_in[1] : next_in, m->u, W};
+            j2 = hb_join{nullptr, 0, nullptr, S, W, L.hc_mix[1], L.hc_out[1], next_in, m->u, W};
+        }
+        j2.scale = L.ls2;
         const bool one_norm = L.block == VOX_BLOCK_PARALLEL_ONE_NORM;
         const bool parallel = L.block == VOX_BLOCK_PARALLEL || one_norm;
         // a parallel layer norms x once for both branches before anything is added; a mixer with a sibling needs the normed rows twice
@@ -3616,22 +4201,23 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
             hn = m->h;
         }
         const float* hf = one_norm ? m->h : m->h2;      // what the feed-forward of a parallel layer reads
-        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, hn, cur, ldx, n, n_req, max_kvlen));
+        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, hn, src, lds_x, cur, ldx, n, n_req, max_kvlen, j1));
         if (L.sibling >= 0)
-            VOX_TRY(hb_mixer<T>(m, st, io, m->layers[L.sibling], run.side_cache, run.side_pool, run.side_state, hn, cur, ldx, n, n_req, max_kvlen));
+            VOX_TRY(hb_mixer<T>(m, st, io, m->layers[L.sibling], run.side_cache, run.side_pool, run.side_state, hn, src, lds_x, cur, ldx, n, n_req,
+                                max_kvlen, j1));
         if (L.moe) {
-            if (!parallel) hb_norm(m, st, n, cur, ldx, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
-            VOX_TRY(hb_moe<T>(m, st, *L.moe, hf, cur, ldx, n, L.ls2));
+            if (!parallel) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
+            VOX_TRY(hb_moe<T>(m, st, L, hf, cur, ldx, n, j2));
         } else if (L.ff > 0 && L.ff_kind == VOX_FF_GATED) {
             // down(act(gate h + b) * (up h + b)) + b: gate and up rows in one product, the activation in place behind it
-            if (!parallel) hb_norm(m, st, n, cur, ldx, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
+            if (!parallel) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
             const float* hd = parallel ? hf : m->h2;
             if (n == 1) {
                 // one row: gate and up rows of a column by one wave, biases and activation in its epilogue (the routed feed-forward's
                 // kernel with the dense unit in the place of the shared expert and nothing routed); more rows would stream the matrix
                 // once per row
                 const hb_moe_small q{nullptr, nullptr, 0, 0, 0, L.ff, L.ff, INFINITY, INFINITY, 1.0f, 0.0f, 0, L.b_up, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0,
-                                     0, 0, nullptr};
+                                     0, 0, {}, nullptr, nullptr, nullptr};
                 hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((L.ff + 3) / 4, n), dim3(256), 0, st, hd, (long)W, (const T*)nullptr, (const T*)L.w_up,
                                    m->ff_act, W, q);
             } else {
@@ -3639,25 +4225,35 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
                 hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (L.ff + 1023) / 1024), dim3(256), 0, st, m->ff, m->ff_act, L.ff, INFINITY, 1.0f,
                                    (const int*)nullptr, 0, 0.0f, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0, 0, 0);
             }
-            VOX_TRY(hb_gemm_resid<T>(st, m->ff_act, L.ff, (const T*)L.w_down, L.b_down, cur, ldx, n, W, L.ff, L.ls2));
+            VOX_TRY(hb_gemm_resid<T>(st, m->ff_act, L.ff, (const T*)L.w_down, L.b_down, cur, ldx, n, W, L.ff, j2));
         } else if (L.ff > 0) {
+            // up rows with their activation, then (a residual gate) its rows, as one product
+            const int nf = L.ff + L.res_gate, epi = L.ff_act == VOX_ACT_RELU2 ? HB_EPI_RELU2 : HB_EPI_GELU;
+            hb_rowmap rm = hb_plain();
+            rm.epi_arg = (float)L.ff;
             if (parallel) {
-                VOX_TRY(hb_gemm<T>(st, HB_EPI_GELU, hf, W, (const T*)L.w_up, nullptr, m->ff, L.ff, n, L.ff, W));
-            } else if (!(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_GELU, cur, ldx, nullptr, L.norm2, (const T*)L.w_up, nullptr, m->ff, L.ff, W))) {
-                hb_norm(m, st, n, cur, ldx, nullptr, L.norm2, m->h, nullptr, nullptr, (long)W);
-                VOX_TRY(hb_gemm<T>(st, HB_EPI_GELU, m->h, W, (const T*)L.w_up, nullptr, m->ff, L.ff, n, L.ff, W));
+                VOX_TRY(hb_gemm<T>(st, epi, hf, W, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
+            } else if (!(n == 1 && hb_try_norm_gemv<T>(m, st, epi, src, lds_x, nullptr, L.norm2, (const T*)L.w_up, L.b_up, m->ff, nf, W, rm.epi_arg))) {
+                hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h, nullptr, nullptr, (long)W);
+                VOX_TRY(hb_gemm<T>(st, epi, m->h, W, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
             }
-            VOX_TRY(hb_gemm_resid<T>(st, m->ff, L.ff, (const T*)L.w_down, nullptr, cur, ldx, n, W, L.ff, L.ls2));
+            if (L.res_gate) { j2.gate = m->ff + L.ff; j2.ldg = nf; }
+            VOX_TRY(hb_gemm_resid<T>(st, m->ff, nf, (const T*)L.w_down, nullptr, cur, ldx, n, W, L.ff, j2));
         }
-        if (io->trace)
+        if (io->trace && S > 0)
+            hipLaunchKernelGGL(k_hb_sum_streams, dim3(n), dim3(256), 0, st, cur, S, io->trace + (size_t)ri * c.max_rows * W, (long)W, W);
+        else if (io->trace)
             hipLaunchKernelGGL(k_hb_copy_rows, dim3(n), dim3(256), 0, st, cur, ldx, io->trace + (size_t)ri * c.max_rows * W, (long)W, W);
     }
     if (n_out > 0) {
+        // (several streams: the last sublayer left their sum in m->u)
+        const float* last = S > 0 ? m->u : cur;
+        const long ld_last = S > 0 ? W : ldx;
         const bool scaled = c.logit_scale != 0.f && c.logit_scale != 1.0f;
         if (!(n_out == 1 && !(c.logit_softcap > 0.f) &&
-              hb_try_norm_gemv<T>(m, st, scaled ? HB_EPI_SCALE : HB_EPI_STORE, cur, ldx, io->out_rows, m->w.final_norm, (const T*)m->w.head, nullptr,
+              hb_try_norm_gemv<T>(m, st, scaled ? HB_EPI_SCALE : HB_EPI_STORE, last, ld_last, io->out_rows, m->w.final_norm, (const T*)m->w.head, nullptr,
                                   io->logits, c.vocab, W, c.logit_scale))) {
-            hb_norm(m, st, n_out, cur, ldx, io->out_rows, m->w.final_norm, m->hout, nullptr, nullptr, (long)W);
+            hb_norm(m, st, n_out, last, ld_last, io->out_rows, m->w.final_norm, m->hout, nullptr, nullptr, (long)W);
             hb_rowmap rm = hb_plain();
             rm.epi_arg = c.logit_softcap > 0.f ? c.logit_softcap : c.logit_scale;
             VOX_TRY(hb_gemm<T>(st, c.logit_softcap > 0.f ? HB_EPI_SOFTCAP : (scaled ? HB_EPI_SCALE : HB_EPI_STORE), m->hout, W, (const T*)m->w.head,
@@ -3680,6 +4276,8 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         return vox_fail(VOX_ERR_INVALID, "hybrid_create: a logit scale beside a soft cap");
     if (cfg->norm_kind == VOX_NORM_RMS_GROUPS && (cfg->norm_groups < 1 || cfg->width % cfg->norm_groups != 0))
         return vox_fail(VOX_ERR_INVALID, "hybrid_create: %d norm groups do not divide width %d", cfg->norm_groups, cfg->width);
+    if (cfg->streams < 0 || cfg->streams > HB_MAX_STREAMS) return vox_fail(VOX_ERR_INVALID, "hybrid_create: %d residual streams (at most %d)", cfg->streams, HB_MAX_STREAMS);
+    if (cfg->streams > 0 && cfg->n_runs < 1) return vox_fail(VOX_ERR_INVALID, "hybrid_create: no layers");
     vox_hybrid* m = new vox_hybrid();
     m->ctx = ctx; m->cfg = *cfg; m->w = *w;
     m->layers.assign(w->layers, w->layers + cfg->n_layers);
@@ -3704,7 +4302,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         else if (L.kind == VOX_MIXER_RETENTION && (!L.decay || L.rot_dims < 0 || L.rot_dims > L.dim || (L.rot_dims & 1) || (L.rot_dims > 0 && !L.inv_freq)))
             bad = "retention needs decay and an even rot_dims <= dim";
         else if (L.kind == VOX_MIXER_LATENT_ATTN) {
-            if (L.q_rank < 1 || L.kv_rank < 1 || L.rot_dim < 0 || !L.w_uq || !L.w_ukT || !L.w_uv || !L.q_lat_norm || !L.kv_lat_norm) bad = "latent attention: ranks / expansions / norms";
+            if (L.q_rank < 0 || L.kv_rank < 1 || L.rot_dim < 0 || !L.w_ukT || !L.w_uv || !L.kv_lat_norm || (L.q_rank > 0 && (!L.w_uq || !L.q_lat_norm))) bad = "latent attention: ranks / expansions / norms";
             else if (L.kv_rank > 64 * HB_MAX_VPL) bad = "latent attention: kv_rank above 512";
             else if (L.kv_rank + L.rot_dim > 768) bad = "latent attention: kv_rank + rot_dim above 768 (a key tile and 16 queries have to fit the LDS)";
             else if (L.rot_dims < 0 || L.rot_dims > L.rot_dim || (L.rot_dims & 1) || (L.rot_dims > 0 && !L.inv_freq)) bad = "latent attention: rot_dims";
@@ -3725,14 +4323,29 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         else if (L.kind == VOX_MIXER_SHIFT_DECAY && (L.dim != L.vdim || L.lora < 1 || !L.shift_mu || !L.w_decay2 || !L.decay0 || !L.bonus || !L.head_norm))
             bad = "shift-decay needs mu, decay and bonus tensors";
         else if (hb_is_attn(L.kind) && L.kind != VOX_MIXER_LATENT_ATTN) {
-            if (L.kv_heads < 1 || L.heads % L.kv_heads != 0 || (L.heads / L.kv_heads > 16 && L.kind != VOX_MIXER_CAUSAL_ATTN))
+            if (L.kv_heads < 1 || L.heads % L.kv_heads != 0 || (L.heads / L.kv_heads > 16 && L.kind == VOX_MIXER_POOLED_WINDOW_ATTN))
                 bad = "heads / kv_heads (group of at most 16)";
+            else if (L.kind == VOX_MIXER_SIGMOID_ATTN && (!L.q_norm || !L.k_norm)) bad = "sigmoid attention needs q_norm and k_norm";
+            else if (L.kind == VOX_MIXER_SIGMOID_ATTN && (L.chunk < 0 || (L.dist_bias && L.dist_n < 1))) bad = "sigmoid attention: chunk / distance biases";
             else if (hb_conv_attn(L) && (!L.conv_w || (L.qk_norm_whole && (!L.q_norm || !L.k_norm)))) bad = "attention behind a convolution: conv_w / q_norm / k_norm";
             else if (hb_conv_attn(L) && (L.rot_dims < 0 || L.rot_dims > L.dim || (L.rot_dims & 1) || (L.rot_dims > 0 && !L.inv_freq))) bad = "rot_dims";
             else if (hb_conv_attn(L) && (L.q_temp_coef != 0.f || L.v_unit_rms)) bad = "attention behind a convolution: no query temperature / unit values";
             else if (L.dim > 64 * HB_MAX_DPL) bad = "dim above 512";
             else if (L.kind == VOX_MIXER_POOLED_WINDOW_ATTN && (L.window < 1 || L.pool < 1)) bad = "window / pool";
             else if (L.kind == VOX_MIXER_POOLED_WINDOW_ATTN && (L.rot_dims < 0 || L.rot_dims > L.dim || (L.rot_dims & 1) || (L.rot_dims > 0 && !L.inv_freq))) bad = "rot_dims";
+        }
+        if (!bad && L.res_gate) {
+            if (L.res_gate != cfg->width) bad = "residual gate: one row per column";
+            else if (L.kind == VOX_MIXER_RGLRU || L.kind == VOX_MIXER_SHIFT_DECAY || L.block != VOX_BLOCK_SEQUENTIAL || L.sibling >= 0)
+                bad = "residual gate: sequential layers of one mixer whose input is one projection";
+            else if (L.moe && !L.w_gate_ff) bad = "residual gate of the routed feed-forward";
+            else if (L.ff > 0 && !L.moe && L.ff_kind != VOX_FF_UP_DOWN) bad = "residual gate: the dense feed-forward has to be the up / down form";
+        }
+        if (!bad && cfg->streams > 0) {
+            const bool ff = L.ff > 0 || L.moe;
+            if (L.block != VOX_BLOCK_SEQUENTIAL || L.sibling >= 0) bad = "several residual streams: sequential layers of one mixer";
+            else if (!L.hc_in[0] || !L.hc_out[0] || !L.hc_mix[0] || (ff && (!L.hc_in[1] || !L.hc_out[1] || !L.hc_mix[1]))) bad = "several residual streams: hc_in / hc_out / hc_mix";
+            else if (L.moe && L.moe->shared_ff > 0) bad = "several residual streams: no shared expert";
         }
         if (!bad && L.moe) {
             const vox_hybrid_moe& E = *L.moe;
@@ -3742,13 +4355,16 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
             else if (!E.router || (!L.norm2 && L.block != VOX_BLOCK_PARALLEL_ONE_NORM)) bad = "moe: router or norm2 missing";
             else if (E.score_kind != VOX_ROUTER_SOFTMAX && E.score_kind != VOX_ROUTER_SIGMOID) bad = "moe: score kind";
             else if (E.experts > 0 && (E.ff < 1 || !E.w_gate_up || !E.w_down)) bad = "moe: expert weights";
+            else if (E.groups > 1 && (E.identity > 0 || E.experts % E.groups != 0 || E.keep < 1 || E.keep > E.groups || E.top > E.keep * (E.experts / E.groups)))
+                bad = "moe: groups / keep";
             else if (E.shared_ff > 0 && (!E.shared_gate_up || !E.shared_down)) bad = "moe: shared expert weights";
         }
         if (bad) { delete m; return vox_fail(VOX_ERR_INVALID, "hybrid_create: layer: %s", bad); }
         const int n_proj = hb_layer_proj(L);
         if (n_proj > m->max_in) m->max_in = n_proj;
         if (L.heads * L.vdim > m->max_mix) m->max_mix = L.heads * L.vdim;
-        if ((L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff > m->max_ff) m->max_ff = (L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff;
+        if ((L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff + L.res_gate > m->max_ff) m->max_ff = (L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff + L.res_gate;
+        if (L.moe && L.res_gate) m->any_rgate = true;
         if (L.ff_kind == VOX_FF_GATED && L.ff > m->max_gated) m->max_gated = L.ff;
         if (L.kind == VOX_MIXER_RETENTION) {
             const size_t f = ((size_t)cfg->max_rows / HB_SCAN_CHUNK + cfg->max_batch + 1) * L.heads * ((size_t)L.dim * L.vdim);
@@ -3788,17 +4404,26 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
                     bad = "missing cache / state of the sibling mixer";
             }
             if (!bad && r.loop_in && !w->loop_in) bad = "loop_in weight";
+            if (!bad && r.loop_in && cfg->streams > 0) bad = "several residual streams: no loop input";
         }
         if (bad) { delete m; return vox_fail(VOX_ERR_INVALID, "hybrid_create: run: %s", bad); }
     }
     const size_t R = cfg->max_rows, W = cfg->width;
-    bool ok = hipMalloc((void**)&m->xa, R * 2 * W * 4) == hipSuccess && hipMalloc((void**)&m->xb, R * 2 * W * 4) == hipSuccess &&
+    const size_t xw = cfg->streams > 2 ? (size_t)cfg->streams : 2;
+    bool ok = hipMalloc((void**)&m->xa, R * xw * W * 4) == hipSuccess && hipMalloc((void**)&m->xb, R * (cfg->streams > 0 ? 1 : 2) * W * 4) == hipSuccess &&
               hipMalloc((void**)&m->h, R * W * 4) == hipSuccess && hipMalloc((void**)&m->h2, R * W * 4) == hipSuccess &&
               hipMalloc((void**)&m->proj, R * (size_t)m->max_in * 4) == hipSuccess &&
               hipMalloc((void**)&m->mix, R * (size_t)m->max_mix * 4) == hipSuccess &&
               hipMalloc((void**)&m->ff, R * (size_t)(m->max_ff > 0 ? m->max_ff : 1) * 4) == hipSuccess &&
               hipMalloc((void**)&m->hout, (size_t)cfg->max_out * W * 4) == hipSuccess &&
               hipMalloc((void**)&m->logits16, (size_t)cfg->max_batch * cfg->vocab * 2) == hipSuccess;
+    if (ok && cfg->streams > 0) {
+        float one[HB_MAX_STREAMS];
+        for (float& v : one) v = 1.0f;
+        ok = hipMalloc((void**)&m->u, R * W * 4) == hipSuccess && hipMalloc((void**)&m->ones, sizeof(one)) == hipSuccess &&
+             hipMemcpy(m->ones, one, sizeof(one), hipMemcpyHostToDevice) == hipSuccess;
+    }
+    if (ok && m->any_rgate) ok = hipMalloc((void**)&m->rgate, R * W * 4) == hipSuccess;
     if (ok && m->any_shift) ok = hipMalloc((void**)&m->shift, 5 * R * W * 4) == hipSuccess;
     if (ok && m->max_gated) ok = hipMalloc((void**)&m->ff_act, R * (size_t)m->max_gated * 4) == hipSuccess;
     if (ok && m->scan_ws_floats && cfg->max_rows > HB_SCAN_CHUNK) ok = hipMalloc((void**)&m->scan_ws, m->scan_ws_floats * 4) == hipSuccess;
@@ -3814,7 +4439,12 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
     }
     // partial results of segmented attention launches: few rows x heads x segments of the longest sequence
     for (const vox_hybrid_layer& L : m->layers)
-        if (hb_is_attn(L.kind)) {
+        if (L.kind == VOX_MIXER_SIGMOID_ATTN) {
+            const int max_keys = L.chunk > 0 && L.chunk < cfg->max_seq_len ? L.chunk : cfg->max_seq_len;
+            const size_t nseg = ((size_t)(max_keys + 63) / 64 + HB_SIG_SEG - 1) / HB_SIG_SEG;
+            const size_t b = (size_t)HB_ATTN_SEG_ROWS * L.heads * nseg * L.vdim * 4;
+            if (b > m->attn_ws_bytes) m->attn_ws_bytes = b;
+        } else if (hb_is_attn(L.kind)) {
             const bool causal = L.kind == VOX_MIXER_CAUSAL_ATTN, latent = L.kind == VOX_MIXER_LATENT_ATTN;
             const int max_keys = causal || (latent && L.window < 1) ? cfg->max_seq_len
                                  : (cfg->max_seq_len < L.window ? cfg->max_seq_len : L.window) + (latent ? 0 : cfg->max_seq_len / L.pool + 1);
@@ -3832,7 +4462,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
 void vox_hybrid_destroy(vox_hybrid* m) {
     if (!m) return;
     (void)hipFree(m->xa); (void)hipFree(m->xb); (void)hipFree(m->h); (void)hipFree(m->h2); (void)hipFree(m->proj); (void)hipFree(m->mix);
-    (void)hipFree(m->ff); (void)hipFree(m->ff_act); (void)hipFree(m->hout); (void)hipFree(m->logits16); (void)hipFree(m->attn_ws); (void)hipFree(m->shift); (void)hipFree(m->scan_ws);
+    (void)hipFree(m->ff); (void)hipFree(m->ff_act); (void)hipFree(m->u); (void)hipFree(m->ones); (void)hipFree(m->rgate); (void)hipFree(m->hout); (void)hipFree(m->logits16); (void)hipFree(m->attn_ws); (void)hipFree(m->shift); (void)hipFree(m->scan_ws);
     (void)hipFree(m->moe_wgt); (void)hipFree(m->moe_sel); (void)hipFree(m->moe_act); (void)hipFree(m->moe_out);
     (void)hipFree(m->moe_list); (void)hipFree(m->moe_count);
     delete m;

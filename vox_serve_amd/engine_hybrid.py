@@ -2,9 +2,9 @@
 diagonal unit behind a short convolution, a matrix state with token shift and per-channel decay, retention with a fixed decay
 per head, the gated delta rule behind short convolutions) and with attention over a paged cache (a sliding window with pooled
 history, plain causal attention with normed q / k / v -- optionally behind a short convolution, rotated, with a softmax sink --, or
-windowed attention whose keys and values are expanded from a cached low-rank latent), optionally two mixers side by
-side, sequential or parallel layers with an optional layer scale, a dense or a routed feed-forward, and a range of layers looped over
-shared weights.
+attention whose keys and values are expanded from a cached low-rank latent, or attention with independent sigmoid weights inside
+position chunks), optionally two mixers side by side, sequential or parallel layers with an optional layer scale or a residual gate, one
+residual stream or several mixed at every sublayer, a dense or a routed feed-forward, and a range of layers looped over shared weights.
 
 It reuses the plan / stream / hipGraph machinery of the other LM engines (`Qwen3Engine`): one pinned int32 plan block per
 step, decode steps captured per batch size.  Beyond the K / V pages that the worker hands out, every request holds one
@@ -14,6 +14,7 @@ A step is ragged: `prefill(n_rows, n_req, ...)` takes prompt portions of any len
 ...)` is the one-row-per-request special case whose inputs feed back on the device.
 """
 import ctypes
+import math
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional
 
@@ -23,11 +24,11 @@ from . import _native as N
 from .engine import Qwen3Engine
 
 MIXER_HGRN2, MIXER_POOLED_WINDOW_ATTN, MIXER_MLSTM, MIXER_RGLRU, MIXER_CAUSAL_ATTN, MIXER_SHIFT_DECAY = 0, 1, 2, 3, 4, 5
-MIXER_LATENT_ATTN, MIXER_RETENTION, MIXER_DELTA = 6, 7, 8
+MIXER_LATENT_ATTN, MIXER_RETENTION, MIXER_DELTA, MIXER_SIGMOID_ATTN = 6, 7, 8, 9
 MIXER_KINDS = {"hgrn2": MIXER_HGRN2, "attention": MIXER_POOLED_WINDOW_ATTN, "mlstm": MIXER_MLSTM, "rglru": MIXER_RGLRU,
                "causal_attention": MIXER_CAUSAL_ATTN, "shift_decay": MIXER_SHIFT_DECAY, "latent_attention": MIXER_LATENT_ATTN,
-               "retention": MIXER_RETENTION, "delta": MIXER_DELTA}
-ATTENTION_KINDS = ("attention", "causal_attention", "latent_attention")
+               "retention": MIXER_RETENTION, "delta": MIXER_DELTA, "sigmoid_attention": MIXER_SIGMOID_ATTN}
+ATTENTION_KINDS = ("attention", "causal_attention", "latent_attention", "sigmoid_attention")
 NORM_KINDS = {"layer": 0, "rms_groups": 1}
 BLOCK_FORMS = {"sequential": 0, "parallel": 1, "parallel_one_norm": 2}
 FF_KINDS = {"up_down": 0, "gated": 1}
@@ -55,6 +56,9 @@ class MoECfg:
     expert_form: str = "gated"      # "gated" clamped gated units | "up_down" down(act(up h)): experts and the shared one
     expert_act: str = "swish"       # activation of the up_down form ("relu2" | "swish" with slope act_alpha)
     router_bias: bool = False       # a bias [experts + identity] is added to the router logits
+    groups: int = 0                 # > 1: equal groups of neighbouring experts, of which the `keep` best (by their best score) can be chosen from
+    keep: int = 0
+    weight_scale: float = 1.0       # multiplies the weights
 
 
 @dataclass
@@ -69,6 +73,7 @@ class MixerCfg:
     rot_dims: int = 0
     rot_base: float = 10000.0
     rot_factor: float = 1.0         # linear position scaling: every rotary frequency is divided by it
+    rot_yarn: Optional[tuple] = None    # (factor, original, fast, slow): frequency-dependent position scaling, see `yarn_frequencies`
     scale: float = 1.0              # attention score scale
     gate_cap: float = 0.0           # mLSTM: soft cap of the gate pre-activations
     ff: int = 0                     # dense feed-forward width (0: none)
@@ -82,8 +87,8 @@ class MixerCfg:
     block: str = "sequential"       # "sequential": x += mixer(norm1 x); x += ff(norm2 x) | "parallel": x += mixer(norm1 x) + ff(norm2 x)
                                     # | "parallel_one_norm": x += mixer(n) + ff(n), n = norm1 x
     ff_kind: str = "up_down"        # dense feed-forward: "up_down" down(gelu(up h)) | "gated" down(act(gate h + b) * (up h + b)) + b
-    ff_act: str = "gelu_tanh"       # activation of the gated form ("gelu_tanh" | "swish")
-    q_rank: int = 0                 # latent attention: width of the query latent
+    ff_act: str = "gelu_tanh"       # activation of the gated form ("gelu_tanh" | "swish"); "relu2": the up_down form with the square of relu
+    q_rank: int = 0                 # latent attention: width of the query latent (0: none, the query is projected from the normed row)
     kv_rank: int = 0                # latent attention: width of the cached key / value latent
     rot_dim: int = 0                # latent attention: rotated query / key dims per head (the key part is shared by all heads)
     decay: Optional[List[float]] = None     # retention: one decay per head
@@ -93,13 +98,21 @@ class MixerCfg:
     decay_channels: bool = False    # delta: one decay per head and key channel (else per head)
     gate_rank: int = 0              # delta: width of the gate bottleneck (0: one projection); `lora` is the decay bottleneck's
     gate_act: str = "silu"          # delta: activation of the output gate ("none" | "sigmoid" | "silu")
+    head_gate: bool = True          # latent attention: a sigmoid gate per head
+    chunk: int = 0                  # sigmoid attention: tokens per position chunk (0: every earlier token is seen)
+    score_cap: float = 0.0          # sigmoid attention: soft cap of the scaled scores (0: none)
+    dist_max: int = 0               # sigmoid attention: distance from which the last row of the bias table applies (0: no distance bias)
+    out_gate: bool = False          # sigmoid attention: a sigmoid gate per output column
+    res_gate: bool = False          # sublayer results are multiplied by sigmoid(W n + b) before they join the residual sum
     side: Optional["MixerCfg"] = None   # a second mixer on the same normed input, added to the same sum
     moe: Optional[MoECfg] = None    # routed feed-forward (instead of the dense one)
 
     @property
     def n_in(self) -> int:
-        """Rows of the fused input projection."""
+        """Rows of the fused input projection (without the residual gate's)."""
         h, d, v = self.heads, self.dim, self.vdim
+        if self.kind == "sigmoid_attention":
+            return h * d + self.kv_heads * (d + v) + (h * v if self.out_gate else 0)
         if self.kind == "hgrn2":
             return 2 * h * d + h * v
         if self.kind == "attention":
@@ -114,7 +127,7 @@ class MixerCfg:
         if self.kind == "shift_decay":
             return 4 * h * d + self.lora
         if self.kind == "latent_attention":
-            return self.q_rank + self.kv_rank + self.rot_dim + h
+            return (self.q_rank or h * (d + self.rot_dim)) + self.kv_rank + self.rot_dim + (h if self.head_gate else 0)
         if self.kind == "retention":
             return 2 * h * d + 2 * h * v
         return 2 * h * d + 2 * h * v + 2 * h
@@ -149,6 +162,7 @@ class HybridCfg:
     logit_softcap: float = 0.0      # > 0: logits <- cap * tanh(logits / cap)
     bigram: Optional[tuple] = None  # (buckets, mul_prev, mul_cur): x0 += bigram[(prev * mul_prev + id * mul_cur) mod buckets]
     logit_scale: float = 1.0        # logits <- logits * logit_scale
+    streams: int = 0                # > 0: copies of the residual stream, mixed at every sublayer; the head reads their sum
     norm_one_plus: bool = False     # norm weights are stored around zero: the engine multiplies by 1 + w
 
     def runs(self):
@@ -168,7 +182,8 @@ class HybridMoEC(ctypes.Structure):
                [(n, ctypes.c_float) for n in ("limit", "shared_limit", "act_alpha")] + \
                [(n, ctypes.c_void_p) for n in ("router", "correction", "w_gate_up", "w_down", "shared_gate_up", "shared_down")] + \
                [(n, ctypes.c_int32) for n in ("score_kind", "renorm", "scale_input")] + [("up_offset", ctypes.c_float)] + \
-               [("expert_form", ctypes.c_int32), ("expert_act", ctypes.c_int32), ("router_bias", ctypes.c_void_p)]
+               [("expert_form", ctypes.c_int32), ("expert_act", ctypes.c_int32), ("router_bias", ctypes.c_void_p),
+                ("groups", ctypes.c_int32), ("keep", ctypes.c_int32), ("weight_scale", ctypes.c_float)]
 
 
 class HybridLayerC(ctypes.Structure):
@@ -189,7 +204,12 @@ class HybridLayerC(ctypes.Structure):
                 ("q_lat_norm", ctypes.c_void_p), ("kv_lat_norm", ctypes.c_void_p), ("decay", ctypes.c_void_p),
                 ("ls1", ctypes.c_void_p), ("ls2", ctypes.c_void_p), ("qk_norm_whole", ctypes.c_int32), ("sink", ctypes.c_int32),
                 ("decay_channels", ctypes.c_int32), ("gate_rank", ctypes.c_int32), ("gate_act", ctypes.c_int32),
-                ("w_gate2", ctypes.c_void_p), ("a_log", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p)]
+                ("w_gate2", ctypes.c_void_p), ("a_log", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p),
+                ("chunk", ctypes.c_int32), ("dist_n", ctypes.c_int32), ("out_gate", ctypes.c_int32), ("score_cap", ctypes.c_float),
+                ("head_temp", ctypes.c_void_p), ("dist_bias", ctypes.c_void_p), ("weight_bias", ctypes.c_void_p),
+                ("no_head_gate", ctypes.c_int32), ("rot_mag", ctypes.c_float), ("sinks", ctypes.c_void_p),
+                ("res_gate", ctypes.c_int32), ("w_gate_ff", ctypes.c_void_p), ("b_gate_ff", ctypes.c_void_p),
+                ("hc_in", ctypes.c_void_p * 2), ("hc_out", ctypes.c_void_p * 2), ("hc_mix", ctypes.c_void_p * 2)]
 
 
 class HybridRunC(ctypes.Structure):
@@ -203,7 +223,7 @@ class HybridConfigC(ctypes.Structure):
                                               "max_batch", "max_out", "max_pages", "max_seq_len")] + [("eps", ctypes.c_float)] + \
                [("norm_kind", ctypes.c_int32), ("norm_groups", ctypes.c_int32), ("embed_scale", ctypes.c_float),
                 ("logit_softcap", ctypes.c_float), ("bigram_buckets", ctypes.c_int32), ("bigram_mul_prev", ctypes.c_int32),
-                ("bigram_mul_cur", ctypes.c_int32), ("logit_scale", ctypes.c_float)]
+                ("bigram_mul_cur", ctypes.c_int32), ("logit_scale", ctypes.c_float), ("streams", ctypes.c_int32)]
 
 
 class HybridWeightsC(ctypes.Structure):
@@ -221,6 +241,36 @@ def rotary_frequencies(rot_dims: int, base: float, factor: float) -> torch.Tenso
     """f_i = base^(-2i/rot_dims) / factor, i < rot_dims/2, in fp32 arithmetic."""
     i = torch.arange(rot_dims // 2, dtype=torch.float32)
     return torch.pow(torch.tensor(base, dtype=torch.float32), -(2.0 * i) / rot_dims) / factor
+
+
+def yarn_frequencies(rot_dims: int, base: float, factor: float, original: float, fast: float, slow: float):
+    """-> (frequencies [rot_dims/2] fp32, factor of cos and sin).  A pair that turns `t` times over `original` positions has the dimension
+    index rot_dims * ln(original / (2 pi t)) / (2 ln base): pairs below that of `fast` turns keep their frequency, pairs above that of
+    `slow` turns are divided by `factor`, a linear ramp in between."""
+    def index_of(turns):
+        return rot_dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo, hi = max(math.floor(index_of(fast)), 0), min(math.ceil(index_of(slow)), rot_dims - 1)
+    i = torch.arange(rot_dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(base, dtype=torch.float64), -(2.0 * i) / rot_dims)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (f / factor * ramp + f * (1.0 - ramp)).to(torch.float32), 0.1 * math.log(factor) + 1.0
+
+
+def distance_bias(table: torch.Tensor, dist_max: int, longest: int) -> torch.Tensor:
+    """A bias table [rows, heads] over distance buckets -> one bias per head and distance [heads, n] fp32.  Distances below rows/2 have a
+    row each; the other rows share the distances up to dist_max logarithmically; the last row holds beyond.  n covers every distance below
+    `longest`, or ends where the last row begins to hold (a reader clamps)."""
+    rows = table.shape[0]
+    half = rows // 2
+    n = max(min(max(dist_max, half) + 1, longest), 1)
+
+    def bucket(d):
+        if d < half:
+            return d
+        if dist_max <= half or half < 1:
+            return rows - 1
+        return min(rows - 1, half + math.floor(math.log(d / half) / math.log(dist_max / half) * (rows - half)))
+    return table.float()[torch.tensor([bucket(d) for d in range(n)])].t().contiguous()
 
 
 ROTARY_KINDS = ("attention", "latent_attention", "retention", "causal_attention")
@@ -241,7 +291,9 @@ class HybridEngine(Qwen3Engine):
     """`weights`: {"embedding", "head", "final_norm", "loop_in" (or None), "layers": [per layer dict with norm1, norm2, w_in,
     b_in, w_out, lower, head_norm, w_up, w_down, b_up, b_down; per mixer kind also q_norm, k_norm | conv_w, conv_b, w_gates, b_gates,
     lam | shift_mu, w_decay2, decay0, bonus | w_uq, w_ukT, w_uv, q_lat_norm, kv_lat_norm | conv_w, w_decay2, w_gate2, a_log, dt_bias
-    (delta rule); ls1, ls2 (layer scale); "moe": {router, router_bias, correction, w_gate_up (up rows only in the up / down form),
+    (delta rule) | q_norm, k_norm, head_temp, dist_table, weight_bias (sigmoid attention) | sinks (latent attention); ls1, ls2 (layer scale);
+    w_gate_in, b_gate_in, w_gate_ff, b_gate_ff (residual gates of the mixer and of the feed-forward); hc_in, hc_out, hc_mix (several streams:
+    [mixer's, feed-forward's]); "moe": {router, router_bias, correction, w_gate_up (up rows only in the up / down form),
     w_down, shared_gate_up, shared_down}; "side": the same mixer keys for a sibling mixer], "bigram" (or None)} — matrices in any
     float dtype (stored as the engine's dtype), vectors and the router stored as fp32.  dtype: torch.bfloat16 or torch.float32."""
 
@@ -276,6 +328,12 @@ class HybridEngine(Qwen3Engine):
             self._keep.append(t.to(dev, torch.float32).contiguous())
             return self._keep[-1].data_ptr()
 
+        def with_rows(w, b, w2, b2):
+            """(w, b or no bias) with the rows and biases of another product below them."""
+            w2, b2 = w2.to(w.device), b2.float()
+            b = torch.zeros(w.shape[0], dtype=torch.float32, device=b2.device) if b is None else b.float().to(b2.device)
+            return torch.cat([w, w2.to(w.dtype)], 0), torch.cat([b, b2], 0)
+
         def norm_w(t):
             """A norm weight of the residual stream: stored around zero when the config says so (1 + w, formed in fp32)."""
             return vec(t.float() + 1.0) if (t is not None and cfg.norm_one_plus) else vec(t)
@@ -287,6 +345,22 @@ class HybridEngine(Qwen3Engine):
 
         def fill(c, m, lw, i):
             assert tuple(lw["w_in"].shape) == (m.n_in, W), (i, m.kind, tuple(lw["w_in"].shape), m.n_in)
+            w_in, b_in, w_up, b_up = lw["w_in"], lw.get("b_in"), lw.get("w_up"), lw.get("b_up")
+            if m.res_gate:
+                # the gates' rows ride along as the last ones of the products that read the same normed rows
+                w_in, b_in = with_rows(w_in, b_in, lw["w_gate_in"], lw["b_gate_in"])
+                c.res_gate = W
+                if m.moe is not None:
+                    c.w_gate_ff, c.b_gate_ff = mat(lw["w_gate_ff"]), vec(lw["b_gate_ff"])
+                elif m.ff:
+                    w_up, b_up = with_rows(w_up, b_up, lw["w_gate_ff"], lw["b_gate_ff"])
+            for j, t in enumerate(lw.get("hc_in") or []):
+                c.hc_in[j], c.hc_out[j], c.hc_mix[j] = vec(t), vec(lw["hc_out"][j]), vec(lw["hc_mix"][j])
+            c.chunk, c.score_cap, c.out_gate, c.no_head_gate = m.chunk, m.score_cap, int(m.out_gate), int(not m.head_gate)
+            c.head_temp, c.weight_bias, c.sinks = vec(lw.get("head_temp")), vec(lw.get("weight_bias")), vec(lw.get("sinks"))
+            if m.dist_max > 0:
+                bias = distance_bias(lw["dist_table"], m.dist_max, m.chunk or max_seq_len)
+                c.dist_n, c.dist_bias = bias.shape[1], vec(bias)
             assert tuple(lw["w_out"].shape) == (W, m.heads * m.vdim), (i, m.kind, tuple(lw["w_out"].shape))
             c.kind, c.heads, c.kv_heads, c.dim, c.vdim = MIXER_KINDS[m.kind], m.heads, m.kv_heads, m.dim, m.vdim
             c.window, c.pool, c.rot_dims, c.scale, c.gate_cap, c.ff = m.window, m.pool, m.rot_dims, m.scale, m.gate_cap, m.ff
@@ -295,10 +369,14 @@ class HybridEngine(Qwen3Engine):
             c.qk_norm_whole, c.sink = int(m.qk_norm_whole), int(m.sink)
             c.decay_channels, c.gate_rank, c.gate_act = int(m.decay_channels), m.gate_rank, GATE_KINDS[m.gate_act]
             c.w_gate2, c.a_log, c.dt_bias = mat(lw.get("w_gate2")), vec(lw.get("a_log")), vec(lw.get("dt_bias"))
-            c.w_in, c.b_in, c.w_out = mat(lw["w_in"]), vec(lw.get("b_in")), mat(lw["w_out"])
+            c.w_in, c.b_in, c.w_out = mat(w_in), vec(b_in), mat(lw["w_out"])
             c.lower, c.head_norm = vec(lw.get("lower")), vec(lw.get("head_norm"))
-            c.inv_freq = vec(rotary_frequencies(m.rot_dims, m.rot_base, m.rot_factor)) if m.kind in ROTARY_KINDS and m.rot_dims else None
-            c.w_up, c.w_down = mat(lw.get("w_up")), mat(lw.get("w_down"))
+            if m.kind in ROTARY_KINDS and m.rot_dims and m.rot_yarn:
+                freqs, c.rot_mag = yarn_frequencies(m.rot_dims, m.rot_base, *m.rot_yarn)
+                c.inv_freq = vec(freqs)
+            else:
+                c.inv_freq = vec(rotary_frequencies(m.rot_dims, m.rot_base, m.rot_factor)) if m.kind in ROTARY_KINDS and m.rot_dims else None
+            c.w_up, c.w_down = mat(w_up), mat(lw.get("w_down"))
             c.block, c.sibling, c.out_scale = BLOCK_FORMS[m.block], -1, m.out_scale
             c.q_norm, c.k_norm = vec(lw.get("q_norm")), vec(lw.get("k_norm"))
             c.q_temp_coef, c.q_temp_every, c.v_unit_rms = m.q_temp_coef, m.q_temp_every, int(m.v_unit_rms)
@@ -307,7 +385,7 @@ class HybridEngine(Qwen3Engine):
                 vec(lw.get("b_gates")), vec(lw.get("lam"))
             c.lora, c.shift_mu, c.w_decay2 = m.lora, vec(lw.get("shift_mu")), mat(lw.get("w_decay2"))
             c.decay0, c.bonus = vec(lw.get("decay0")), vec(lw.get("bonus"))
-            c.ff_kind, c.ff_act, c.b_up, c.b_down = FF_KINDS[m.ff_kind], ACT_KINDS[m.ff_act], vec(lw.get("b_up")), vec(lw.get("b_down"))
+            c.ff_kind, c.ff_act, c.b_up, c.b_down = FF_KINDS[m.ff_kind], ACT_KINDS[m.ff_act], vec(b_up), vec(lw.get("b_down"))
             c.q_rank, c.kv_rank, c.rot_dim = m.q_rank, m.kv_rank, m.rot_dim
             c.w_uq, c.w_ukT, c.w_uv = mat(lw.get("w_uq")), mat(lw.get("w_ukT")), mat(lw.get("w_uv"))
             c.q_lat_norm, c.kv_lat_norm = vec(lw.get("q_lat_norm")), vec(lw.get("kv_lat_norm"))
@@ -321,7 +399,7 @@ class HybridEngine(Qwen3Engine):
                                 vec(ew["router"]), vec(ew.get("correction")), mat(ew.get("w_gate_up")), mat(ew.get("w_down")),
                                 mat(ew.get("shared_gate_up")), mat(ew.get("shared_down")), ROUTER_SCORES[e.score], int(e.renorm),
                                 int(e.scale_input), e.up_offset, EXPERT_FORMS[e.expert_form], ACT_KINDS[e.expert_act],
-                                vec(ew.get("router_bias")) if e.router_bias else None)
+                                vec(ew.get("router_bias")) if e.router_bias else None, e.groups, e.keep, e.weight_scale)
                 self._moes.append(mc)
                 c.moe = ctypes.pointer(mc)
 
@@ -365,7 +443,7 @@ class HybridEngine(Qwen3Engine):
         bg = reduced_bigram(cfg.bigram)
         cc = HybridConfigC(W, cfg.vocab, len(larr), len(runs), 0 if dtype == torch.bfloat16 else 1, page_size, self.max_rows,
                            max_batch, self.max_out, max_pages, max_seq_len, cfg.eps, NORM_KINDS[cfg.norm_kind], cfg.norm_groups,
-                           cfg.embed_scale, cfg.logit_softcap, int(bg[0]), int(bg[1]), int(bg[2]), float(cfg.logit_scale))
+                           cfg.embed_scale, cfg.logit_softcap, int(bg[0]), int(bg[1]), int(bg[2]), float(cfg.logit_scale), int(cfg.streams))
         # the last token every state slot's sequence has seen (what a bigram embedding needs of the step before)
         self.prev_token = torch.zeros(self.state_slots, dtype=torch.int32, device=dev)
         if cfg.bigram and tuple(weights["bigram"].shape) != (int(bg[0]) + 1, W):

@@ -203,6 +203,13 @@ def _sizitar(model_name, device="cuda:0", weights=None, checkpoint_dir=None, syn
     return _hybrid_lm(".sizitar", "SizitarModel", model_name, device, weights, checkpoint_dir, synthetic, config, kw)
 
 
+@register_model("gaparax")
+def _gaparax(model_name, device="cuda:0", weights=None, checkpoint_dir=None, synthetic=False, config=None, **kw):
+    """LM of chunked sigmoid-weighted attention and latent attention with sinks over several residual streams, gated sublayers and
+    group-limited routing."""
+    return _hybrid_lm(".gaparax", "GaparaxModel", model_name, device, weights, checkpoint_dir, synthetic, config, kw)
+
+
 def load_checkpoint_dir(path: str, device: str = "cuda:0", **kw):
     """A local checkpoint folder whose config.json names its architecture: the registry entry of that name loads it."""
     import json

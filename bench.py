@@ -752,8 +752,15 @@ def main():
     ap.add_argument("--sizitar", action="store_true", help="instead of the default workload: prefill / decode throughput of the Sizitar "
                     "design (random weights) beside Fusanex, the closest existing model, on the same engine at equal width and depth "
                     "(tools/bench_sizitar.py); prints that comparison as one JSON line")
+    ap.add_argument("--gaparax", action="store_true", help="instead of the default workload: prefill / decode throughput of the Gaparax "
+                    "design (random weights) beside Dipivik, the closest existing model, on the same engine at equal width and depth "
+                    "(tools/bench_gaparax.py); prints that comparison as one JSON line")
     args = ap.parse_args()
 
+    if args.gaparax:
+        from tools.bench_gaparax import run as run_gaparax
+        print(json.dumps(run_gaparax(steps=min(args.steps, 50), warmup=min(args.warmup, 10))))
+        return
     if args.sizitar:
         from tools.bench_sizitar import run as run_sizitar
         print(json.dumps(run_sizitar(steps=min(args.steps, 50), warmup=min(args.warmup, 10))))

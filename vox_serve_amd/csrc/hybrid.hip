@@ -112,24 +112,60 @@ struct hb_join {
     float* u;
     long ldu;
 };
-__device__ __forceinline__ void hb_join_add(const hb_join& j, float* x, int row, int col, float v) {
-    if (j.gate) v *= hb_sigmoid(j.gate[(size_t)row * j.ldg + col]);
-    if (j.scale) v *= j.scale[col];
-    if (j.streams == 0) { x[col] += v; return; }
-    float xs[HB_MAX_STREAMS];
+// what a join reads of its place, requested ahead of the product by kernels that have nothing to do meanwhile
+struct hb_join_in {
+    float gate, xs[HB_MAX_STREAMS];
+};
+__device__ __forceinline__ hb_join_in hb_join_load(const hb_join& j, const float* x, int row, int col) {
+    hb_join_in in;
+    in.gate = j.gate ? j.gate[(size_t)row * j.ldg + col] : 0.f;
 #pragma unroll
-    for (int s = 0; s < HB_MAX_STREAMS; ++s) xs[s] = s < j.streams ? x[(size_t)s * j.sld + col] : 0.f;
-    float u = 0.f;
-    for (int t = 0; t < j.streams; ++t) {
-        float nx = 0.f;
+    for (int s = 0; s < HB_MAX_STREAMS; ++s) in.xs[s] = 0.f;
+    if (j.streams == 0) in.xs[0] = x[col];
+    else
 #pragma unroll
         for (int s = 0; s < HB_MAX_STREAMS; ++s)
-            if (s < j.streams) nx = fmaf(j.mix[s * j.streams + t], xs[s], nx);
-        nx = fmaf(j.out[t], v, nx);
+            if (s < j.streams) in.xs[s] = x[(size_t)s * j.sld + col];
+    return in;
+}
+template <int S> __device__ __forceinline__ float hb_join_streams(const hb_join& j, const hb_join_in& in, float* x, int col, float v) {
+    float mix[S * S], out[S], next[S], u = 0.f;
+#pragma unroll
+    for (int i = 0; i < S * S; ++i) mix[i] = j.mix[i];
+#pragma unroll
+    for (int t = 0; t < S; ++t) { out[t] = j.out[t]; next[t] = j.next[t]; }
+#pragma unroll
+    for (int t = 0; t < S; ++t) {
+        float nx = 0.f;
+#pragma unroll
+        for (int s = 0; s < S; ++s) nx = fmaf(mix[s * S + t], in.xs[s], nx);
+        nx = fmaf(out[t], v, nx);
         x[(size_t)t * j.sld + col] = nx;
-        u = fmaf(j.next[t], nx, u);
+        u = fmaf(next[t], nx, u);
     }
+    return u;
+}
+__device__ __forceinline__ void hb_join_apply(const hb_join& j, const hb_join_in& in, float* x, int row, int col, float v) {
+    if (j.gate) v *= hb_sigmoid(in.gate);
+    if (j.scale) v *= j.scale[col];
+    if (j.streams == 0) { x[col] = in.xs[0] + v; return; }
+    float u = 0.f;
+    if (j.streams == 2) u = hb_join_streams<2>(j, in, x, col, v);
+    else if (j.streams == 4) u = hb_join_streams<4>(j, in, x, col, v);
+    else
+        for (int t = 0; t < j.streams; ++t) {
+            float nx = 0.f;
+#pragma unroll
+            for (int s = 0; s < HB_MAX_STREAMS; ++s)
+                if (s < j.streams) nx = fmaf(j.mix[s * j.streams + t], in.xs[s], nx);
+            nx = fmaf(j.out[t], v, nx);
+            x[(size_t)t * j.sld + col] = nx;
+            u = fmaf(j.next[t], nx, u);
+        }
     j.u[(size_t)row * j.ldu + col] = u;
+}
+__device__ __forceinline__ void hb_join_add(const hb_join& j, float* x, int row, int col, float v) {
+    hb_join_apply(j, hb_join_load(j, x, row, col), x, row, col, v);
 }
 // Several products in one launch: product z uses the matrix Wt + z*w_stride, the activations A + z*a_stride, the outputs
 // C + z*c_stride and the bias + z*b_stride (a strided batch: block-diagonal matrices, projections that each read their own input).
@@ -572,6 +608,9 @@ __global__ __launch_bounds__(256) void k_hb_gemv(const float* A, long lda, const
 #pragma unroll
     for (int j = 0; j < HB_GEMV_CPW; ++j) wr[j] = Wt + (size_t)(n0 + j < N ? n0 + j : N - 1) * K;
     const bool vec = (K % CH == 0) && ((((size_t)Wt) & 15) == 0) && (lda % 4 == 0) && ((((size_t)A) & 15) == 0);
+    constexpr bool AHEAD = EPI == HB_EPI_JOIN && MR == 1 && HB_GEMV_CPW == 1;
+    hb_join_in jin;
+    if (AHEAD) jin = hb_join_load(rm.join, C, 0, n0);
     if (vec) {
         for (int k = lane * CH; k < K; k += 64 * CH) {
             float w[HB_GEMV_CPW][CH];
@@ -620,72 +659,111 @@ __global__ __launch_bounds__(256) void k_hb_gemv(const float* A, long lda, const
 #pragma unroll
         for (int j = 0; j < HB_GEMV_CPW; ++j) {
             const float sum = hb_wave_sum(acc[m][j]);
-            if (m < M && n0 + j < N && lane == 0) hb_finish<EPI>(rm, C, ldc, m, n0 + j, sum, bias ? bias[n0 + j] : 0.f);
+            if (AHEAD) {
+                if (lane == 0) hb_join_apply(rm.join, jin, C, 0, n0, sum + (bias ? bias[n0] : 0.f));
+            } else if (m < M && n0 + j < N && lane == 0) hb_finish<EPI>(rm, C, ldc, m, n0 + j, sum, bias ? bias[n0 + j] : 0.f);
         }
 }
 
-// One-row steps: the weight-only LayerNorm of the row fused in front of the GEMV.  Every wave takes the row's statistics itself
-// (mean, then the mean of the squared deviations; lane-chunked sums and a butterfly, an order fixed by K), so the row is read three
-// times from cache instead of once from a normalised copy, and a dependent launch is saved.  Needs K % 8 == 0 (4 for fp32).
-template <typename T, int EPI, int CPW>
+// One-row steps: the norm of the row (weight-only LayerNorm; rms != 0: the RMS norm over the whole row) fused in front of the GEMV.
+// Every wave takes the row's statistics itself (mean, then the mean of the squared deviations; lane-chunked sums and a butterfly, an
+// order fixed by K), so the row is read from cache instead of from a normalised copy, and a dependent launch is saved.  NK > 0: a
+// lane's share of the row and of its weight rows (K <= 64 * CH * NK) is requested at the start and kept in registers, so the weights
+// are on their way while the statistics are taken; NK = 0: any K, several reads.  Same sums in the same order either way.  Needs
+// K % 8 == 0 (4 for fp32).
+template <typename T, int EPI, int CPW, int NK>
 __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, const int* rows, const float* lnw, float eps, const T* Wt,
                                                     const float* bias, float* C, int N, int K, int rms, float epi_arg) {
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CPW;
     if (n0 >= N) return;
-    constexpr int CH = sizeof(T) == 2 ? 8 : 4;
+    constexpr int CH = sizeof(T) == 2 ? 8 : 4, NR = NK > 0 ? NK : 1;
     const float* xr = X + (size_t)(rows ? rows[0] : 0) * ldx;
-    // rms != 0: the RMS norm over the whole row (no mean is taken off)
+    const T* wr[CPW];
+#pragma unroll
+    for (int j = 0; j < CPW; ++j) wr[j] = Wt + (size_t)(n0 + j < N ? n0 + j : N - 1) * K;
+    uint4 wreg[CPW][NR];
+    float4 xreg[NR][CH / 4];
+    if (NK > 0) {
+#pragma unroll
+        for (int i = 0; i < NR; ++i) {
+            const int k = (lane + 64 * i) * CH, kc = k < K ? k : 0;
+#pragma unroll
+            for (int e = 0; e < CH; e += 4) xreg[i][e / 4] = *(const float4*)(xr + kc + e);
+#pragma unroll
+            for (int j = 0; j < CPW; ++j) wreg[j][i] = *(const uint4*)(wr[j] + kc);
+        }
+    }
+    auto each_x = [&](auto&& f) {       // f(k, e, the row's four values at k + e), this lane's chunks in ascending order
+        if (NK > 0) {
+#pragma unroll
+            for (int i = 0; i < NR; ++i) {
+                const int k = (lane + 64 * i) * CH;
+                if (k < K)
+#pragma unroll
+                    for (int e = 0; e < CH; e += 4) f(k, e, xreg[i][e / 4]);
+            }
+        } else {
+            for (int k = lane * CH; k < K; k += 64 * CH)
+#pragma unroll
+                for (int e = 0; e < CH; e += 4) f(k, e, *(const float4*)(xr + k + e));
+        }
+    };
     float mean = 0.f;
     if (!rms) {
         float s = 0.f;
-        for (int k = lane * CH; k < K; k += 64 * CH)
-#pragma unroll
-            for (int e = 0; e < CH; e += 4) {
-                const float4 x4 = *(const float4*)(xr + k + e);
-                s += x4.x; s += x4.y; s += x4.z; s += x4.w;
-            }
+        each_x([&](int, int, const float4& x4) { s += x4.x; s += x4.y; s += x4.z; s += x4.w; });
         mean = hb_wave_sum(s) / (float)K;
     }
     float q = 0.f;
-    for (int k = lane * CH; k < K; k += 64 * CH)
-#pragma unroll
-        for (int e = 0; e < CH; e += 4) {
-            const float4 x4 = *(const float4*)(xr + k + e);
-            const float d0 = x4.x - mean, d1 = x4.y - mean, d2 = x4.z - mean, d3 = x4.w - mean;
-            q += d0 * d0; q += d1 * d1; q += d2 * d2; q += d3 * d3;
-        }
+    each_x([&](int, int, const float4& x4) {
+        const float d0 = x4.x - mean, d1 = x4.y - mean, d2 = x4.z - mean, d3 = x4.w - mean;
+        q += d0 * d0; q += d1 * d1; q += d2 * d2; q += d3 * d3;
+    });
     const float inv = 1.0f / sqrtf(hb_wave_sum(q) / (float)K + eps);
     float acc[CPW];
 #pragma unroll
     for (int j = 0; j < CPW; ++j) acc[j] = 0.f;
-    const T* wr[CPW];
-#pragma unroll
-    for (int j = 0; j < CPW; ++j) wr[j] = Wt + (size_t)(n0 + j < N ? n0 + j : N - 1) * K;
-    for (int k = lane * CH; k < K; k += 64 * CH) {
-        float w[CPW][CH];
-#pragma unroll
-        for (int j = 0; j < CPW; ++j) {
-            if (sizeof(T) == 2) {
-                const uint4 u = *(const uint4*)(wr[j] + k);
-                w[j][0] = bflo(u.x); w[j][1] = bfhi(u.x); w[j][2] = bflo(u.y); w[j][3] = bfhi(u.y);
-                if (CH == 8) { w[j][4] = bflo(u.z); w[j][5] = bfhi(u.z); w[j][6] = bflo(u.w); w[j][7] = bfhi(u.w); }
-            } else {
-                const float4 u = *(const float4*)(wr[j] + k);
-                w[j][0] = u.x; w[j][1] = u.y; w[j][2] = u.z; w[j][3] = u.w;
-            }
-        }
+    auto product = [&](int k, const uint4* u, const float4* xv) {      // one chunk: u = the CPW rows' weights, xv = the row's values
 #pragma unroll
         for (int e = 0; e < CH; e += 4) {
-            const float4 x4 = *(const float4*)(xr + k + e), g4 = *(const float4*)(lnw + k + e);
+            const float4 x4 = xv[e / 4], g4 = *(const float4*)(lnw + k + e);
             const float x[4] = {hb_operand<T>((x4.x - mean) * inv * g4.x), hb_operand<T>((x4.y - mean) * inv * g4.y),
                                 hb_operand<T>((x4.z - mean) * inv * g4.z), hb_operand<T>((x4.w - mean) * inv * g4.w)};
 #pragma unroll
             for (int j = 0; j < CPW; ++j) {
-                acc[j] = fmaf(w[j][e], x[0], acc[j]);
-                acc[j] = fmaf(w[j][e + 1], x[1], acc[j]);
-                acc[j] = fmaf(w[j][e + 2], x[2], acc[j]);
-                acc[j] = fmaf(w[j][e + 3], x[3], acc[j]);
+                const uint4 v = u[j];
+                float w[4];
+                if (sizeof(T) == 2) {
+                    const u32 a = e == 0 ? v.x : v.z, b = e == 0 ? v.y : v.w;
+                    w[0] = bflo(a); w[1] = bfhi(a); w[2] = bflo(b); w[3] = bfhi(b);
+                } else {
+                    w[0] = __uint_as_float(v.x); w[1] = __uint_as_float(v.y); w[2] = __uint_as_float(v.z); w[3] = __uint_as_float(v.w);
+                }
+                acc[j] = fmaf(w[0], x[0], acc[j]);
+                acc[j] = fmaf(w[1], x[1], acc[j]);
+                acc[j] = fmaf(w[2], x[2], acc[j]);
+                acc[j] = fmaf(w[3], x[3], acc[j]);
             }
+        }
+    };
+    if (NK > 0) {
+#pragma unroll
+        for (int i = 0; i < NR; ++i) {
+            const int k = (lane + 64 * i) * CH;
+            uint4 u[CPW];
+#pragma unroll
+            for (int j = 0; j < CPW; ++j) u[j] = wreg[j][i];
+            if (k < K) product(k, u, xreg[i]);
+        }
+    } else {
+        for (int k = lane * CH; k < K; k += 64 * CH) {
+            uint4 u[CPW];
+            float4 xv[CH / 4];
+#pragma unroll
+            for (int j = 0; j < CPW; ++j) u[j] = *(const uint4*)(wr[j] + k);
+#pragma unroll
+            for (int e = 0; e < CH; e += 4) xv[e / 4] = *(const float4*)(xr + k + e);
+            product(k, u, xv);
         }
     }
 #pragma unroll
@@ -703,10 +781,18 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
     if (K % CH || (ldx & 3) || ((size_t)X & 15) || ((size_t)W & 15) || ((size_t)lnw & 15)) return false;
     const bool wide = N >= 16 * 1024;
     const dim3 g(wide ? (N + 15) / 16 : (N + 3) / 4), b(256);
+    const int nk = (K + 64 * CH - 1) / (64 * CH);
+#define HB_LN2(EPI_, CPW_) \
+    do { \
+        if (nk <= 2) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 2>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 4) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 4>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 8) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 8>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 0>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+    } while (0)
 #define HB_LN(EPI_) \
     do { \
-        if (wide) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, 4>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
-        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, 1>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+        if (wide) HB_LN2(EPI_, 4); \
+        else HB_LN2(EPI_, 1); \
     } while (0)
     if (epi == HB_EPI_GELU) HB_LN(HB_EPI_GELU);
     else if (epi == HB_EPI_SCALE) HB_LN(HB_EPI_SCALE);
@@ -714,6 +800,7 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
     else if (epi != HB_EPI_STORE) return false;
     else HB_LN(HB_EPI_STORE);
 #undef HB_LN
+#undef HB_LN2
     return true;
 }
 
@@ -735,6 +822,11 @@ __global__ __launch_bounds__(512) void k_hb_gemm_rows16(const float* A, long lda
     const bf16_t* wrow = Wt + (size_t)(n0 + col < N ? n0 + col : N - 1) * K + kb * 8;
     const float* arow = A + (size_t)(col < M ? col : M - 1) * lda + kb * 8;
     const bool rowok = col < M;
+    // the first 256 threads finish one output each
+    const int orow = threadIdx.x >> 4, ocol = threadIdx.x & 15;
+    const bool mine = threadIdx.x < 256 && orow < M && n0 + ocol < N;
+    hb_join_in jin;
+    if (EPI == HB_EPI_JOIN && mine) jin = hb_join_load(rm.join, C + (size_t)orow * ldc, orow, n0 + ocol);
     constexpr int U = 8;
     for (int s0 = wv; s0 < nsteps; s0 += 8 * U) {
         uint4 wf[U];
@@ -761,13 +853,12 @@ __global__ __launch_bounds__(512) void k_hb_gemm_rows16(const float* A, long lda
 #pragma unroll
     for (int r = 0; r < 4; ++r) red[wv][kb * 4 + r][col] = acc[r];
     __syncthreads();
-    if (wv == 0 && n0 + col < N) {
-        const float bz = bias ? bias[n0 + col] : 0.f;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int row = kb * 4 + r;
-            if (row < M) hb_finish<EPI>(rm, C, ldc, row, n0 + col, ((((((red[0][row][col] + red[1][row][col]) + red[2][row][col]) + red[3][row][col]) + red[4][row][col]) + red[5][row][col]) + red[6][row][col]) + red[7][row][col], bz);
-        }
+    if (mine) {
+        const float bz = bias ? bias[n0 + ocol] : 0.f;
+        const float sum = ((((((red[0][orow][ocol] + red[1][orow][ocol]) + red[2][orow][ocol]) + red[3][orow][ocol]) + red[4][orow][ocol]) + red[5][orow][ocol]) +
+                           red[6][orow][ocol]) + red[7][orow][ocol];
+        if (EPI == HB_EPI_JOIN) hb_join_apply(rm.join, jin, C + (size_t)orow * ldc, orow, n0 + ocol, sum + bz);
+        else hb_finish<EPI>(rm, C, ldc, orow, n0 + ocol, sum, bz);
     }
 }
 // every operand of every product of a strided batch is 16-byte aligned
@@ -2682,7 +2773,7 @@ template <typename T> static int hb_lat_dp(int D) {
 //                                                          product (lane group g holds keys 4g..4g+3 of each 16-key tile: the k index of
 //                                                          the product is laid out to match, so no weight leaves its lane), hi + lo
 // Scores, maxima, sums and weights are fp32; the two-part operands keep 16 bits of mantissa of the queries and weights.
-// Tile t of the launch is found by walking the requests' row counts (ceil(rows / 4) tiles each); blocks beyond the last tile leave.
+// Tile t of the launch (blocks in descending order) is found by walking the requests' row counts (ceil(rows / 4) tiles each); blocks beyond the last tile leave.
 #define HB_LM_VLD 72      // keys per row of the transposed value tile (64 + 8: rows 16 bytes apart in banks)
 __device__ __forceinline__ void hb_split_bf16x8(const float* v, uint4& hi, uint4& lo) {
     float h[8];
@@ -2707,7 +2798,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     bf16_t* Kt = (bf16_t*)(sm + 128);              // [64][DPK]
     bf16_t* Vt = Kt + 64 * DPK;                    // [ct_n * 16][HB_LM_VLD]
     const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, col = lane & 15, g = lane >> 4;
-    int t = blockIdx.x, rq = -1, rs = 0, re = 0;
+    // later rows of a request see more keys: their tiles start first, so that the launch does not end on them
+    int t = gridDim.x - 1 - blockIdx.x, rq = -1, rs = 0, re = 0;
     for (int q = 0; q < n_req; ++q) {
         const int a = req_rows[q], b = req_rows[q + 1], nt = (b - a + 3) >> 2;
         if (t < nt) { rq = q; rs = a + 4 * t; re = b; break; }
@@ -2887,119 +2979,122 @@ __device__ __forceinline__ float hb_sig_weight(const hb_sig_score& sc, int h, fl
     return hb_sigmoid(z);
 }
 // Steps of few rows (and every step of shapes or dtypes the matrix-core form does not take): block = (row, HPB query heads of one key
-// head, segment of cpb 64-key chunks); wave w takes the segment's chunks w, w + waves, ...: lane = key for the scores of the HPB heads,
-// then lane = value columns (two adjacent ones of each 128 with a bf16 cache and even sizes) for the weighted sums; the waves' sums are
-// added in wave order.  part != NULL: the segment's sums are left there for k_hb_sig_merge; else gate and scale are applied here.
+// head, segment of cpb 64-key chunks), four waves.  Scores: lane = key, a wave takes one head (fewer than three heads: a part of the key
+// dims of one head, the parts added in order).  Weighted sums: a wave takes 16 keys of the chunk and all heads, lane = value columns (two
+// adjacent ones of each 128 with a bf16 cache and even sizes, the first 128 columns requested before the scores are formed); the waves'
+// sums are added in wave order.  part != NULL: the segment's sums are left there for k_hb_sig_merge; else gate and scale are applied here.
 template <typename T, int HPB>
-__global__ __launch_bounds__(1024) void k_hb_sig_attn_rows(const float* q, long ldq, const T* cache, float* out, long ldo, const int* pos,
-                                                           const int* row_req, const int* ptab, int pts, int H, int G, int dim, int vdim, int ps,
-                                                           long v_base, hb_sig_score sc, int cpb, float* part, const float* gate, long ldg,
-                                                           float out_scale) {
+__global__ __launch_bounds__(256) void k_hb_sig_attn_rows(const float* q, long ldq, const T* cache, float* out, long ldo, const int* pos,
+                                                          const int* row_req, const int* ptab, int pts, int H, int G, int dim, int vdim, int ps,
+                                                          long v_base, hb_sig_score sc, int cpb, float* part, const float* gate, long ldg,
+                                                          float out_scale) {
     extern __shared__ float sm[];
-    const int NW = blockDim.x >> 6, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    constexpr int DS = HPB == 1 ? 4 : (HPB == 2 ? 2 : 1), VE = 16 / sizeof(T);
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int dimp = (dim + 3) & ~3;
-    long* loc = (long*)sm;                       // [NW][64] cache token of each lane's key
-    float* pw = sm + NW * 128;                   // [NW][64][HPB] weights
-    float* qs = pw + NW * 64 * HPB;              // [HPB][dimp]
-    float* red = qs + HPB * dimp;                // [NW][HPB * vdim]
+    float* qs = sm;                              // [HPB][dimp]
+    float* dots = qs + HPB * dimp;               // [4][64] partial dots
+    float* pw = dots + 256;                      // [64][HPB] weights
+    float* red = pw + 64 * HPB;                  // [4][HPB * vdim]
     const int row = blockIdx.x, h0 = blockIdx.y * HPB, g = h0 / (H / G), p = pos[row];
     const int* pt = ptab + (size_t)row_req[row] * pts;
     const int lo = hb_chunk_start(p, sc.chunk), total = p - lo + 1, nchunks = (total + 63) >> 6;
     const int c0 = blockIdx.z * cpb, c1 = c0 + cpb < nchunks ? c0 + cpb : nchunks;
     if (c0 >= nchunks) return;
-    for (int i = tid; i < HPB * dimp; i += blockDim.x) {
+    for (int i = tid; i < HPB * dimp; i += 256) {
         const int h = i / dimp, d = i - h * dimp;
         qs[i] = d < dim ? q[(size_t)row * ldq + (size_t)(h0 + h) * dim + d] : 0.f;
     }
     __syncthreads();
-    constexpr int VE = 16 / sizeof(T);
     const bool kvec = (dim % VE == 0) && ((((size_t)cache) & 15) == 0);
     const bool pair = sizeof(T) == 2 && (vdim % 2 == 0) && (dim % 2 == 0);
     const size_t kld = (size_t)G * dim, vld = (size_t)G * vdim;
+    // the wave's part of the scores: head sh, dims sd0 .. sd1 (HPB = 3: the fourth wave has none)
+    const int sh = wv / DS, step = kvec ? VE : 1, per = (dim / step + DS - 1) / DS * step;
+    const int sd0 = wv % DS * per, sd1 = sd0 + per < dim ? sd0 + per : dim;
+    const float* qh = qs + (sh < HPB ? sh : 0) * dimp;
     float acc[HPB][HB_MAX_VPL];
 #pragma unroll
     for (int h = 0; h < HPB; ++h)
 #pragma unroll
         for (int e = 0; e < HB_MAX_VPL; ++e) acc[h][e] = 0.f;
-    long* wloc = loc + wv * 64;
-    float* wpw = pw + wv * 64 * HPB;
-    for (int c = c0 + wv; c < c1; c += NW) {
+    for (int c = c0; c < c1; ++c) {
         const int base = c * 64, cnt = total - base < 64 ? total - base : 64;
         const int t = lo + base + (lane < cnt ? lane : cnt - 1);
-        const long tok = (long)pt[t / ps] * ps + t % ps;
-        __builtin_amdgcn_wave_barrier();
-        wloc[lane] = tok;
-        const T* kr = cache + (size_t)tok * kld + (size_t)g * dim;
-        float dot[HPB];
+        const int tok = pt[t / ps] * ps + t % ps;
+        u32 v0[16];
+        if (pair) {
+            const T* vb = cache + v_base + (size_t)g * vdim + (2 * lane < vdim ? 2 * lane : vdim - 2);
 #pragma unroll
-        for (int h = 0; h < HPB; ++h) dot[h] = 0.f;
-        if (kvec) {
-#pragma unroll 4
-            for (int d = 0; d < dim; d += VE) {
-                const uint4 u = *(const uint4*)(kr + d);
-                float k[VE];
-                if (sizeof(T) == 2) {
-                    k[0] = bflo(u.x); k[1] = bfhi(u.x); k[2] = bflo(u.y); k[3] = bfhi(u.y);
-                    if (VE == 8) { k[VE - 4] = bflo(u.z); k[VE - 3] = bfhi(u.z); k[VE - 2] = bflo(u.w); k[VE - 1] = bfhi(u.w); }
-                } else {
-                    k[0] = __uint_as_float(u.x); k[1] = __uint_as_float(u.y); k[2] = __uint_as_float(u.z); k[3] = __uint_as_float(u.w);
-                }
-#pragma unroll
-                for (int h = 0; h < HPB; ++h)
-#pragma unroll
-                    for (int e = 0; e < VE; ++e) dot[h] = fmaf(qs[h * dimp + d + e], k[e], dot[h]);
-            }
-        } else {
-            for (int d = 0; d < dim; ++d) {
-                const float k = hb_ld(kr + d);
-#pragma unroll
-                for (int h = 0; h < HPB; ++h) dot[h] = fmaf(qs[h * dimp + d], k, dot[h]);
-            }
+            for (int x = 0; x < 16; ++x) v0[x] = *(const u32*)(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
         }
+        if (sh < HPB) {
+            const T* kr = cache + (size_t)tok * kld + (size_t)g * dim;
+            float dot = 0.f;
+            if (kvec) {
+#pragma unroll 8
+                for (int d = sd0; d < sd1; d += VE) {
+                    const uint4 u = *(const uint4*)(kr + d);
+                    float k[VE];
+                    if (sizeof(T) == 2) {
+                        k[0] = bflo(u.x); k[1] = bfhi(u.x); k[2] = bflo(u.y); k[3] = bfhi(u.y);
+                        if (VE == 8) { k[VE - 4] = bflo(u.z); k[VE - 3] = bfhi(u.z); k[VE - 2] = bflo(u.w); k[VE - 1] = bfhi(u.w); }
+                    } else {
+                        k[0] = __uint_as_float(u.x); k[1] = __uint_as_float(u.y); k[2] = __uint_as_float(u.z); k[3] = __uint_as_float(u.w);
+                    }
 #pragma unroll
-        for (int h = 0; h < HPB; ++h) wpw[lane * HPB + h] = lane < cnt ? hb_sig_weight(sc, h0 + h, dot[h], p - t) : 0.f;
-        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-        __builtin_amdgcn_wave_barrier();
+                    for (int e = 0; e < VE; ++e) dot = fmaf(qh[d + e], k[e], dot);
+                }
+            } else {
+                for (int d = sd0; d < sd1; ++d) dot = fmaf(qh[d], hb_ld(kr + d), dot);
+            }
+            dots[wv * 64 + lane] = dot;
+        }
+        if (DS > 1) __syncthreads();
+        if (wv % DS == 0 && sh < HPB) {
+            float dot = dots[wv * 64 + lane];
+#pragma unroll
+            for (int x = 1; x < DS; ++x) dot += dots[(wv + x) * 64 + lane];
+            pw[lane * HPB + sh] = lane < cnt ? hb_sig_weight(sc, h0 + sh, dot, p - t) : 0.f;
+        }
+        __syncthreads();
+        const float* wpw = pw + wv * 16 * HPB;      // (weights behind the last key are zero)
         if (pair) {
 #pragma unroll
             for (int cc = 0; cc < HB_MAX_VPL / 2; ++cc) {
                 if (cc * 128 < vdim) {
-                    const int j = cc * 128 + 2 * lane, jj = j < vdim ? j : vdim - 2;
-                    const T* vb = cache + v_base + (size_t)g * vdim + jj;
-                    for (int k0 = 0; k0 < cnt; k0 += 16) {
-                        u32 vv[16];
+                    if (cc > 0) {
+                        const int j = cc * 128 + 2 * lane;
+                        const T* vb = cache + v_base + (size_t)g * vdim + (j < vdim ? j : vdim - 2);
 #pragma unroll
-                        for (int x = 0; x < 16; ++x) vv[x] = *(const u32*)(vb + (size_t)wloc[k0 + x < cnt ? k0 + x : cnt - 1] * vld);
-#pragma unroll
-                        for (int x = 0; x < 16; ++x)
-#pragma unroll
-                            for (int h = 0; h < HPB; ++h) {
-                                const float w = wpw[(k0 + x) * HPB + h];        // (zero behind the last key)
-                                acc[h][2 * cc] = fmaf(w, bflo(vv[x]), acc[h][2 * cc]);
-                                acc[h][2 * cc + 1] = fmaf(w, bfhi(vv[x]), acc[h][2 * cc + 1]);
-                            }
+                        for (int x = 0; x < 16; ++x) v0[x] = *(const u32*)(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
                     }
+#pragma unroll
+                    for (int x = 0; x < 16; ++x)
+#pragma unroll
+                        for (int h = 0; h < HPB; ++h) {
+                            acc[h][2 * cc] = fmaf(wpw[x * HPB + h], bflo(v0[x]), acc[h][2 * cc]);
+                            acc[h][2 * cc + 1] = fmaf(wpw[x * HPB + h], bfhi(v0[x]), acc[h][2 * cc + 1]);
+                        }
                 }
             }
         } else {
 #pragma unroll
             for (int cc = 0; cc < HB_MAX_VPL; ++cc) {
                 if (cc * 64 < vdim) {
-                    const int j = cc * 64 + lane, jj = j < vdim ? j : vdim - 1;
-                    const T* vb = cache + v_base + (size_t)g * vdim + jj;
-                    for (int k0 = 0; k0 < cnt; k0 += 8) {
-                        float vv[8];
+                    const int j = cc * 64 + lane;
+                    const T* vb = cache + v_base + (size_t)g * vdim + (j < vdim ? j : vdim - 1);
+                    float vv[16];
 #pragma unroll
-                        for (int x = 0; x < 8; ++x) vv[x] = hb_ld(vb + (size_t)wloc[k0 + x < cnt ? k0 + x : cnt - 1] * vld);
+                    for (int x = 0; x < 16; ++x) vv[x] = hb_ld(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
 #pragma unroll
-                        for (int x = 0; x < 8; ++x)
+                    for (int x = 0; x < 16; ++x)
 #pragma unroll
-                            for (int h = 0; h < HPB; ++h) acc[h][cc] = fmaf(wpw[(k0 + x) * HPB + h], vv[x], acc[h][cc]);
-                    }
+                        for (int h = 0; h < HPB; ++h) acc[h][cc] = fmaf(wpw[x * HPB + h], vv[x], acc[h][cc]);
                 }
             }
         }
-        __builtin_amdgcn_wave_barrier();
+        __syncthreads();
     }
     float* mine = red + (size_t)wv * HPB * vdim;
 #pragma unroll
@@ -3010,9 +3105,9 @@ __global__ __launch_bounds__(1024) void k_hb_sig_attn_rows(const float* q, long 
             if (j < vdim) mine[h * vdim + j] = acc[h][e];
         }
     __syncthreads();
-    for (int i = tid; i < HPB * vdim; i += blockDim.x) {
-        float a = 0.f;
-        for (int w = 0; w < NW; ++w) a += red[(size_t)w * HPB * vdim + i];
+    const int nv = HPB * vdim;
+    for (int i = tid; i < nv; i += 256) {
+        float a = ((red[i] + red[nv + i]) + red[2 * nv + i]) + red[3 * nv + i];
         const int h = h0 + i / vdim, j = i % vdim;
         if (part) { part[((size_t)(row * H + h) * gridDim.z + blockIdx.z) * vdim + j] = a; continue; }
         a *= out_scale;
@@ -3028,6 +3123,7 @@ __global__ __launch_bounds__(64) void k_hb_sig_merge(const float* part, int nseg
     const float* src = part + (size_t)(row * H + h) * nseg_grid * vdim;
     for (int j = threadIdx.x; j < vdim; j += 64) {
         float a = 0.f;
+#pragma unroll 8
         for (int s = 0; s < nseg; ++s) a += src[(size_t)s * vdim + j];
         a *= out_scale;
         if (gate) a *= hb_sigmoid(gate[(size_t)row * ldg + h * vdim + j]);
@@ -3038,48 +3134,57 @@ __global__ __launch_bounds__(64) void k_hb_sig_merge(const float* part, int nseg
 // cached (Kt[key][dim]), values transposed two keys at a time (Vt[column][key]); the next tile's requests are on their way while a tile is
 // multiplied.  Per tile and wave, rows being the 16 columns of both products:
 //   S^T[key][row] = sum_dim Kt[key][dim] Q[row][dim]     v_mfma_f32_16x16x32_bf16, the query in registers as two bf16 parts (hi + lo)
-//   weights of the lane's 16 (key, row) pairs, fp32; masked pairs 0
+//   weights of the lane's 16 (key, row) pairs, fp32; masked pairs 0.  With a = cap (1 - tanh) folded into a table over distances:
+//   weight = 1 / (1 + 2^(table[d] + k2 / (1 + 2^(k1 score)))), from the hardware's exponential and reciprocal (a few 1e-6 relative)
 //   O^T[col][row] += sum_key Vt[col][key] P[row][key]    the weights as they sit in the lanes (k index laid out to match), hi + lo
 // Row tiles of the launch are found by walking the requests' row counts; blocks beyond the last tile leave.  KS 32-dim steps of the key
 // and CT 16-column tiles of the value at most.
 #define HB_SIG_VLD 76        // keys per row of the transposed value tile (64 + 12: rows 8 bytes aligned, eight rows 16 banks apart)
 #define HB_SIG_DIST_LDS 4096 // distance biases per head that are kept in LDS
-// tanh and the logistic function from the hardware's exponential and reciprocal: absolute error of a few 1e-7
-__device__ __forceinline__ float hb_fast_tanh(float x) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(__expf(2.0f * x) + 1.0f); }
-__device__ __forceinline__ float hb_fast_sigmoid(float x) { return __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
 template <int KS, int CT>
 __global__ __launch_bounds__(256) void k_hb_sig_attn_mfma(const float* q, long ldq, const bf16_t* cache, float* out, long ldo, const int* pos,
                                                           const int* req_rows, int n_req, const int* ptab, int pts, int H, int G, int dim, int vdim,
                                                           int ps, long v_base, hb_sig_score sc, const float* gate, long ldg, float out_scale,
-                                                          int ks_n, int ct_n) {
+                                                          int ks_n, int ct_n, int fold) {
     extern __shared__ float sm[];
     const int DPK = ks_n * 32 + 8;
     const int nbias = sc.dist && sc.dist_n <= HB_SIG_DIST_LDS ? sc.dist_n : 0;
     bf16_t* Kt = (bf16_t*)sm;                            // [64][DPK]
     bf16_t* Vt = Kt + 64 * DPK;                          // [ct_n * 16][HB_SIG_VLD]
-    float* sbias = (float*)(Vt + ct_n * 16 * HB_SIG_VLD);   // [nbias]
+    float* tab = (float*)(Vt + ct_n * 16 * HB_SIG_VLD);   // [nbias]
     const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, col = lane & 15, g4 = lane >> 4;
-    int t = blockIdx.x, rq = -1, rs = 0, re = 0;
+    // Blocks in launch order: all heads of a tile, then the next tile.  Later rows of a request see more keys, so their tiles start first;
+    // a launch that fits the chip at once (fold) follows the heavier half in descending order with the lighter half in ascending order:
+    // the two blocks that share a compute unit have about the same work together everywhere.
+    const int nt_all = gridDim.y, half = (nt_all + 1) >> 1;
+    int t = nt_all - 1 - (int)blockIdx.y, rq = -1, rs = 0, re = 0;
+    if (fold && (int)blockIdx.y >= half) t = (int)blockIdx.y - half;
     for (int r = 0; r < n_req; ++r) {
         const int a = req_rows[r], b = req_rows[r + 1], nt = (b - a + 63) >> 6;
         if (t < nt) { rq = r; rs = a + 64 * t; re = b; break; }
         t -= nt;
     }
     if (rq < 0) return;
-    const int h = blockIdx.y, g = h / (H / G);
+    const int h = blockIdx.x, g = h / (H / G);
     const int nrows = re - rs < 64 ? re - rs : 64;
     const int w0 = wv * 16, wn = nrows - w0 < 16 ? nrows - w0 : 16;      // the wave's rows: w0 .. w0 + wn - 1 of the tile (wn may be <= 0)
     const bool active = wn > 0;
     const bool rowok = col < wn;
-    const int row = rs + (rowok ? w0 + col : 0);
+    const int row = rs + (active ? w0 + (rowok ? col : wn - 1) : 0);      // (a lane without a row follows the wave's last one)
     const int p = pos[row], lo_r = hb_chunk_start(p, sc.chunk);
     const int p0 = pos[rs], pl = pos[rs + nrows - 1];
     const int wp_lo = active ? hb_chunk_start(pos[rs + w0], sc.chunk) : 0, wp_hi = active ? pos[rs + w0 + wn - 1] : -1;
     const int lo_t = hb_chunk_start(p0, sc.chunk), ntiles = (pl - lo_t + 64) >> 6;
     const int* pt = ptab + (size_t)rq * pts;
     const float zmul = sc.temp ? sc.scale * sc.temp[h] : sc.scale, wbias = sc.wb ? sc.wb[h] : 0.f;
-    const float icap = sc.cap > 0.f ? 1.0f / sc.cap : 0.f;
-    for (int i = tid; i < nbias; i += 256) sbias[i] = sc.dist[(size_t)h * sc.dist_n + i];
+    const bool capped = sc.cap > 0.f;
+    constexpr float LOG2E = 1.44269504088896340736f;
+    // the exponent of the weight's denominator: -log2(e) (z + wbias), z = cap - 2 cap / (1 + e^(2 s / cap)) + dist
+    const float k1 = capped ? 2.0f * LOG2E * zmul / sc.cap : -LOG2E * zmul, k2 = 2.0f * LOG2E * sc.cap;
+    const float flat = -LOG2E * ((capped ? sc.cap : 0.f) + wbias);
+    for (int i = tid; i < nbias; i += 256) tab[i] = flat - LOG2E * sc.dist[(size_t)h * sc.dist_n + i];
+    const int wp_in = active ? hb_chunk_start(wp_hi, sc.chunk) : 0;      // keys from here on are in the chunk of every row of the wave
+    const int wp_first = active ? pos[rs + w0] : 0;
     uint4 qh[KS], ql[KS];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -3164,20 +3269,32 @@ __global__ __launch_bounds__(256) void k_hb_sig_attn_mfma(const float* q, long l
         }
         // lane (col, g4) holds the scores of row `col` against keys base + kt*16 + g4*4 + i
         float pr[4][4];
+        auto weight = [&](float s, float tb) {
+            const float e = capped ? fmaf(__builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * k1) + 1.0f), k2, tb) : fmaf(s, k1, tb);
+            return __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(e) + 1.0f);
+        };
+        if (base >= wp_in && base + 63 <= wp_first && nbias > wp_hi - base) {
+            // every row of the wave sees the whole tile and every distance has its table entry
+            const float* tb = tab + (p - base - g4 * 4);
 #pragma unroll
-        for (int kt = 0; kt < 4; ++kt)
+            for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int key = base + kt * 16 + g4 * 4 + i;
-                float z = st[kt][i] * zmul;
-                if (icap > 0.f) z = sc.cap * hb_fast_tanh(z * icap);
-                if (sc.dist) {
-                    int d = p - key;
-                    d = d < 0 ? 0 : (d < sc.dist_n ? d : sc.dist_n - 1);
-                    z += nbias ? sbias[d] : sc.dist[(size_t)h * sc.dist_n + d];
+                for (int i = 0; i < 4; ++i) pr[kt][i] = weight(st[kt][i], tb[-(kt * 16 + i)]);
+        } else {
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int key = base + kt * 16 + g4 * 4 + i;
+                    float tb = flat;
+                    if (sc.dist) {
+                        int d = p - key;
+                        d = d < 0 ? 0 : (d < sc.dist_n ? d : sc.dist_n - 1);
+                        tb = nbias ? tab[d] : flat - LOG2E * sc.dist[(size_t)h * sc.dist_n + d];
+                    }
+                    pr[kt][i] = key >= lo_r && key <= p ? weight(st[kt][i], tb) : 0.f;
                 }
-                pr[kt][i] = key >= lo_r && key <= p ? hb_fast_sigmoid(z + wbias) : 0.f;
-            }
+        }
         uint4 ph[2], plo[2];
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
@@ -3477,6 +3594,7 @@ __global__ __launch_bounds__(256) void k_hb_moe_down_combine(const float* h, lon
     const int row = blockIdx.y, lane = threadIdx.x & 63, c = blockIdx.x * 4 + (threadIdx.x >> 6);
     if (c >= W) return;
     constexpr int CH = sizeof(T) == 2 ? 8 : 4;
+    const hb_join_in jin = hb_join_load(q.join, x + (size_t)row * ldx, row, c);
     const bool avec = (q.ld_act % 4 == 0) && ((((size_t)act) & 15) == 0);
     float acc = 0.f;
     for (int k = 0; k < q.top; ++k) {
@@ -3492,7 +3610,7 @@ __global__ __launch_bounds__(256) void k_hb_moe_down_combine(const float* h, lon
         const bool vec = avec && (q.shared_ff % CH == 0) && ((((size_t)shared_down) & 15) == 0);
         acc += hb_dot_wave<T>(shared_down + (size_t)c * q.shared_ff, act + (size_t)(row * per + q.top) * q.ld_act, q.shared_ff, vec, lane);
     }
-    if (lane == 0) hb_join_add(q.join, x + (size_t)row * ldx, row, c, acc);
+    if (lane == 0) hb_join_apply(q.join, jin, x + (size_t)row * ldx, row, c, acc);
 }
 // x[row] += sum_k wgt[row*top + k] * (identity output ? h[row] : expert_out[row*top + k]), k ascending
 // (scale_input: an expert's output enters with weight 1, its input was scaled instead)
@@ -3744,12 +3862,13 @@ static bool hb_try_sig_mfma(hipStream_t st, const vox_hybrid_io* io, const vox_h
     const int ks_n = (L.dim + 31) / 32, ct_n = (L.vdim + 15) / 16;
     const int nbias = sc.dist && sc.dist_n <= HB_SIG_DIST_LDS ? sc.dist_n : 0;
     const size_t lds = (size_t)64 * (ks_n * 32 + 8) * 2 + (size_t)ct_n * 16 * HB_SIG_VLD * 2 + (size_t)nbias * 4;
-    const dim3 grid((n + 63) / 64 + n_req, L.heads), block(256);
+    const dim3 grid(L.heads, (n + 63 * n_req) / 64), block(256);      // (at least the sum of the requests' tiles)
+    const int fold = grid.x * grid.y <= 2 * 256 ? 1 : 0;
 #define HB_SM(KS_, CT_) \
     do { \
         if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_sig_attn_mfma<KS_, CT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
         hipLaunchKernelGGL((k_hb_sig_attn_mfma<KS_, CT_>), grid, block, lds, st, q, ldp, cache, out, ldo, io->pos, io->req_rows, n_req, io->page_table, \
-                           io->pt_stride, L.heads, L.kv_heads, L.dim, L.vdim, ps, v_base, sc, gate, ldp, L.out_scale, ks_n, ct_n); \
+                           io->pt_stride, L.heads, L.kv_heads, L.dim, L.vdim, ps, v_base, sc, gate, ldp, L.out_scale, ks_n, ct_n, fold); \
     } while (0)
     if (ks_n <= 4 && ct_n <= 8) HB_SM(4, 8);
     else HB_SM(8, 16);
@@ -3765,9 +3884,10 @@ static int hb_sig_heads(const vox_hybrid_layer& L) {
         if (qg % h == 0) return h;
     return 1;
 }
-#define HB_SIG_SEG 16     // 64-key chunks per block of the few-row sigmoid attention (one per wave)
-static size_t hb_sig_lds(const vox_hybrid_layer& L, int hpb, int nw) {
-    return (size_t)(nw * 128 + nw * 64 * hpb + hpb * ((L.dim + 3) & ~3) + nw * hpb * L.vdim) * 4;
+#define HB_SIG_MAX_SEG 64     // blocks that share the keys of one row and head in the few-row sigmoid attention
+static int hb_sig_segments(int max_keys) {
+    const int nchunks = (max_keys + 63) / 64;
+    return nchunks < HB_SIG_MAX_SEG ? nchunks : HB_SIG_MAX_SEG;
 }
 template <typename T>
 static int hb_sig_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const T* cache, long ldp, int n, int n_req,
@@ -3778,14 +3898,13 @@ static int hb_sig_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* 
     const bool few = n <= HB_ATTN_SEG_ROWS;
     if (!few && hb_try_sig_mfma(st, io, L, cache, m->proj, ldp, m->mix, (long)n_mix, sc, gate, v_base, n, n_req, ps)) return VOX_OK;
     const int hpb = hb_sig_heads(L);
-    int nw = few ? 16 : 4;
-    while (nw > 1 && hb_sig_lds(L, hpb, nw) > 64 * 1024) nw >>= 1;
     const int max_keys = L.chunk > 0 && L.chunk < max_kvlen ? L.chunk : max_kvlen, nchunks = (max_keys + 63) / 64;
-    const int cpb = few ? HB_SIG_SEG : nchunks, nseg = (nchunks + cpb - 1) / cpb;
+    const int want = few ? hb_sig_segments(max_keys) : 1, cpb = (nchunks + want - 1) / want, nseg = (nchunks + cpb - 1) / cpb;
     if (nseg > 1 && (size_t)n * H * nseg * L.vdim * 4 > m->attn_ws_bytes) return vox_fail(VOX_ERR_INVALID, "hybrid_step: attention workspace");
     float* part = nseg > 1 ? m->attn_ws : nullptr;
+    const size_t lds = (size_t)(hpb * ((L.dim + 3) & ~3) + 256 + 64 * hpb + 4 * hpb * L.vdim) * 4;
 #define HB_SR(HPB_) \
-    hipLaunchKernelGGL((k_hb_sig_attn_rows<T, HPB_>), dim3(n, H / HPB_, nseg), dim3(64 * nw), hb_sig_lds(L, HPB_, nw), st, m->proj, ldp, cache, m->mix, \
+    hipLaunchKernelGGL((k_hb_sig_attn_rows<T, HPB_>), dim3(n, H / HPB_, nseg), dim3(256), lds, st, m->proj, ldp, cache, m->mix, \
                        (long)n_mix, io->pos, io->row_req, io->page_table, io->pt_stride, H, G, L.dim, L.vdim, ps, v_base, sc, cpb, part, gate, ldp, \
                        L.out_scale)
     if (hpb == 4) HB_SR(4);
@@ -4441,8 +4560,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
     for (const vox_hybrid_layer& L : m->layers)
         if (L.kind == VOX_MIXER_SIGMOID_ATTN) {
             const int max_keys = L.chunk > 0 && L.chunk < cfg->max_seq_len ? L.chunk : cfg->max_seq_len;
-            const size_t nseg = ((size_t)(max_keys + 63) / 64 + HB_SIG_SEG - 1) / HB_SIG_SEG;
-            const size_t b = (size_t)HB_ATTN_SEG_ROWS * L.heads * nseg * L.vdim * 4;
+            const size_t b = (size_t)HB_ATTN_SEG_ROWS * L.heads * hb_sig_segments(max_keys) * L.vdim * 4;
             if (b > m->attn_ws_bytes) m->attn_ws_bytes = b;
         } else if (hb_is_attn(L.kind)) {
             const bool causal = L.kind == VOX_MIXER_CAUSAL_ATTN, latent = L.kind == VOX_MIXER_LATENT_ATTN;

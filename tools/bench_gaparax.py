@@ -6,7 +6,7 @@ one GPU; both are driven directly (plan upload + one native step).
 
 Gaparax layers per block of four: latent attention (heads = width/128 of 128 plain + 64 rotated dims, values of 128, cached latent
 width/4 + 64 rotated key dims, scaled rotary) with a dense relu-squared feed-forward of 4 x width | latent attention with a routed
-feed-forward of 8 experts in 4 groups of which 3 are kept, 2 per token, expert width = width | sigmoid-weighted attention (heads = width/128 on a quarter as
+feed-forward of 8 experts in 4 groups of which 2 are kept, 2 per token, expert width = width | sigmoid-weighted attention (heads = width/128 on a quarter as
 many key heads, 128 dims, chunks of 2048 positions, distance biases up to 2048) with the dense feed-forward | the same with the routed
 one.  Two residual streams, a gate of width x width on every sublayer.  Vocabulary 32 000.  Prints one JSON object.
 """
@@ -27,17 +27,17 @@ def gaparax_cfg(width, blocks, vocab, experts=8, top=2, chunk=2048):
 
     def moe():
         return dict(moe=MoECfg(experts=experts, identity=0, top=top, ff=width, limit=float("inf"), act_alpha=1.0, score="softmax", renorm=False,
-                               up_offset=0.0, groups=4, keep=3, weight_scale=2.5))
+                               up_offset=0.0, groups=4, keep=2, weight_scale=1.5))
 
     def dense():
         return dict(ff=4 * width, ff_kind="up_down", ff_act="relu2")
 
     def lat(ff):
-        return MixerCfg("latent_attention", h, 128, 128, kv_rank=width // 4, rot_dim=64, rot_dims=64, rot_base=5e4, rot_yarn=(4.0, 1024.0, 32.0, 1.0),
+        return MixerCfg("latent_attention", h, 128, 128, kv_rank=width // 4, rot_dim=64, rot_dims=64, rot_base=1e5, rot_yarn=(8.0, 4096.0, 24.0, 2.0),
                         scale=192 ** -0.5, head_gate=False, res_gate=True, **ff)
 
     def sig(ff):
-        return MixerCfg("sigmoid_attention", h, 128, 128, kv_heads=max(1, h // 4), chunk=chunk, score_cap=50.0, dist_max=chunk, scale=128 ** -0.5,
+        return MixerCfg("sigmoid_attention", h, 128, 128, kv_heads=max(1, h // 4), chunk=chunk, score_cap=30.0, dist_max=chunk, scale=128 ** -0.5,
                         out_gate=True, res_gate=True, **ff)
     layers = []
     for _ in range(blocks):

@@ -357,8 +357,9 @@ int vox_lm_prefill(vox_lm* m, void* stream, const vox_lm_io* io, const int32_t* 
  * A decoder whose layers mix tokens with a linear recurrence (HGRN2, mLSTM, a real-gated diagonal unit behind a short
  * convolution, a matrix state with token shift and per-channel decay, retention, the gated delta rule) or with attention
  * over a paged cache (a sliding window that also keeps one mean key / value per block of older tokens, plain causal
- * attention with normed q / k / v, attention over a cached low-rank latent, or attention whose key weights are independent
- * sigmoids inside position chunks); two mixers may run side by side on the
+ * attention with normed q / k / v, attention over a cached low-rank latent, attention whose key weights are independent
+ * sigmoids inside position chunks, or softmax attention over a window and the first tokens, whose keys and values may be
+ * those of an earlier layer); two mixers may run side by side on the
  * same input; a layer's outputs may carry a layer scale; a contiguous range of layers may run several times with the
  * same weights (every run owns its cache or state).  A layer is sequential (x += mixer(norm1 x); x += ff(norm2 x)) or
  * parallel (x += mixer(norm1 x) + ff(norm2 x)); the feed-forward is dense or a routed mixture of experts.  Residual
@@ -368,12 +369,12 @@ int vox_lm_prefill(vox_lm* m, void* stream, const vox_lm_io* io, const int32_t* 
 typedef struct vox_hybrid vox_hybrid;
 enum { VOX_MIXER_HGRN2 = 0, VOX_MIXER_POOLED_WINDOW_ATTN = 1, VOX_MIXER_MLSTM = 2, VOX_MIXER_RGLRU = 3, VOX_MIXER_CAUSAL_ATTN = 4,
        VOX_MIXER_SHIFT_DECAY = 5, VOX_MIXER_LATENT_ATTN = 6, VOX_MIXER_RETENTION = 7, VOX_MIXER_DELTA = 8,
-       VOX_MIXER_SIGMOID_ATTN = 9 };
+       VOX_MIXER_SIGMOID_ATTN = 9, VOX_MIXER_WINDOW_ATTN = 10 };
 enum { VOX_HYBRID_BF16 = 0, VOX_HYBRID_F32 = 1 };
-enum { VOX_NORM_LAYER = 0 /* weight-only layer norm */, VOX_NORM_RMS_GROUPS = 1 /* RMS norm over norm_groups equal slices */ };
+enum { VOX_NORM_LAYER = 0 /* layer norm with a weight and an optional bias */, VOX_NORM_RMS_GROUPS = 1 /* RMS norm over norm_groups equal slices */ };
 /* sequential: x += mixer(norm1 x); x += ff(norm2 x).  parallel: x += mixer(norm1 x) + ff(norm2 x).  parallel, one norm:
- * x += mixer(n) + ff(n) with n = norm1 x (norm2 is not used) */
-enum { VOX_BLOCK_SEQUENTIAL = 0, VOX_BLOCK_PARALLEL = 1, VOX_BLOCK_PARALLEL_ONE_NORM = 2 };
+ * x += mixer(n) + ff(n) with n = norm1 x (norm2 is not used).  post-normed: x += norm1 mixer(x); x += norm2 ff(x) */
+enum { VOX_BLOCK_SEQUENTIAL = 0, VOX_BLOCK_PARALLEL = 1, VOX_BLOCK_PARALLEL_ONE_NORM = 2, VOX_BLOCK_POST_NORM = 3 };
 enum { VOX_FF_UP_DOWN = 0 /* down(gelu_erf(up h)), with ff_act VOX_ACT_RELU2 down(max(up h, 0)^2) */, VOX_FF_GATED = 1 /* down(act(gate h + b) * (up h + b)) + b */ };
 enum { VOX_ACT_GELU_TANH = 0, VOX_ACT_SWISH = 1 /* g * sigmoid(alpha g) */, VOX_ACT_RELU2 = 2 /* max(g, 0)^2 */ };
 enum { VOX_EXPERT_GATED = 0 /* down(act(gate h) * (up h + up_offset)), clamped */, VOX_EXPERT_UP_DOWN = 1 /* down(act(up h)) */ };
@@ -403,6 +404,7 @@ typedef struct {
      * of the `keep` best groups can be chosen (identity = 0 then).  weight_scale multiplies the weights (0: as 1). */
     int32_t groups, keep;
     float weight_scale;
+    int32_t group_best_two;       /* a group's score is the sum of its two largest choice values instead */
 } vox_hybrid_moe;
 typedef struct {
     int32_t kind, heads, kv_heads, dim, vdim;
@@ -417,6 +419,7 @@ typedef struct {
      *   RGLRU         gated branch (C) | recurrent branch (C), C = heads*dim channels in `heads` blocks of dim (= vdim)
      *   causal attn   q (heads*dim) | k (kv_heads*dim) | v (kv_heads*vdim)
      *   sigmoid attn  q (heads*dim) | k (kv_heads*dim) | v (kv_heads*vdim) | output gate (heads*vdim; out_gate only)
+     *   window attn   q (heads*dim) | k (kv_heads*dim) | v (kv_heads*vdim) | output gate (heads*vdim; out_gate only); kv_shared: no k, no v
      *   shift-decay   r | k | v | g (heads*dim each, dim = vdim) | decay bottleneck (lora); each of the five reads its own token-shift mix */
     const void* w_in;                     /* [n_in, width] engine dtype */
     const float* b_in;                    /* [n_in] fp32 or NULL */
@@ -511,6 +514,16 @@ typedef struct {
     /* several residual streams (config.streams = s > 0): sublayer i (0 mixer, 1 feed-forward) reads u = sum hc_in[i][a] x_a and
      * leaves x_b <- sum hc_mix[i][a*s + b] x_a + hc_out[i][b] y, every new stream from the old ones; fp32 */
     const float *hc_in[2], *hc_out[2], *hc_mix[2];
+    /* window attention (VOX_MIXER_WINDOW_ATTN): a position sees the positions up to itself among the last `window` (0: all) and among the
+     * first keep_first of its sequence; q and k are RMS-normed over their whole projection (q_norm [heads*dim], k_norm [kv_heads*dim]),
+     * then the first rot_dims dims of every head rotated (interleaved pairs, cos and sin times rot_mag); softmax of (q . k) * scale with
+     * exp(sinks[h]) in the denominator (sinks NULL: none); out_gate: every output column times the sigmoid of its gate.  kv_shared: the
+     * layer has no keys and values of its own, the run's cache is that of an earlier run whose layer has the same kv_heads, dim and vdim. */
+    int32_t keep_first, kv_shared;
+    const float *norm1_b, *norm2_b;       /* [width] fp32 or NULL: biases of the layer norms */
+    /* gated dense feed-forward: down(g * sigmoid(alpha g) * (u + up_offset)) with g = min(gate h, limit), u = clamp(up h, -limit, limit);
+     * ff_limit 0: not clamped; ff_alpha 0: as 1 */
+    float ff_limit, ff_alpha, ff_up_offset;
 } vox_hybrid_layer;
 typedef struct {
     int32_t layer;       /* index into layers */
@@ -545,6 +558,7 @@ typedef struct {
     const float* final_norm;
     const void* bigram;                   /* [bigram_buckets + 1, width] or NULL */
     int32_t* prev_token;                  /* state, [slots]: the last token each slot's sequence has seen (bigram embedding) */
+    const float* final_norm_b;            /* [width] fp32 or NULL */
 } vox_hybrid_weights;
 typedef struct {
     const int32_t *pos, *row_req, *page, *slot;   /* per row: position, request index in this step, K/V page and slot */

@@ -111,6 +111,7 @@ struct hb_join {
     const float *mix, *out, *next;
     float* u;
     long ldu;
+    int store;      // one stream: v takes the place of what is there (a result that is normed before it joins)
 };
 // what a join reads of its place, requested ahead of the product by kernels that have nothing to do meanwhile
 struct hb_join_in {
@@ -121,7 +122,7 @@ __device__ __forceinline__ hb_join_in hb_join_load(const hb_join& j, const float
     in.gate = j.gate ? j.gate[(size_t)row * j.ldg + col] : 0.f;
 #pragma unroll
     for (int s = 0; s < HB_MAX_STREAMS; ++s) in.xs[s] = 0.f;
-    if (j.streams == 0) in.xs[0] = x[col];
+    if (j.streams == 0) in.xs[0] = j.store ? 0.f : x[col];
     else
 #pragma unroll
         for (int s = 0; s < HB_MAX_STREAMS; ++s)
@@ -244,12 +245,12 @@ __global__ void k_hb_store_prev(const int* ids, int id_stride, int vocab, const 
     if (r < n_req && req_rows[r + 1] > req_rows[r]) prev[req_state[r]] = hb_clamp_id(ids[(size_t)(req_rows[r + 1] - 1) * id_stride], vocab);
 }
 
-// ---- layer norm with a weight and no bias, fp32; optional row gather ----------------------------------------------------
+// ---- layer norm with a weight and an optional bias, fp32; optional row gather --------------------------------------------
 // mean, then the mean of the squared deviations (two passes over the row).  NV > 0: the row (width <= 256 * NV) is read once
 // into registers; NV = 0: any width, three reads.  Same sums in the same order either way.
 template <int NV>
-__global__ __launch_bounds__(256) void k_hb_layernorm(const float* x, long ldx, const int* rows, const float* w, float* y, long ldy, int W,
-                                                      float eps) {
+__global__ __launch_bounds__(256) void k_hb_layernorm(const float* x, long ldx, const int* rows, const float* w, const float* b, float* y,
+                                                      long ldy, int W, float eps) {
     __shared__ float red[2][4];
     const int r = blockIdx.x, src = rows ? rows[r] : r;
     const float* xr = x + (size_t)src * ldx;
@@ -293,16 +294,85 @@ __global__ __launch_bounds__(256) void k_hb_layernorm(const float* x, long ldx, 
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
             const int k = threadIdx.x + i * 256;
-            if (k < W) y[(size_t)r * ldy + k] = (xv[i] - mean) * inv * w[k];
+            if (k < W) y[(size_t)r * ldy + k] = (xv[i] - mean) * inv * w[k] + (b ? b[k] : 0.f);
         }
     } else {
-        for (int i = threadIdx.x; i < W; i += 256) y[(size_t)r * ldy + i] = (xr[i] - mean) * inv * w[i];
+        for (int i = threadIdx.x; i < W; i += 256) y[(size_t)r * ldy + i] = (xr[i] - mean) * inv * w[i] + (b ? b[i] : 0.f);
     }
 }
-static void hb_layernorm(hipStream_t st, int n, const float* x, long ldx, const int* rows, const float* w, float* y, long ldy, int W, float eps) {
-    if (W <= 1024) hipLaunchKernelGGL(k_hb_layernorm<4>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, y, ldy, W, eps);
-    else if (W <= 4096) hipLaunchKernelGGL(k_hb_layernorm<16>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, y, ldy, W, eps);
-    else hipLaunchKernelGGL(k_hb_layernorm<0>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, y, ldy, W, eps);
+static void hb_layernorm(hipStream_t st, int n, const float* x, long ldx, const int* rows, const float* w, const float* b, float* y, long ldy, int W,
+                         float eps) {
+    if (W <= 1024) hipLaunchKernelGGL(k_hb_layernorm<4>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, b, y, ldy, W, eps);
+    else if (W <= 4096) hipLaunchKernelGGL(k_hb_layernorm<16>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, b, y, ldy, W, eps);
+    else hipLaunchKernelGGL(k_hb_layernorm<0>, dim3(n), dim3(256), 0, st, x, ldx, rows, w, b, y, ldy, W, eps);
+}
+
+// ---- norm of a sublayer's output, added to the residual row: x += norm(y) * w + b ------------------------------------------------
+// The layer norm above, or (rms) the RMS norm over the row; 256 threads per row.  NV > 0: the row (width <= 256 * NV) stays in registers.
+struct hb_post {
+    const float* y;         // [rows][ldy] the sublayer's output (NULL: nothing to do)
+    long ldy;
+    const float *w, *b;
+    float eps;
+    int rms;
+};
+template <int NV> __device__ __forceinline__ void hb_post_norm_row(const hb_post& p, int row, float* xr, int W, float (*red)[4]) {
+    const float* yr = p.y + (size_t)row * p.ldy;
+    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    float yv[NV > 0 ? NV : 1];
+    float s = 0.f, q = 0.f;
+    if (NV > 0) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int k = threadIdx.x + i * 256;
+            yv[i] = k < W ? yr[k] : 0.f;
+        }
+#pragma unroll
+        for (int i = 0; i < NV; ++i) s += yv[i];
+    } else {
+        for (int i = threadIdx.x; i < W; i += 256) s += yr[i];
+    }
+    float mean = 0.f;
+    if (!p.rms) {
+        s = hb_wave_sum(s);
+        if (lane == 0) red[0][wv] = s;
+        __syncthreads();
+        mean = (((red[0][0] + red[0][1]) + red[0][2]) + red[0][3]) / (float)W;
+    }
+    if (NV > 0) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const float d = threadIdx.x + i * 256 < W ? yv[i] - mean : 0.f;
+            q += d * d;
+        }
+    } else {
+        for (int i = threadIdx.x; i < W; i += 256) {
+            const float d = yr[i] - mean;
+            q += d * d;
+        }
+    }
+    q = hb_wave_sum(q);
+    if (lane == 0) red[1][wv] = q;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((((red[1][0] + red[1][1]) + red[1][2]) + red[1][3]) / (float)W + p.eps);
+    if (NV > 0) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int k = threadIdx.x + i * 256;
+            if (k < W) xr[k] += (yv[i] - mean) * inv * p.w[k] + (p.b ? p.b[k] : 0.f);
+        }
+    } else {
+        for (int i = threadIdx.x; i < W; i += 256) xr[i] += (yr[i] - mean) * inv * p.w[i] + (p.b ? p.b[i] : 0.f);
+    }
+}
+template <int NV> __global__ __launch_bounds__(256) void k_hb_post_norm(hb_post p, float* x, long ldx, int W) {
+    __shared__ float red[2][4];
+    hb_post_norm_row<NV>(p, blockIdx.x, x + (size_t)blockIdx.x * ldx, W, red);
+}
+static void hb_post_norm(hipStream_t st, int n, const hb_post& p, float* x, long ldx, int W) {
+    if (W <= 1024) hipLaunchKernelGGL(k_hb_post_norm<4>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
+    else if (W <= 4096) hipLaunchKernelGGL(k_hb_post_norm<16>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
+    else hipLaunchKernelGGL(k_hb_post_norm<0>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
 }
 
 // ---- RMS norm over `groups` equal consecutive slices of the row, fp32; optional row gather; one or two weights --------------
@@ -665,15 +735,15 @@ __global__ __launch_bounds__(256) void k_hb_gemv(const float* A, long lda, const
         }
 }
 
-// One-row steps: the norm of the row (weight-only LayerNorm; rms != 0: the RMS norm over the whole row) fused in front of the GEMV.
+// One-row steps: the norm of the row (LayerNorm with a weight and, lnb != NULL, a bias; rms != 0: the RMS norm over the whole row) fused in front of the GEMV.
 // Every wave takes the row's statistics itself (mean, then the mean of the squared deviations; lane-chunked sums and a butterfly, an
 // order fixed by K), so the row is read from cache instead of from a normalised copy, and a dependent launch is saved.  NK > 0: a
 // lane's share of the row and of its weight rows (K <= 64 * CH * NK) is requested at the start and kept in registers, so the weights
 // are on their way while the statistics are taken; NK = 0: any K, several reads.  Same sums in the same order either way.  Needs
 // K % 8 == 0 (4 for fp32).
 template <typename T, int EPI, int CPW, int NK>
-__global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, const int* rows, const float* lnw, float eps, const T* Wt,
-                                                    const float* bias, float* C, int N, int K, int rms, float epi_arg) {
+__global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, const int* rows, const float* lnw, const float* lnb, float eps,
+                                                    const T* Wt, const float* bias, float* C, int N, int K, int rms, float epi_arg) {
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CPW;
     if (n0 >= N) return;
     constexpr int CH = sizeof(T) == 2 ? 8 : 4, NR = NK > 0 ? NK : 1;
@@ -727,8 +797,9 @@ __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, co
 #pragma unroll
         for (int e = 0; e < CH; e += 4) {
             const float4 x4 = xv[e / 4], g4 = *(const float4*)(lnw + k + e);
-            const float x[4] = {hb_operand<T>((x4.x - mean) * inv * g4.x), hb_operand<T>((x4.y - mean) * inv * g4.y),
-                                hb_operand<T>((x4.z - mean) * inv * g4.z), hb_operand<T>((x4.w - mean) * inv * g4.w)};
+            const float4 b4 = lnb ? *(const float4*)(lnb + k + e) : make_float4(0.f, 0.f, 0.f, 0.f);
+            const float x[4] = {hb_operand<T>((x4.x - mean) * inv * g4.x + b4.x), hb_operand<T>((x4.y - mean) * inv * g4.y + b4.y),
+                                hb_operand<T>((x4.z - mean) * inv * g4.z + b4.z), hb_operand<T>((x4.w - mean) * inv * g4.w + b4.w)};
 #pragma unroll
             for (int j = 0; j < CPW; ++j) {
                 const uint4 v = u[j];
@@ -776,18 +847,18 @@ __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, co
 // true: the fused form was launched (one row, aligned operands); false: the caller normalises and multiplies in two launches
 template <typename T>
 bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int* rows, const float* lnw, float eps, const T* W, const float* bias,
-                    float* C, int N, int K, int rms = 0, float epi_arg = 0.f) {
+                    float* C, int N, int K, int rms = 0, float epi_arg = 0.f, const float* lnb = nullptr) {
     constexpr int CH = sizeof(T) == 2 ? 8 : 4;
-    if (K % CH || (ldx & 3) || ((size_t)X & 15) || ((size_t)W & 15) || ((size_t)lnw & 15)) return false;
+    if (K % CH || (ldx & 3) || ((size_t)X & 15) || ((size_t)W & 15) || ((size_t)lnw & 15) || ((size_t)lnb & 15)) return false;
     const bool wide = N >= 16 * 1024;
     const dim3 g(wide ? (N + 15) / 16 : (N + 3) / 4), b(256);
     const int nk = (K + 64 * CH - 1) / (64 * CH);
 #define HB_LN2(EPI_, CPW_) \
     do { \
-        if (nk <= 2) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 2>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
-        else if (nk <= 4) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 4>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
-        else if (nk <= 8) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 8>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
-        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 0>), g, b, 0, st, X, ldx, rows, lnw, eps, W, bias, C, N, K, rms, epi_arg); \
+        if (nk <= 2) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 2>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 4) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 4>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 8) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 8>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 0>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
     } while (0)
 #define HB_LN(EPI_) \
     do { \
@@ -797,6 +868,7 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
     if (epi == HB_EPI_GELU) HB_LN(HB_EPI_GELU);
     else if (epi == HB_EPI_SCALE) HB_LN(HB_EPI_SCALE);
     else if (epi == HB_EPI_RELU2) HB_LN(HB_EPI_RELU2);
+    else if (epi == HB_EPI_SOFTCAP) HB_LN(HB_EPI_SOFTCAP);
     else if (epi != HB_EPI_STORE) return false;
     else HB_LN(HB_EPI_STORE);
 #undef HB_LN
@@ -2485,14 +2557,16 @@ __global__ __launch_bounds__(1024) __attribute__((amdgpu_waves_per_eu(1, 4))) vo
     }
 }
 
-// few-row steps: the segments' partial results of a (row, head), merged in segment order; output gate applied here
+// few-row steps: the segments' partial results of a (row, head), merged in segment order; output gate (one per head, or gate_cols: one per
+// output column) applied here.  keep: the first tokens of the sequence that stay visible before the window
 __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nseg_grid, float* out, long ldo, const int* pos, int H, int vdim,
                                                       int window, int P, int seg_chunks, const float* gate, long ldg, float out_scale, int chunk,
-                                                      hb_sink sink) {
+                                                      hb_sink sink, int keep = 0, int gate_cols = 0) {
     const int row = blockIdx.x, hq = blockIdx.y, lane = threadIdx.x;
     const int p = pos[row];
     const int first = p - window + 1;
-    const int total = (first > 0 ? first / P : 0) + (p - (first > 0 ? first : 0) + 1);
+    const int lo = first > 0 ? first : 0;
+    const int total = lo / P + (keep < lo ? keep : lo) + (p - lo + 1);
     const int nseg = ((total + chunk - 1) / chunk + seg_chunks - 1) / seg_chunks;
     const float* src = part + (size_t)(row * H + hq) * nseg_grid * (vdim + 2);
     // lane s of each 64 segments fetches segment s's maximum and sum; the total is added in segment order
@@ -2500,7 +2574,7 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
     float mm = sk;
     for (int s0 = 0; s0 < nseg; s0 += 64) mm = fmaxf(mm, s0 + lane < nseg ? src[(size_t)(s0 + lane) * (vdim + 2) + vdim] : -INFINITY);
     mm = hb_wave_max(mm);
-    const float gmul = (gate ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
+    const float gmul = (gate && !gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
     float lt = 0.f;
     float acc[HB_MAX_VPL];
 #pragma unroll
@@ -2536,7 +2610,7 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
 #pragma unroll
     for (int e = 0; e < HB_MAX_VPL; ++e) {
         const int j = lane + e * 64;
-        if (j < vdim) out[(size_t)row * ldo + hq * vdim + j] = acc[e] / lt * gmul;
+        if (j < vdim) out[(size_t)row * ldo + hq * vdim + j] = acc[e] / lt * gmul * (gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq * vdim + j]) : 1.0f);
     }
 }
 
@@ -3329,16 +3403,480 @@ __global__ __launch_bounds__(256) void k_hb_sig_attn_mfma(const float* q, long l
             }
 }
 
+// ---- softmax attention over a window and the first tokens -------------------------------------------------------------------------
+// Position p sees the positions up to itself among the last `window` (0: all) and among the first `keep` of its sequence; exp(sink_h)
+// joins the denominator.  Keys in order: the kept tokens before the window, then the window.
+struct hb_win {
+    int window, keep;
+};
+__device__ __forceinline__ int hb_win_start(const hb_win& w, int p) { return w.window > 0 && p >= w.window ? p - w.window + 1 : 0; }
+
+// What a row leaves in the cache, and its query: q and k RMS-normed over their whole projection (all heads at once, weights q_norm
+// [H*dim], k_norm [G*dim]), then the first `rot` dims of every head rotated (interleaved pairs, cos and sin times `mag`).  proj row =
+// [q | k | v | ...]; the query stays in place, k and v go into the cache.  Block (row, part 0 q / 1 k / 2 v); a thread owns whole pairs.
+template <typename T>
+__global__ __launch_bounds__(256) void k_hb_win_prep(float* proj, long ldp, T* cache, const float* q_norm, const float* k_norm, const float* inv_freq,
+                                                     float mag, const int* pos, const int* page, const int* slot, int H, int G, int dim, int vdim,
+                                                     int rot, int ps, long v_base, float eps) {
+    __shared__ float2 turn[32 * HB_MAX_DPL];
+    __shared__ float red[4];
+    const int row = blockIdx.x, part = blockIdx.y, tid = threadIdx.x, nq = H * dim, nk = G * dim, nv = G * vdim;
+    float* pr = proj + (size_t)row * ldp;
+    const size_t tok = (size_t)page[row] * ps + slot[row];
+    if (part == 2) {
+        T* dst = cache + v_base + tok * (size_t)nv;
+        for (int i = tid; i < nv; i += 256) hb_st(dst + i, pr[nq + nk + i]);
+        return;
+    }
+    float* src = part == 0 ? pr : pr + nq;
+    const int n = part == 0 ? nq : nk, heads = part == 0 ? H : G;
+    const float* nw = part == 0 ? q_norm : k_norm;
+    const float pf = (float)pos[row];
+    for (int i = tid; i < rot / 2; i += 256) {
+        float sn, cs;
+        sincosf(pf * inv_freq[i], &sn, &cs);
+        turn[i] = make_float2(cs * mag, sn * mag);
+    }
+    float ss = 0.f;
+    for (int i = tid; i < n; i += 256) ss = fmaf(src[i], src[i], ss);
+    const float inv = 1.0f / sqrtf(hb_block_sum256(ss, red) / (float)n + eps);
+    T* kd = part == 1 ? cache + tok * (size_t)nk : nullptr;
+    const int pph = (dim + 1) >> 1;
+    for (int i = tid; i < heads * pph; i += 256) {
+        const int h = i / pph, j = i - h * pph, c = h * dim + 2 * j;
+        const bool two = 2 * j + 1 < dim;
+        float u = src[c] * inv * nw[c], v = two ? src[c + 1] * inv * nw[c + 1] : 0.f;
+        if (2 * j < rot) {
+            const float2 t = turn[j];
+            const float u2 = fmaf(u, t.x, -(v * t.y));
+            v = fmaf(v, t.x, u * t.y);
+            u = u2;
+        }
+        if (part == 0) {
+            src[c] = u;
+            if (two) src[c + 1] = v;
+        } else {
+            hb_st(kd + c, u);
+            if (two) hb_st(kd + c + 1, v);
+        }
+    }
+}
+
+// Steps of few rows (and every step of shapes or dtypes the matrix-core form does not take): block = (row, HPB query heads of one key
+// head, segment of cpb 64-key chunks), four waves.  Scores: lane = key, a wave takes one head (fewer than three heads: a part of the key
+// dims of one head, the parts added in order); running maximum and sum per head.  Weighted sums: a wave takes 16 keys of the chunk and all
+// heads, lane = value columns (two adjacent ones of each 128 with a bf16 cache and even sizes, the first 128 columns requested before the
+// scores are formed); the waves' sums are added in wave order.  part != NULL: the segment's unnormalised sums, maximum and sum are left
+// there for k_hb_attn_merge; else sink, gate (per output column) and scale are applied here.
+template <typename T, int HPB>
+__global__ __launch_bounds__(256) void k_hb_win_attn_rows(const float* q, long ldq, const T* cache, float* out, long ldo, const int* pos,
+                                                          const int* row_req, const int* ptab, int pts, int H, int G, int dim, int vdim, int ps,
+                                                          long v_base, hb_win w, float scale, hb_sink sink, int cpb, float* part, const float* gate,
+                                                          long ldg, float out_scale) {
+    extern __shared__ float sm[];
+    constexpr int DS = HPB == 1 ? 4 : (HPB == 2 ? 2 : 1), VE = 16 / sizeof(T);
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int dimp = (dim + 3) & ~3;
+    float* qs = sm;                              // [HPB][dimp]
+    float* dots = qs + HPB * dimp;               // [4][64] partial dots
+    float* pw = dots + 256;                      // [64][HPB] weights
+    float* ml = pw + 64 * HPB;                   // [HPB][4]: what the sums so far are multiplied by, maximum, sum
+    float* red = ml + 4 * HPB;                   // [4][HPB * vdim]
+    const int row = blockIdx.x, h0 = blockIdx.y * HPB, g = h0 / (H / G), p = pos[row];
+    const int* pt = ptab + (size_t)row_req[row] * pts;
+    const int lo = hb_win_start(w, p), kept = w.keep < lo ? w.keep : lo, total = kept + p - lo + 1, nchunks = (total + 63) >> 6;
+    const int c0 = blockIdx.z * cpb, c1 = c0 + cpb < nchunks ? c0 + cpb : nchunks;
+    if (c0 >= nchunks) return;
+    for (int i = tid; i < HPB * dimp; i += 256) {
+        const int h = i / dimp, d = i - h * dimp;
+        qs[i] = d < dim ? q[(size_t)row * ldq + (size_t)(h0 + h) * dim + d] : 0.f;
+    }
+    __syncthreads();
+    const bool kvec = (dim % VE == 0) && ((((size_t)cache) & 15) == 0);
+    const bool pair = sizeof(T) == 2 && (vdim % 2 == 0) && (dim % 2 == 0);
+    const size_t kld = (size_t)G * dim, vld = (size_t)G * vdim;
+    // the wave's part of the scores: head sh, dims sd0 .. sd1 (HPB = 3: the fourth wave has none)
+    const int sh = wv / DS, step = kvec ? VE : 1, per = (dim / step + DS - 1) / DS * step;
+    const int sd0 = wv % DS * per, sd1 = sd0 + per < dim ? sd0 + per : dim;
+    const float* qh = qs + (sh < HPB ? sh : 0) * dimp;
+    float m = -INFINITY, l = 0.f, acc[HPB][HB_MAX_VPL];
+#pragma unroll
+    for (int h = 0; h < HPB; ++h)
+#pragma unroll
+        for (int e = 0; e < HB_MAX_VPL; ++e) acc[h][e] = 0.f;
+    for (int c = c0; c < c1; ++c) {
+        const int base = c * 64, cnt = total - base < 64 ? total - base : 64;
+        const int u0 = base + (lane < cnt ? lane : cnt - 1), t = u0 < kept ? u0 : lo + (u0 - kept);
+        const int tok = pt[t / ps] * ps + t % ps;
+        u32 v0[16];
+        if (pair) {
+            const T* vb = cache + v_base + (size_t)g * vdim + (2 * lane < vdim ? 2 * lane : vdim - 2);
+#pragma unroll
+            for (int x = 0; x < 16; ++x) v0[x] = *(const u32*)(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
+        }
+        if (sh < HPB) {
+            const T* kr = cache + (size_t)tok * kld + (size_t)g * dim;
+            float dot = 0.f;
+            if (kvec) {
+#pragma unroll 8
+                for (int d = sd0; d < sd1; d += VE) {
+                    const uint4 u = *(const uint4*)(kr + d);
+                    float k[VE];
+                    if (sizeof(T) == 2) {
+                        k[0] = bflo(u.x); k[1] = bfhi(u.x); k[2] = bflo(u.y); k[3] = bfhi(u.y);
+                        if (VE == 8) { k[VE - 4] = bflo(u.z); k[VE - 3] = bfhi(u.z); k[VE - 2] = bflo(u.w); k[VE - 1] = bfhi(u.w); }
+                    } else {
+                        k[0] = __uint_as_float(u.x); k[1] = __uint_as_float(u.y); k[2] = __uint_as_float(u.z); k[3] = __uint_as_float(u.w);
+                    }
+#pragma unroll
+                    for (int e = 0; e < VE; ++e) dot = fmaf(qh[d + e], k[e], dot);
+                }
+            } else {
+                for (int d = sd0; d < sd1; ++d) dot = fmaf(qh[d], hb_ld(kr + d), dot);
+            }
+            dots[wv * 64 + lane] = dot;
+        }
+        if (DS > 1) __syncthreads();
+        if (wv % DS == 0 && sh < HPB) {
+            float dot = dots[wv * 64 + lane];
+#pragma unroll
+            for (int x = 1; x < DS; ++x) dot += dots[(wv + x) * 64 + lane];
+            const float z = lane < cnt ? dot * scale : -INFINITY;
+            const float mn = fmaxf(m, hb_wave_max(z)), e = lane < cnt ? expf(z - mn) : 0.f, alpha = expf(m - mn);
+            l = fmaf(l, alpha, hb_wave_sum(e));
+            m = mn;
+            pw[lane * HPB + sh] = e;
+            if (lane == 0) { ml[sh * 4] = alpha; ml[sh * 4 + 1] = m; ml[sh * 4 + 2] = l; }
+        }
+        __syncthreads();
+        if (c > c0) {
+#pragma unroll
+            for (int h = 0; h < HPB; ++h) {
+                const float alpha = ml[h * 4];
+#pragma unroll
+                for (int e = 0; e < HB_MAX_VPL; ++e) acc[h][e] *= alpha;
+            }
+        }
+        const float* wpw = pw + wv * 16 * HPB;      // (weights behind the last key are zero)
+        if (pair) {
+#pragma unroll
+            for (int cc = 0; cc < HB_MAX_VPL / 2; ++cc) {
+                if (cc * 128 < vdim) {
+                    if (cc > 0) {
+                        const int j = cc * 128 + 2 * lane;
+                        const T* vb = cache + v_base + (size_t)g * vdim + (j < vdim ? j : vdim - 2);
+#pragma unroll
+                        for (int x = 0; x < 16; ++x) v0[x] = *(const u32*)(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
+                    }
+#pragma unroll
+                    for (int x = 0; x < 16; ++x)
+#pragma unroll
+                        for (int h = 0; h < HPB; ++h) {
+                            acc[h][2 * cc] = fmaf(wpw[x * HPB + h], bflo(v0[x]), acc[h][2 * cc]);
+                            acc[h][2 * cc + 1] = fmaf(wpw[x * HPB + h], bfhi(v0[x]), acc[h][2 * cc + 1]);
+                        }
+                }
+            }
+        } else {
+#pragma unroll
+            for (int cc = 0; cc < HB_MAX_VPL; ++cc) {
+                if (cc * 64 < vdim) {
+                    const int j = cc * 64 + lane;
+                    const T* vb = cache + v_base + (size_t)g * vdim + (j < vdim ? j : vdim - 1);
+                    float vv[16];
+#pragma unroll
+                    for (int x = 0; x < 16; ++x) vv[x] = hb_ld(vb + (size_t)__builtin_amdgcn_readlane(tok, wv * 16 + x) * vld);
+#pragma unroll
+                    for (int x = 0; x < 16; ++x)
+#pragma unroll
+                        for (int h = 0; h < HPB; ++h) acc[h][cc] = fmaf(wpw[x * HPB + h], vv[x], acc[h][cc]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    float* mine = red + (size_t)wv * HPB * vdim;
+#pragma unroll
+    for (int h = 0; h < HPB; ++h)
+#pragma unroll
+        for (int e = 0; e < HB_MAX_VPL; ++e) {
+            const int j = pair ? (e >> 1) * 128 + 2 * lane + (e & 1) : lane + e * 64;
+            if (j < vdim) mine[h * vdim + j] = acc[h][e];
+        }
+    __syncthreads();
+    const int nv = HPB * vdim;
+    for (int i = tid; i < nv; i += 256) {
+        float a = ((red[i] + red[nv + i]) + red[2 * nv + i]) + red[3 * nv + i];
+        const int hh = i / vdim, h = h0 + hh, j = i - hh * vdim;
+        const float mh = ml[hh * 4 + 1], lh = ml[hh * 4 + 2];
+        if (part) {
+            float* dst = part + ((size_t)(row * H + h) * gridDim.z + blockIdx.z) * (vdim + 2);
+            dst[j] = a;
+            if (j == 0) { dst[vdim] = mh; dst[vdim + 1] = lh; }
+            continue;
+        }
+        float den = lh;
+        if (sink.on) {
+            const float sk = hb_sink_of(sink, h), mm = fmaxf(mh, sk), f = expf(mh - mm);
+            a *= f;
+            den = fmaf(lh, f, expf(sk - mm));
+        }
+        a = a / den * out_scale;
+        if (gate) a *= hb_sigmoid(gate[(size_t)row * ldg + h * vdim + j]);
+        out[(size_t)row * ldo + (size_t)h * vdim + j] = a;
+    }
+}
+// Steps of many rows, bf16 cache: block = 64 * RT consecutive rows of one request (RT groups of 16 per wave) and one head; tiles of 64 keys
+// in LDS, keys as cached (Kt[key][dim]), values transposed two keys at a time (Vt[column][key]); the next tile's requests are on their way
+// while a tile is multiplied.  Tiles: the kept tokens before the first row's window, then the windows of all rows.  Per tile, wave and group,
+// rows being the 16 columns of both products:
+//   S^T[key][row] = sum_dim Kt[key][dim] Q[row][dim]     v_mfma_f32_16x16x32_bf16, the query in registers as two bf16 parts (hi + lo)
+//   weights 2^(score - running maximum) of the lane's 16 (key, row) pairs, fp32, scores carrying scale * log2(e); masked pairs 0
+//   O^T[col][row] += sum_key Vt[col][key] P[row][key]    the weights as they sit in the lanes (k index laid out to match), hi + lo
+// Row tiles of the launch are found by walking the requests' row counts; blocks beyond the last tile leave.  KS 32-dim steps of the key
+// and CT 16-column tiles of the value at most.
+template <int KS, int CT, int RT>
+__global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long ldq, const bf16_t* cache, float* out, long ldo, const int* pos,
+                                                          const int* req_rows, int n_req, const int* ptab, int pts, int H, int G, int dim, int vdim,
+                                                          int ps, long v_base, hb_win w, float scale, hb_sink sink, const float* gate, long ldg,
+                                                          float out_scale, int ks_n, int ct_n, int fold) {
+    extern __shared__ float sm[];
+    constexpr int BR = 64 * RT, WR = 16 * RT;
+    constexpr float LOG2E = 1.44269504088896340736f, LOWEST = -1e30f;
+    const int DPK = ks_n * 32 + 8;
+    bf16_t* Kt = (bf16_t*)sm;                            // [64][DPK]
+    bf16_t* Vt = Kt + 64 * DPK;                          // [ct_n * 16][HB_SIG_VLD]
+    const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, col = lane & 15, g4 = lane >> 4;
+    // Blocks in launch order: all heads of a tile, then the next tile, the later rows of a request (more keys) first; a launch that fits the
+    // chip at once (fold) follows the heavier half in descending order with the lighter half in ascending order
+    const int nt_all = gridDim.y, half = (nt_all + 1) >> 1;
+    int t = nt_all - 1 - (int)blockIdx.y, rq = -1, rs = 0, re = 0;
+    if (fold && (int)blockIdx.y >= half) t = (int)blockIdx.y - half;
+    for (int r = 0; r < n_req; ++r) {
+        const int a = req_rows[r], b = req_rows[r + 1], nt = (b - a + BR - 1) / BR;
+        if (t < nt) { rq = r; rs = a + BR * t; re = b; break; }
+        t -= nt;
+    }
+    if (rq < 0) return;
+    const int h = blockIdx.x, g = h / (H / G);
+    const int nrows = re - rs < BR ? re - rs : BR;
+    const int w0 = wv * WR, wn = nrows - w0 < WR ? nrows - w0 : WR;      // the wave's rows: w0 .. w0 + wn - 1 of the tile (wn may be <= 0)
+    const bool active = wn > 0;
+    const int p0 = pos[rs], pl = pos[rs + nrows - 1];
+    const int wp_first = active ? pos[rs + w0] : 0, wp_hi = active ? pos[rs + w0 + wn - 1] : -1;
+    const int lo_t = hb_win_start(w, p0), kept = w.keep < lo_t ? w.keep : lo_t, nkt = (kept + 63) >> 6;
+    const int ntiles = nkt + ((pl - lo_t + 64) >> 6);
+    const int wlo_first = hb_win_start(w, wp_first), wlo_hi = active ? hb_win_start(w, wp_hi) : 0;
+    const int* pt = ptab + (size_t)rq * pts;
+    const float zmul = scale * LOG2E;
+    int p[RT], lo_r[RT];
+    bool rowok[RT];
+    uint4 qh[RT][KS], ql[RT][KS];
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        rowok[rt] = rt * 16 + col < wn;
+        const int row = rs + (active ? w0 + (rowok[rt] ? rt * 16 + col : wn - 1) : 0);      // (a lane without a row follows the wave's last one)
+        p[rt] = pos[row];
+        lo_r[rt] = hb_win_start(w, p[rt]);
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            float v[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[i] = 0.f;
+            const int d0 = ks * 32 + g4 * 8;
+            if (ks < ks_n && rowok[rt] && d0 < dim) {
+                const float* src = q + (size_t)row * ldq + (size_t)h * dim + d0;
+                const float4 a = *(const float4*)src, b = *(const float4*)(src + 4);
+                v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+            }
+            hb_split_bf16x8(v, qh[rt][ks], ql[rt][ks]);
+        }
+    }
+    hb_f32x4 oacc[RT][CT];
+    float m[RT], l[RT];         // running maximum of the row (log2 units), the lane's share of its sum
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        m[rt] = LOWEST;
+        l[rt] = 0.f;
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) oacc[rt][ct] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    // staging: keys -- four threads per key, pieces of 8 dims (tid & 3) + 4k; values -- eight threads per pair of keys, pieces of 8
+    // columns (tid & 7) + 8k of both keys
+    constexpr int NV = (CT * 2 + 7) / 8;
+    uint4 rk[KS], rv0[NV], rv1[NV];
+    const int kj = tid >> 2, kpiece = tid & 3, vj = (tid >> 3) * 2, vpiece = tid & 7, dpie = dim >> 3, vpie = vdim >> 3;
+    auto fetch = [&](int c) {
+        const int base = c < nkt ? c * 64 : lo_t + (c - nkt) * 64, end = c < nkt ? kept : pl + 1;
+        const int cnt = end - base < 64 ? end - base : 64;
+        const bool kok = kj < cnt;
+        const int tk = base + (kok ? kj : 0);
+        const bf16_t* kp = cache + ((size_t)pt[tk / ps] * ps + tk % ps) * (size_t)(G * dim) + (size_t)g * dim;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) {
+            const int v = kpiece + 4 * k;
+            rk[k] = kok && v < dpie ? *(const uint4*)(kp + v * 8) : make_uint4(0, 0, 0, 0);
+        }
+        const bool ok0 = vj < cnt, ok1 = vj + 1 < cnt;
+        const int t0 = base + (ok0 ? vj : 0), t1 = base + (ok1 ? vj + 1 : 0);
+        const bf16_t* vb = cache + v_base + (size_t)g * vdim;
+        const bf16_t* v0 = vb + ((size_t)pt[t0 / ps] * ps + t0 % ps) * (size_t)(G * vdim);
+        const bf16_t* v1 = vb + ((size_t)pt[t1 / ps] * ps + t1 % ps) * (size_t)(G * vdim);
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int v = vpiece + 8 * k;
+            rv0[k] = ok0 && v < vpie ? *(const uint4*)(v0 + v * 8) : make_uint4(0, 0, 0, 0);
+            rv1[k] = ok1 && v < vpie ? *(const uint4*)(v1 + v * 8) : make_uint4(0, 0, 0, 0);
+        }
+    };
+    fetch(0);
+    for (int c = 0; c < ntiles; ++c) {
+        const bool early = c < nkt;                  // a tile of kept tokens: every row sees those below `kept`
+        const int base = early ? c * 64 : lo_t + (c - nkt) * 64;
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < KS; ++k)
+            if (k < ks_n) *(uint4*)(Kt + kj * DPK + (kpiece + 4 * k) * 8) = rk[k];
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int cc = (vpiece + 8 * k) * 8;
+            if (cc < ct_n * 16) {
+                const u32 a[4] = {rv0[k].x, rv0[k].y, rv0[k].z, rv0[k].w}, b[4] = {rv1[k].x, rv1[k].y, rv1[k].z, rv1[k].w};
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    u32* d0 = (u32*)(Vt + (size_t)(cc + 2 * i) * HB_SIG_VLD + vj);
+                    *d0 = (a[i] & 0xffffu) | (b[i] << 16);
+                    u32* d1 = (u32*)(Vt + (size_t)(cc + 2 * i + 1) * HB_SIG_VLD + vj);
+                    *d1 = (a[i] >> 16) | (b[i] & 0xffff0000u);
+                }
+            }
+        }
+        __syncthreads();
+        if (c + 1 < ntiles) fetch(c + 1);
+        // (a wave whose rows see no key of the tile)
+        if (!active || (!early && (base > wp_hi || (base + 63 < wlo_first && base >= w.keep)))) continue;
+        hb_f32x4 st[RT][4];
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt) st[rt][kt] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            if (ks < ks_n) {
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt) {
+                    const uint4 a = *(const uint4*)(Kt + (size_t)(kt * 16 + col) * DPK + ks * 32 + g4 * 8);
+#pragma unroll
+                    for (int rt = 0; rt < RT; ++rt) {
+                        st[rt][kt] = hb_mfma_bf16(a, qh[rt][ks], st[rt][kt]);
+                        st[rt][kt] = hb_mfma_bf16(a, ql[rt][ks], st[rt][kt]);
+                    }
+                }
+            }
+        }
+        // lane (col, g4) holds the scores of row `col` of each group against keys base + kt*16 + g4*4 + i
+        const bool full = early ? base + 63 < kept : (base + 63 <= wp_first && base >= wlo_hi);     // every row of the wave sees the whole tile
+        uint4 ph[RT][2], plo[RT][2];
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt) {
+            float z[4][4], top = LOWEST;
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    float s = st[rt][kt][i] * zmul;
+                    if (!full) {
+                        const int key = base + kt * 16 + g4 * 4 + i;
+                        const bool see = early ? key < kept : key <= p[rt] && (key >= lo_r[rt] || key < w.keep);
+                        s = see ? s : -INFINITY;
+                    }
+                    z[kt][i] = s;
+                    top = fmaxf(top, s);
+                }
+            top = fmaxf(top, __shfl_xor(top, 16, 64));
+            top = fmaxf(top, __shfl_xor(top, 32, 64));
+            if (__ballot(top > m[rt])) {
+                const float mn = fmaxf(m[rt], top), alpha = __builtin_amdgcn_exp2f(m[rt] - mn);
+                m[rt] = mn;
+                l[rt] *= alpha;
+#pragma unroll
+                for (int ct = 0; ct < CT; ++ct)
+                    if (ct < ct_n)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) oacc[rt][ct][i] *= alpha;
+            }
+            float sum = 0.f;
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    z[kt][i] = __builtin_amdgcn_exp2f(z[kt][i] - m[rt]);
+                    sum += z[kt][i];
+                }
+            l[rt] += sum;
+#pragma unroll
+            for (int kk = 0; kk < 2; ++kk) {
+                const float v[8] = {z[2 * kk][0], z[2 * kk][1], z[2 * kk][2], z[2 * kk][3], z[2 * kk + 1][0], z[2 * kk + 1][1], z[2 * kk + 1][2],
+                                    z[2 * kk + 1][3]};
+                hb_split_bf16x8(v, ph[rt][kk], plo[rt][kk]);
+            }
+        }
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) {
+            if (ct < ct_n) {
+#pragma unroll
+                for (int kk = 0; kk < 2; ++kk) {
+                    const bf16_t* vr = Vt + (size_t)(ct * 16 + col) * HB_SIG_VLD + kk * 32 + g4 * 4;
+                    const uint2 a0 = *(const uint2*)vr, a1 = *(const uint2*)(vr + 16);
+                    const uint4 a = make_uint4(a0.x, a0.y, a1.x, a1.y);
+#pragma unroll
+                    for (int rt = 0; rt < RT; ++rt) {
+                        oacc[rt][ct] = hb_mfma_bf16(a, ph[rt][kk], oacc[rt][ct]);
+                        oacc[rt][ct] = hb_mfma_bf16(a, plo[rt][kk], oacc[rt][ct]);
+                    }
+                }
+            }
+        }
+    }
+    const float sk = sink.on ? hb_sink_of(sink, h) * LOG2E : 0.f;
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        float den = l[rt];
+        den += __shfl_xor(den, 16, 64);
+        den += __shfl_xor(den, 32, 64);
+        float f = out_scale;
+        if (sink.on) {
+            const float mm = fmaxf(m[rt], sk), a = __builtin_amdgcn_exp2f(m[rt] - mm);
+            den = fmaf(den, a, __builtin_amdgcn_exp2f(sk - mm));
+            f *= a;
+        }
+        if (!rowok[rt]) continue;
+        const int row = rs + w0 + rt * 16 + col;
+        f /= den;
+        float* dst = out + (size_t)row * ldo + (size_t)h * vdim;
+        const float* gr = gate ? gate + (size_t)row * ldg + (size_t)h * vdim : nullptr;
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct)
+            if (ct < ct_n)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int cc = ct * 16 + g4 * 4 + i;
+                    if (cc < vdim) dst[cc] = oacc[rt][ct][i] * f * (gr ? hb_sigmoid(gr[cc]) : 1.0f);
+                }
+    }
+}
+
 // ---- routed feed-forward --------------------------------------------------------------------------------------------------
 // One block per row: router logits z_j = router[j] . h in fp32 (lane-strided sums over four waves and a butterfly: an order fixed by
 // the width, the same for every step shape), then one wave: s = softmax(z) over all nE router outputs, choice = s + correction, the `top` largest choices (first
 // index wins a tie) in descending order; weights = their s / (sum + 1e-20).  sel[row*top + k] = router output index, wgt likewise.
 // sigmoid != 0: s_j = sigmoid(z_j) instead of the softmax; renorm == 0: the weights are the chosen s as they are.
 // bias != NULL: added to the logits before the scores are formed.  groups > 1: only experts of the `keep` best groups can be chosen.
-// wscale multiplies the weights.
+// wscale multiplies the weights.  A group's score is its largest choice value, or (best_two) the sum of its two largest.
+// post.y != NULL: the row is first completed with a normed sublayer output, x_out (= h) += norm(y).
 __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh, const float* router, const float* corr, int W, int nE, int top,
                                                        int* sel, float* wgt, int sigmoid, int renorm, const float* bias, int groups, int keep,
-                                                       float wscale) {
+                                                       float wscale, int best_two, hb_post post, float* x_out) {
     extern __shared__ float sm[];
     float* sc = sm;                    // [nE] logits, then scores
     float* ch = sm + nE;               // [nE] choice values
@@ -3347,6 +3885,14 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
     float* gs = part + 4 * nE;         // [groups] group scores (groups > 1)
     const int row = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const float* x = h + (size_t)row * ldh;
+    if (post.y) {
+        __shared__ float red[2][4];
+        float* xr = x_out + (size_t)row * ldh;
+        if (W <= 1024) hb_post_norm_row<4>(post, row, xr, W, red);
+        else if (W <= 4096) hb_post_norm_row<16>(post, row, xr, W, red);
+        else hb_post_norm_row<0>(post, row, xr, W, red);
+        __syncthreads();
+    }
     const bool vec = (W % 4 == 0) && (ldh % 4 == 0) && ((((size_t)h) & 15) == 0) && ((((size_t)router) & 15) == 0);
     // wave w sums the k-chunks w, w + 4, ... (64 lanes x 4 values, or 64 values); a logit = the four waves' sums added in wave order
     for (int j0 = 0; j0 < nE; j0 += 8) {
@@ -3427,13 +3973,17 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
     __builtin_amdgcn_wave_barrier();
     if (groups > 1 && keep < groups) {
-        // groups of neighbours: a group's score is its largest choice value; `keep` groups stay (the first of equal ones), the experts of
+        // groups of neighbours: a group's score comes from its largest choice values; `keep` groups stay (the first of equal ones), the experts of
         // the others cannot be chosen
         const int per = nE / groups;
         for (int g = lane; g < groups; g += 64) {
-            float best = -INFINITY;
-            for (int i = 0; i < per; ++i) best = fmaxf(best, ch[g * per + i]);
-            gs[g] = best;
+            float best = -INFINITY, second = -INFINITY;
+            for (int i = 0; i < per; ++i) {
+                const float v = ch[g * per + i];
+                second = fmaxf(second, fminf(best, v));
+                best = fmaxf(best, v);
+            }
+            gs[g] = best_two && per > 1 ? best + second : best;
         }
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
         __builtin_amdgcn_wave_barrier();
@@ -3694,6 +4244,7 @@ struct vox_hybrid {
     std::vector<vox_hybrid_run> runs;
     vox_hybrid_weights w;
     float *xa = nullptr, *xb = nullptr, *h = nullptr, *h2 = nullptr, *proj = nullptr, *mix = nullptr, *ff = nullptr, *hout = nullptr;
+    float *y = nullptr;                     // [max_rows][width]: a sublayer's output that is normed before it joins
     float *u = nullptr, *ones = nullptr;    // [max_rows][width]: what the next sublayer reads of several residual streams; [HB_MAX_STREAMS]
     float *rgate = nullptr;                 // [max_rows][width]: residual gate logits of a routed feed-forward
     float *ff_act = nullptr;                // [max_rows][max gated dense width]: activation output of the gated dense feed-forward
@@ -3708,12 +4259,13 @@ struct vox_hybrid {
     size_t attn_ws_bytes = 0;
     int max_in = 0, max_mix = 0, max_ff = 0;
     int max_ne = 0, max_top = 0, max_eff = 0, max_experts = 0;
-    bool any_shift = false, any_rgate = false;
+    bool any_shift = false, any_rgate = false, any_post = false;
     bool attn_big_lds = false;              // the attention kernel was given the right to more than 64 KB of LDS
     bool lat_big_lds = false;               // the same for the few-row latent attention
 };
 
-static bool hb_is_attn(int kind) { return kind == VOX_MIXER_POOLED_WINDOW_ATTN || kind == VOX_MIXER_CAUSAL_ATTN || kind == VOX_MIXER_LATENT_ATTN || kind == VOX_MIXER_SIGMOID_ATTN; }
+static bool hb_is_attn(int kind) { return kind == VOX_MIXER_POOLED_WINDOW_ATTN || kind == VOX_MIXER_CAUSAL_ATTN || kind == VOX_MIXER_LATENT_ATTN || kind == VOX_MIXER_SIGMOID_ATTN ||
+           kind == VOX_MIXER_WINDOW_ATTN; }
 static inline int hb_up4(int v) { return (v + 3) & ~3; }
 // Where a latent-attention row keeps what it derives from the fused projection [query latent | kv latent | rotated key | gate]:
 // (without a query latent: [q | kv latent | rotated key | gate], the query at column 0), then the residual gate's columns.
@@ -3792,6 +4344,7 @@ static int hb_layer_in(const vox_hybrid_layer& L) {
         case VOX_MIXER_LATENT_ATTN: return hb_latent(L).n_in;
         case VOX_MIXER_RETENTION: return 2 * L.heads * L.dim + 2 * L.heads * L.vdim + rg;
         case VOX_MIXER_DELTA: return L.kv_heads > 0 ? hb_delta(L).n_in : -1;
+        case VOX_MIXER_WINDOW_ATTN: return L.heads * L.dim + (L.kv_shared ? 0 : L.kv_heads * (L.dim + L.vdim)) + (L.out_gate ? L.heads * L.vdim : 0) + rg;
         case VOX_MIXER_SIGMOID_ATTN: return L.heads * L.dim + L.kv_heads * (L.dim + L.vdim) + (L.out_gate ? L.heads * L.vdim : 0) + rg;
     }
     return -1;
@@ -3803,12 +4356,12 @@ static int hb_layer_proj(const vox_hybrid_layer& L) {
     if (L.kind == VOX_MIXER_LATENT_ATTN) return hb_latent(L).n_proj;
     if (L.kind == VOX_MIXER_DELTA) return hb_delta(L).n_proj;
     if (hb_conv_attn(L)) return hb_conv_attn_cols(L).n_proj;
-    if (L.kind == VOX_MIXER_SIGMOID_ATTN) return hb_up4(hb_layer_in(L));
+    if (L.kind == VOX_MIXER_SIGMOID_ATTN || L.kind == VOX_MIXER_WINDOW_ATTN) return hb_up4(hb_layer_in(L));
     return hb_layer_in(L);
 }
 
 static void hb_norm(const vox_hybrid* m, hipStream_t st, int n, const float* x, long ldx, const int* rows, const float* w1, float* y1,
-                    const float* w2, float* y2, long ldy) {
+                    const float* w2, float* y2, long ldy, const float* b1 = nullptr, const float* b2 = nullptr) {
     const vox_hybrid_config& c = m->cfg;
     if (c.norm_kind == VOX_NORM_RMS_GROUPS && c.norm_groups == 1) {
         hipLaunchKernelGGL(k_hb_rms_row, dim3(n), dim3(256), 0, st, x, ldx, rows, w1, y1, w2, y2, ldy, c.width, c.eps);
@@ -3816,16 +4369,16 @@ static void hb_norm(const vox_hybrid* m, hipStream_t st, int n, const float* x, 
         hipLaunchKernelGGL(k_hb_rms_groups, dim3(n, (c.norm_groups + 3) / 4 < 8 ? (c.norm_groups + 3) / 4 : 8), dim3(256), 0, st, x, ldx, rows, w1, y1,
                            w2, y2, ldy, c.width, c.norm_groups, c.eps);
     } else {
-        hb_layernorm(st, n, x, ldx, rows, w1, y1, ldy, c.width, c.eps);
-        if (w2) hb_layernorm(st, n, x, ldx, rows, w2, y2, ldy, c.width, c.eps);
+        hb_layernorm(st, n, x, ldx, rows, w1, b1, y1, ldy, c.width, c.eps);
+        if (w2) hb_layernorm(st, n, x, ldx, rows, w2, b2, y2, ldy, c.width, c.eps);
     }
 }
 // the fused one-row norm + GEMV exists for the layer norm and for the RMS norm over one slice
 template <typename T>
 static bool hb_try_norm_gemv(const vox_hybrid* m, hipStream_t st, int epi, const float* X, long ldx, const int* rows, const float* nw, const T* W,
-                             const float* bias, float* C, int N, int K, float epi_arg = 0.f) {
+                             const float* bias, float* C, int N, int K, float epi_arg = 0.f, const float* nb = nullptr) {
     const bool rms = m->cfg.norm_kind == VOX_NORM_RMS_GROUPS && m->cfg.norm_groups == 1;
-    return (m->cfg.norm_kind == VOX_NORM_LAYER || rms) && hb_try_ln_gemv<T>(st, epi, X, ldx, rows, nw, m->cfg.eps, W, bias, C, N, K, rms ? 1 : 0, epi_arg);
+    return (m->cfg.norm_kind == VOX_NORM_LAYER || rms) && hb_try_ln_gemv<T>(st, epi, X, ldx, rows, nw, m->cfg.eps, W, bias, C, N, K, rms ? 1 : 0, epi_arg, nb);
 }
 
 // The matrix-core latent attention for steps of many rows over a bf16 cache.  false: the shapes do not fit it (rows of the cache that are
@@ -3918,6 +4471,61 @@ static int hb_sig_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* 
     return VOX_OK;
 }
 
+// The matrix-core window attention for steps of many rows over a bf16 cache.  false: the sizes do not fit it (head dims that are no
+// multiple of 8, or above 256).
+static bool hb_try_win_mfma(hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const bf16_t* cache, const float* q, long ldp,
+                            float* out, long ldo, const hb_sink& sink, const float* gate, long v_base, int n, int n_req, int ps) {
+    if ((L.dim & 7) || (L.vdim & 7) || L.dim > 256 || L.vdim > 256 || (ldp & 3) || ((size_t)q & 15) || ((size_t)cache & 15)) return false;
+    const int ks_n = (L.dim + 31) / 32, ct_n = (L.vdim + 15) / 16;
+    const size_t lds = (size_t)64 * (ks_n * 32 + 8) * 2 + (size_t)ct_n * 16 * HB_SIG_VLD * 2;
+#define HB_WM(KS_, CT_, RT_) \
+    do { \
+        const dim3 grid(L.heads, (n + (64 * RT_ - 1) * n_req) / (64 * RT_)), block(256);      /* (at least the sum of the requests' tiles) */ \
+        if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_win_attn_mfma<KS_, CT_, RT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        hipLaunchKernelGGL((k_hb_win_attn_mfma<KS_, CT_, RT_>), grid, block, lds, st, q, ldp, cache, out, ldo, io->pos, io->req_rows, n_req, io->page_table, \
+                           io->pt_stride, L.heads, L.kv_heads, L.dim, L.vdim, ps, v_base, hb_win{L.window, L.keep_first}, L.scale, sink, gate, ldp, \
+                           L.out_scale, ks_n, ct_n, grid.x * grid.y <= 2 * 256 ? 1 : 0); \
+    } while (0)
+    if (ks_n <= 4 && ct_n <= 8) HB_WM(4, 8, 1);
+    else HB_WM(8, 16, 1);
+#undef HB_WM
+    return true;
+}
+static bool hb_try_win_mfma(hipStream_t, const vox_hybrid_io*, const vox_hybrid_layer&, const float*, const float*, long, float*, long, const hb_sink&,
+                            const float*, long, int, int, int) { return false; }
+// keys a position can see at most
+static int hb_win_keys(const vox_hybrid_layer& L, int max_kvlen) {
+    return L.window > 0 && L.window < max_kvlen - L.keep_first ? L.window + L.keep_first : max_kvlen;
+}
+template <typename T>
+static int hb_win_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const T* cache, long ldp, int n, int n_req,
+                            int max_kvlen, long v_base) {
+    const int H = L.heads, G = L.kv_heads, ps = m->cfg.page_size, n_mix = H * L.vdim;
+    const hb_sink sink{L.sinks ? 1 : 0, L.sinks};
+    const float* gate = L.out_gate ? m->proj + H * L.dim + (L.kv_shared ? 0 : G * (L.dim + L.vdim)) : nullptr;
+    const bool few = n <= HB_ATTN_SEG_ROWS;
+    if (!few && hb_try_win_mfma(st, io, L, cache, m->proj, ldp, m->mix, (long)n_mix, sink, gate, v_base, n, n_req, ps)) return VOX_OK;
+    const int hpb = hb_sig_heads(L);
+    const int nchunks = (hb_win_keys(L, max_kvlen) + 63) / 64;
+    const int want = few ? (nchunks < HB_SIG_MAX_SEG ? nchunks : HB_SIG_MAX_SEG) : 1, cpb = (nchunks + want - 1) / want, nseg = (nchunks + cpb - 1) / cpb;
+    if (nseg > 1 && (size_t)n * H * nseg * (L.vdim + 2) * 4 > m->attn_ws_bytes) return vox_fail(VOX_ERR_INVALID, "hybrid_step: attention workspace");
+    float* part = nseg > 1 ? m->attn_ws : nullptr;
+    const size_t lds = (size_t)(hpb * ((L.dim + 3) & ~3) + 256 + 64 * hpb + 4 * hpb + 4 * hpb * L.vdim) * 4;
+#define HB_WR(HPB_) \
+    hipLaunchKernelGGL((k_hb_win_attn_rows<T, HPB_>), dim3(n, H / HPB_, nseg), dim3(256), lds, st, m->proj, ldp, cache, m->mix, (long)n_mix, io->pos, \
+                       io->row_req, io->page_table, io->pt_stride, H, G, L.dim, L.vdim, ps, v_base, hb_win{L.window, L.keep_first}, L.scale, sink, cpb, \
+                       part, gate, ldp, L.out_scale)
+    if (hpb == 4) HB_WR(4);
+    else if (hpb == 3) HB_WR(3);
+    else if (hpb == 2) HB_WR(2);
+    else HB_WR(1);
+#undef HB_WR
+    if (nseg > 1)
+        hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim,
+                           L.window > 0 ? L.window : 0x7fffffff, 0x7fffffff, cpb, gate, ldp, L.out_scale, 64, sink, L.keep_first, gate ? 1 : 0);
+    return VOX_OK;
+}
+
 // cur joins (A . W^T + bias)
 template <typename T>
 static int hb_gemm_resid(hipStream_t st, const float* A, long lda, const T* W, const float* bias, float* cur, long ldx, int n, int N, int K,
@@ -3925,14 +4533,14 @@ static int hb_gemm_resid(hipStream_t st, const float* A, long lda, const T* W, c
     hb_rowmap rm = hb_plain();
     rm.col_scale = j.scale;
     rm.join = j;
-    const int epi = j.gate || j.streams > 0 ? HB_EPI_JOIN : (j.scale ? HB_EPI_RESID_SCALED : HB_EPI_RESID);
+    const int epi = j.store ? HB_EPI_STORE : j.gate || j.streams > 0 ? HB_EPI_JOIN : (j.scale ? HB_EPI_RESID_SCALED : HB_EPI_RESID);
     return hb_gemm<T>(st, epi, A, lda, W, bias, cur, ldx, n, N, K, rm);
 }
-// One mixer: reads the normed rows (hn != NULL) or norms src (rows lds apart) itself with L.norm1; out_scale * mixer(.) joins cur as `jn`
+// One mixer: reads the rows hn (!= NULL, ldh apart: normed already, or read as they are) or norms src (rows lds apart) itself with L.norm1; out_scale * mixer(.) joins cur as `jn`
 // says (the layer's residual gate, when it has one, is added to it here: its logits are the last columns of the input projection).
 template <typename T>
 static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, void* cache, float* pool, float* state,
-                    const float* hn, const float* src, long lds_x, float* cur, long ldx, int n, int n_req, int max_kvlen, hb_join jn) {
+                    const float* hn, long ldh, const float* src, long lds_x, float* cur, long ldx, int n, int n_req, int max_kvlen, hb_join jn) {
     const vox_hybrid_config& c = m->cfg;
     const int W = c.width, ps = c.page_size;
     const int n_in = hb_layer_in(L), n_proj = hb_layer_proj(L), n_mix = L.heads * L.vdim;
@@ -3940,7 +4548,7 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
     if (L.res_gate) { jn.gate = m->proj + n_in - L.res_gate; jn.ldg = n_proj; }
     if (L.kind == VOX_MIXER_SHIFT_DECAY) {
         // five token-shift mixes of the normed input, each with its own projection
-        if (!hn) { hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W); hn = m->h; }
+        if (!hn) { hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W, L.norm1_b); hn = m->h; }
         const int HD = L.heads * L.dim;
         const long per_slot = (long)HD * L.dim + W, rows_stride = (long)c.max_rows * W;
         const T* wi = (const T*)L.w_in;
@@ -3995,11 +4603,12 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
                                (int)HB_GATE_SILU, L.vdim, c.eps, L.out_scale);
         return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
     }
-    if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, src, lds_x, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W))) {
-        hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W);
+    if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, src, lds_x, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W, 0.f, L.norm1_b))) {
+        hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W, L.norm1_b);
         hn = m->h;
+        ldh = W;
     }
-    if (hn) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hn, W, (const T*)L.w_in, L.b_in, m->proj, n_proj, n, n_in, W));
+    if (hn) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hn, ldh, (const T*)L.w_in, L.b_in, m->proj, n_proj, n, n_in, W));
     const int vt = (L.vdim + 63) / 64;
     // dims per wave of the scans: the smallest of 16 / 32 / 64 that covers dim with at most 16 waves
     const int dpw = L.dim <= 16 * HB_SCAN_MAX_WAVES ? 16 : (L.dim <= 32 * HB_SCAN_MAX_WAVES ? 32 : 64);
@@ -4169,6 +4778,13 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
         else
             hipLaunchKernelGGL(k_hb_rglru_scan, dim3(n_req, (C + 63) / 64), dim3(64), 0, st, m->proj, (long)n_proj, m->mix, (long)n_mix, L.lam, state,
                                io->req_rows, io->req_state, io->pos, C, bs, L.conv_taps, L.rec_scale, L.out_scale);
+    } else if (L.kind == VOX_MIXER_WINDOW_ATTN) {
+        // (kv_shared: the run's cache is another layer's, nothing is added to it)
+        const int H = L.heads, G = L.kv_heads;
+        const long v_base = (long)c.max_pages * ps * G * L.dim;
+        hipLaunchKernelGGL((k_hb_win_prep<T>), dim3(n, L.kv_shared ? 1 : 3), dim3(256), 0, st, m->proj, (long)n_proj, (T*)cache, L.q_norm, L.k_norm,
+                           L.inv_freq, L.rot_mag != 0.f ? L.rot_mag : 1.0f, io->pos, io->page, io->slot, H, G, L.dim, L.vdim, L.rot_dims, ps, v_base, c.eps);
+        VOX_TRY(hb_win_attention<T>(m, st, io, L, (const T*)cache, (long)n_proj, n, n_req, max_kvlen, v_base));
     } else if (L.kind == VOX_MIXER_SIGMOID_ATTN) {
         const int H = L.heads, G = L.kv_heads;
         const long v_base = (long)c.max_pages * ps * G * L.dim;
@@ -4231,35 +4847,35 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
     return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
 }
 
-// Routed feed-forward of the normed rows h2, added to cur.  Few rows: one GEMV pair per routed entry; more: the entries are
+// Routed feed-forward of the rows h2 (first completed by `post` when it names a sublayer's output), added to cur.  Few rows: one GEMV pair per routed entry; more: the entries are
 // listed per expert and every expert multiplies its own rows in one tile launch.
 template <typename T>
-static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_layer& L, const float* h2, float* cur, long ldx, int n, hb_join jn) {
+static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_layer& L, const float* h2, long ldh, const hb_post& post, float* cur, long ldx, int n, hb_join jn) {
     const vox_hybrid_moe& E = *L.moe;
     jn.scale = L.ls2;
     if (L.res_gate) { jn.gate = m->rgate; jn.ldg = m->cfg.width; }
     const int W = m->cfg.width, nE = E.experts + E.identity, top = E.top, ne = n * top, ff = E.ff;
     const int up_down = E.expert_form == VOX_EXPERT_UP_DOWN ? 1 : 0, relu2 = E.expert_act == VOX_ACT_RELU2 ? 1 : 0, nf = up_down ? 1 : 2;
-    hipLaunchKernelGGL(k_hb_moe_router, dim3(n), dim3(256), (size_t)(6 * nE + top + (E.groups > 1 ? E.groups : 0)) * 4, st, h2, (long)W, E.router, E.correction,
+    hipLaunchKernelGGL(k_hb_moe_router, dim3(n), dim3(256), (size_t)(6 * nE + top + (E.groups > 1 ? E.groups : 0)) * 4, st, h2, ldh, E.router, E.correction,
                        W, nE, top, m->moe_sel, m->moe_wgt, E.score_kind == VOX_ROUTER_SIGMOID ? 1 : 0, E.renorm, E.router_bias, E.groups, E.keep,
-                       E.weight_scale != 0.f ? E.weight_scale : 1.0f);
+                       E.weight_scale != 0.f ? E.weight_scale : 1.0f, E.group_best_two, post, post.y ? const_cast<float*>(h2) : (float*)nullptr);
     if (n <= HB_MOE_GEMV_ROWS) {
         const int per = top + (E.shared_ff > 0 ? 1 : 0), maxf = ff > E.shared_ff ? ff : E.shared_ff;
         const hb_moe_small q{m->moe_sel, m->moe_wgt, top, E.experts, ff, E.shared_ff, m->max_eff, E.limit, E.shared_limit, E.act_alpha, E.up_offset,
                              E.scale_input, nullptr, 0, up_down, relu2, jn, L.res_gate ? L.w_gate_ff : nullptr, L.b_gate_ff, m->rgate};
         const int cols = L.res_gate && W > maxf ? W : maxf, per_y = per + (L.res_gate ? 1 : 0);
         if (cols > 0 && per_y > 0 && (E.experts > 0 || E.shared_ff > 0 || L.res_gate))
-            hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((cols + 3) / 4, n * per_y), dim3(256), 0, st, h2, (long)W, (const T*)E.w_gate_up,
+            hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((cols + 3) / 4, n * per_y), dim3(256), 0, st, h2, ldh, (const T*)E.w_gate_up,
                                (const T*)E.shared_gate_up, m->moe_act, W, q);
-        hipLaunchKernelGGL((k_hb_moe_down_combine<T>), dim3((W + 3) / 4, n), dim3(256), 0, st, h2, (long)W, (const T*)E.w_down,
+        hipLaunchKernelGGL((k_hb_moe_down_combine<T>), dim3((W + 3) / 4, n), dim3(256), 0, st, h2, ldh, (const T*)E.w_down,
                            (const T*)E.shared_down, m->moe_act, cur, ldx, W, q);
         return VOX_OK;
     }
-    if (L.res_gate) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, W, (const T*)L.w_gate_ff, L.b_gate_ff, m->rgate, W, n, W, W));
+    if (L.res_gate) VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, ldh, (const T*)L.w_gate_ff, L.b_gate_ff, m->rgate, W, n, W, W));
     if (E.experts > 0) {
         const int cap = m->cfg.max_rows;
         hipLaunchKernelGGL(k_hb_moe_group, dim3(E.experts), dim3(256), 0, st, m->moe_sel, ne, cap, m->moe_list, m->moe_count);
-        VOX_TRY(hb_gemm_tiles<HB_EPI_STORE>(st, h2, (long)W, (const T*)E.w_gate_up, nullptr, m->ff, (long)nf * ff, n, nf * ff, W,
+        VOX_TRY(hb_gemm_tiles<HB_EPI_STORE>(st, h2, ldh, (const T*)E.w_gate_up, nullptr, m->ff, (long)nf * ff, n, nf * ff, W,
                                             hb_rowmap{m->moe_count, m->moe_list, cap, top, (long)nf * ff * W, 0, 0, 0,
                                                       E.scale_input ? m->moe_wgt : (const float*)nullptr, 0.f}, E.experts));
         hipLaunchKernelGGL(k_hb_glu_clamp, dim3(ne, (ff + 1023) / 1024), dim3(256), 0, st, m->ff, m->moe_act, ff, E.limit, E.act_alpha,
@@ -4267,13 +4883,14 @@ static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_layer& L, cons
         VOX_TRY(hb_gemm_tiles<HB_EPI_STORE>(st, m->moe_act, (long)ff, (const T*)E.w_down, nullptr, m->moe_out, (long)W, n, W, ff,
                                             hb_rowmap{m->moe_count, m->moe_list, cap, 1, (long)W * ff, 0, 0, 0}, E.experts));
     }
-    hipLaunchKernelGGL(k_hb_moe_combine, dim3(n), dim3(256), 0, st, cur, ldx, h2, (long)W, m->moe_out, m->moe_sel, m->moe_wgt, top, E.experts, W,
+    hipLaunchKernelGGL(k_hb_moe_combine, dim3(n), dim3(256), 0, st, cur, ldx, h2, ldh, m->moe_out, m->moe_sel, m->moe_wgt, top, E.experts, W,
                        E.scale_input, jn);
     if (E.shared_ff > 0) {
         const int sf = E.shared_ff;
-        VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, W, (const T*)E.shared_gate_up, nullptr, m->ff, nf * sf, n, nf * sf, W));
+        VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, h2, ldh, (const T*)E.shared_gate_up, nullptr, m->ff, nf * sf, n, nf * sf, W));
         hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (sf + 1023) / 1024), dim3(256), 0, st, m->ff, m->moe_act, sf, E.shared_limit, E.act_alpha,
                            (const int*)nullptr, 0, E.up_offset, 0, up_down, relu2);
+        jn.store = 0;      // (the routed sum is there already)
         VOX_TRY(hb_gemm_resid<T>(st, m->moe_act, sf, (const T*)E.shared_down, nullptr, cur, ldx, n, W, sf, jn));
     }
     return VOX_OK;
@@ -4313,52 +4930,63 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
         j2.scale = L.ls2;
         const bool one_norm = L.block == VOX_BLOCK_PARALLEL_ONE_NORM;
         const bool parallel = L.block == VOX_BLOCK_PARALLEL || one_norm;
+        // post-normed layer: a sublayer reads the stream as it is, its output goes to m->y and is normed into the stream
+        const bool post = L.block == VOX_BLOCK_POST_NORM;
+        const int rms = c.norm_kind == VOX_NORM_RMS_GROUPS ? 1 : 0;
+        const hb_post none{}, post1{m->y, W, L.norm1, L.norm1_b, c.eps, rms}, post2{m->y, W, L.norm2, L.norm2_b, c.eps, rms};
+        float* dst = post ? m->y : cur;
+        const long ldd = post ? W : ldx;
+        if (post) j1.store = j2.store = 1;
         // a parallel layer norms x once for both branches before anything is added; a mixer with a sibling needs the normed rows twice
         const float* hn = nullptr;
         if (parallel || L.sibling >= 0) {
-            hb_norm(m, st, n, cur, ldx, nullptr, L.norm1, m->h, parallel && has_ff && !one_norm ? L.norm2 : nullptr, m->h2, (long)W);
+            hb_norm(m, st, n, cur, ldx, nullptr, L.norm1, m->h, parallel && has_ff && !one_norm ? L.norm2 : nullptr, m->h2, (long)W, L.norm1_b, L.norm2_b);
             hn = m->h;
         }
-        const float* hf = one_norm ? m->h : m->h2;      // what the feed-forward of a parallel layer reads
-        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, hn, src, lds_x, cur, ldx, n, n_req, max_kvlen, j1));
+        const float* hf = post ? cur : one_norm ? m->h : m->h2;      // what the feed-forward of a parallel or post-normed layer reads
+        const long ldf = post ? ldx : W;
+        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, post ? cur : hn, post ? ldx : W, src, lds_x, dst, ldd, n, n_req, max_kvlen, j1));
+        if (post && !L.moe) hb_post_norm(st, n, post1, cur, ldx, W);
         if (L.sibling >= 0)
-            VOX_TRY(hb_mixer<T>(m, st, io, m->layers[L.sibling], run.side_cache, run.side_pool, run.side_state, hn, src, lds_x, cur, ldx, n, n_req,
+            VOX_TRY(hb_mixer<T>(m, st, io, m->layers[L.sibling], run.side_cache, run.side_pool, run.side_state, hn, W, src, lds_x, cur, ldx, n, n_req,
                                 max_kvlen, j1));
         if (L.moe) {
-            if (!parallel) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
-            VOX_TRY(hb_moe<T>(m, st, L, hf, cur, ldx, n, j2));
+            if (!parallel && !post) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W, L.norm2_b);
+            VOX_TRY(hb_moe<T>(m, st, L, hf, ldf, post ? post1 : none, dst, ldd, n, j2));
         } else if (L.ff > 0 && L.ff_kind == VOX_FF_GATED) {
             // down(act(gate h + b) * (up h + b)) + b: gate and up rows in one product, the activation in place behind it
-            if (!parallel) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W);
-            const float* hd = parallel ? hf : m->h2;
+            if (!parallel && !post) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W, L.norm2_b);
+            const float* hd = parallel || post ? hf : m->h2;
+            const float limit = L.ff_limit > 0.f ? L.ff_limit : INFINITY, alpha = L.ff_alpha != 0.f ? L.ff_alpha : 1.0f;
             if (n == 1) {
                 // one row: gate and up rows of a column by one wave, biases and activation in its epilogue (the routed feed-forward's
                 // kernel with the dense unit in the place of the shared expert and nothing routed); more rows would stream the matrix
                 // once per row
-                const hb_moe_small q{nullptr, nullptr, 0, 0, 0, L.ff, L.ff, INFINITY, INFINITY, 1.0f, 0.0f, 0, L.b_up, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0,
+                const hb_moe_small q{nullptr, nullptr, 0, 0, 0, L.ff, L.ff, INFINITY, limit, alpha, L.ff_up_offset, 0, L.b_up, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0,
                                      0, 0, {}, nullptr, nullptr, nullptr};
-                hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((L.ff + 3) / 4, n), dim3(256), 0, st, hd, (long)W, (const T*)nullptr, (const T*)L.w_up,
+                hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((L.ff + 3) / 4, n), dim3(256), 0, st, hd, ldf, (const T*)nullptr, (const T*)L.w_up,
                                    m->ff_act, W, q);
             } else {
-                VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hd, W, (const T*)L.w_up, L.b_up, m->ff, 2 * L.ff, n, 2 * L.ff, W));
-                hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (L.ff + 1023) / 1024), dim3(256), 0, st, m->ff, m->ff_act, L.ff, INFINITY, 1.0f,
-                                   (const int*)nullptr, 0, 0.0f, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0, 0, 0);
+                VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hd, ldf, (const T*)L.w_up, L.b_up, m->ff, 2 * L.ff, n, 2 * L.ff, W));
+                hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (L.ff + 1023) / 1024), dim3(256), 0, st, m->ff, m->ff_act, L.ff, limit, alpha,
+                                   (const int*)nullptr, 0, L.ff_up_offset, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0, 0, 0);
             }
-            VOX_TRY(hb_gemm_resid<T>(st, m->ff_act, L.ff, (const T*)L.w_down, L.b_down, cur, ldx, n, W, L.ff, j2));
+            VOX_TRY(hb_gemm_resid<T>(st, m->ff_act, L.ff, (const T*)L.w_down, L.b_down, dst, ldd, n, W, L.ff, j2));
         } else if (L.ff > 0) {
             // up rows with their activation, then (a residual gate) its rows, as one product
             const int nf = L.ff + L.res_gate, epi = L.ff_act == VOX_ACT_RELU2 ? HB_EPI_RELU2 : HB_EPI_GELU;
             hb_rowmap rm = hb_plain();
             rm.epi_arg = (float)L.ff;
-            if (parallel) {
-                VOX_TRY(hb_gemm<T>(st, epi, hf, W, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
-            } else if (!(n == 1 && hb_try_norm_gemv<T>(m, st, epi, src, lds_x, nullptr, L.norm2, (const T*)L.w_up, L.b_up, m->ff, nf, W, rm.epi_arg))) {
-                hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h, nullptr, nullptr, (long)W);
+            if (parallel || post) {
+                VOX_TRY(hb_gemm<T>(st, epi, hf, ldf, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
+            } else if (!(n == 1 && hb_try_norm_gemv<T>(m, st, epi, src, lds_x, nullptr, L.norm2, (const T*)L.w_up, L.b_up, m->ff, nf, W, rm.epi_arg, L.norm2_b))) {
+                hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h, nullptr, nullptr, (long)W, L.norm2_b);
                 VOX_TRY(hb_gemm<T>(st, epi, m->h, W, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
             }
             if (L.res_gate) { j2.gate = m->ff + L.ff; j2.ldg = nf; }
-            VOX_TRY(hb_gemm_resid<T>(st, m->ff, nf, (const T*)L.w_down, nullptr, cur, ldx, n, W, L.ff, j2));
+            VOX_TRY(hb_gemm_resid<T>(st, m->ff, nf, (const T*)L.w_down, nullptr, dst, ldd, n, W, L.ff, j2));
         }
+        if (post && has_ff) hb_post_norm(st, n, post2, cur, ldx, W);
         if (io->trace && S > 0)
             hipLaunchKernelGGL(k_hb_sum_streams, dim3(n), dim3(256), 0, st, cur, S, io->trace + (size_t)ri * c.max_rows * W, (long)W, W);
         else if (io->trace)
@@ -4369,13 +4997,13 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
         const float* last = S > 0 ? m->u : cur;
         const long ld_last = S > 0 ? W : ldx;
         const bool scaled = c.logit_scale != 0.f && c.logit_scale != 1.0f;
-        if (!(n_out == 1 && !(c.logit_softcap > 0.f) &&
-              hb_try_norm_gemv<T>(m, st, scaled ? HB_EPI_SCALE : HB_EPI_STORE, last, ld_last, io->out_rows, m->w.final_norm, (const T*)m->w.head, nullptr,
-                                  io->logits, c.vocab, W, c.logit_scale))) {
-            hb_norm(m, st, n_out, last, ld_last, io->out_rows, m->w.final_norm, m->hout, nullptr, nullptr, (long)W);
-            hb_rowmap rm = hb_plain();
-            rm.epi_arg = c.logit_softcap > 0.f ? c.logit_softcap : c.logit_scale;
-            VOX_TRY(hb_gemm<T>(st, c.logit_softcap > 0.f ? HB_EPI_SOFTCAP : (scaled ? HB_EPI_SCALE : HB_EPI_STORE), m->hout, W, (const T*)m->w.head,
+        const int epi = c.logit_softcap > 0.f ? HB_EPI_SOFTCAP : (scaled ? HB_EPI_SCALE : HB_EPI_STORE);
+        hb_rowmap rm = hb_plain();
+        rm.epi_arg = c.logit_softcap > 0.f ? c.logit_softcap : c.logit_scale;
+        if (!(n_out == 1 && hb_try_norm_gemv<T>(m, st, epi, last, ld_last, io->out_rows, m->w.final_norm, (const T*)m->w.head, nullptr, io->logits, c.vocab,
+                                                W, rm.epi_arg, m->w.final_norm_b))) {
+            hb_norm(m, st, n_out, last, ld_last, io->out_rows, m->w.final_norm, m->hout, nullptr, nullptr, (long)W, m->w.final_norm_b);
+            VOX_TRY(hb_gemm<T>(st, epi, m->hout, W, (const T*)m->w.head,
                                nullptr, io->logits, c.vocab, n_out, c.vocab, W, rm));
         }
     }
@@ -4414,7 +5042,12 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         else if (!L.norm1 || !L.w_in || !L.w_out) bad = "missing weights";
         else if (L.ff > 0 && ((!L.norm2 && L.block != VOX_BLOCK_PARALLEL_ONE_NORM) || !L.w_up || !L.w_down)) bad = "missing feed-forward weights";
         else if (L.ff > 0 && L.ff_kind != VOX_FF_UP_DOWN && L.ff_kind != VOX_FF_GATED) bad = "feed-forward form";
-        else if (L.block != VOX_BLOCK_SEQUENTIAL && L.block != VOX_BLOCK_PARALLEL && L.block != VOX_BLOCK_PARALLEL_ONE_NORM) bad = "block form";
+        else if (L.block != VOX_BLOCK_SEQUENTIAL && L.block != VOX_BLOCK_PARALLEL && L.block != VOX_BLOCK_PARALLEL_ONE_NORM &&
+                 L.block != VOX_BLOCK_POST_NORM) bad = "block form";
+        else if (L.block == VOX_BLOCK_POST_NORM && (L.sibling >= 0 || L.res_gate || cfg->streams > 0 || L.kind == VOX_MIXER_SHIFT_DECAY ||
+                                                    (cfg->norm_kind == VOX_NORM_RMS_GROUPS && cfg->norm_groups != 1)))
+            bad = "post-normed layers: one mixer whose input is one projection, one stream, one norm slice, no residual gate";
+        else if (cfg->norm_kind != VOX_NORM_LAYER && (L.norm1_b || L.norm2_b)) bad = "norm bias: layer norms only";
         else if (L.sibling >= cfg->n_layers || (L.sibling >= 0 && m->layers[L.sibling].sibling >= 0)) bad = "sibling index";
         else if (L.kind == VOX_MIXER_HGRN2 && (!L.lower || !L.head_norm)) bad = "hgrn2 needs lower and head_norm";
         else if (L.kind == VOX_MIXER_MLSTM && (!L.head_norm || !(L.gate_cap > 0.f))) bad = "mlstm needs head_norm and gate_cap";
@@ -4444,6 +5077,9 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         else if (hb_is_attn(L.kind) && L.kind != VOX_MIXER_LATENT_ATTN) {
             if (L.kv_heads < 1 || L.heads % L.kv_heads != 0 || (L.heads / L.kv_heads > 16 && L.kind == VOX_MIXER_POOLED_WINDOW_ATTN))
                 bad = "heads / kv_heads (group of at most 16)";
+            else if (L.kind == VOX_MIXER_WINDOW_ATTN && (!L.q_norm || (!L.kv_shared && !L.k_norm))) bad = "window attention needs q_norm and k_norm";
+            else if (L.kind == VOX_MIXER_WINDOW_ATTN && (L.window < 0 || L.keep_first < 0)) bad = "window attention: window / keep_first";
+            else if (L.kind == VOX_MIXER_WINDOW_ATTN && (L.rot_dims < 0 || L.rot_dims > L.dim || (L.rot_dims & 1) || (L.rot_dims > 0 && !L.inv_freq))) bad = "rot_dims";
             else if (L.kind == VOX_MIXER_SIGMOID_ATTN && (!L.q_norm || !L.k_norm)) bad = "sigmoid attention needs q_norm and k_norm";
             else if (L.kind == VOX_MIXER_SIGMOID_ATTN && (L.chunk < 0 || (L.dist_bias && L.dist_n < 1))) bad = "sigmoid attention: chunk / distance biases";
             else if (hb_conv_attn(L) && (!L.conv_w || (L.qk_norm_whole && (!L.q_norm || !L.k_norm)))) bad = "attention behind a convolution: conv_w / q_norm / k_norm";
@@ -4484,6 +5120,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
         if (L.heads * L.vdim > m->max_mix) m->max_mix = L.heads * L.vdim;
         if ((L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff + L.res_gate > m->max_ff) m->max_ff = (L.ff_kind == VOX_FF_GATED ? 2 : 1) * L.ff + L.res_gate;
         if (L.moe && L.res_gate) m->any_rgate = true;
+        if (L.block == VOX_BLOCK_POST_NORM) m->any_post = true;
         if (L.ff_kind == VOX_FF_GATED && L.ff > m->max_gated) m->max_gated = L.ff;
         if (L.kind == VOX_MIXER_RETENTION) {
             const size_t f = ((size_t)cfg->max_rows / HB_SCAN_CHUNK + cfg->max_batch + 1) * L.heads * ((size_t)L.dim * L.vdim);
@@ -4543,6 +5180,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
              hipMemcpy(m->ones, one, sizeof(one), hipMemcpyHostToDevice) == hipSuccess;
     }
     if (ok && m->any_rgate) ok = hipMalloc((void**)&m->rgate, R * W * 4) == hipSuccess;
+    if (ok && m->any_post) ok = hipMalloc((void**)&m->y, R * W * 4) == hipSuccess;
     if (ok && m->any_shift) ok = hipMalloc((void**)&m->shift, 5 * R * W * 4) == hipSuccess;
     if (ok && m->max_gated) ok = hipMalloc((void**)&m->ff_act, R * (size_t)m->max_gated * 4) == hipSuccess;
     if (ok && m->scan_ws_floats && cfg->max_rows > HB_SCAN_CHUNK) ok = hipMalloc((void**)&m->scan_ws, m->scan_ws_floats * 4) == hipSuccess;
@@ -4562,6 +5200,10 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
             const int max_keys = L.chunk > 0 && L.chunk < cfg->max_seq_len ? L.chunk : cfg->max_seq_len;
             const size_t b = (size_t)HB_ATTN_SEG_ROWS * L.heads * hb_sig_segments(max_keys) * L.vdim * 4;
             if (b > m->attn_ws_bytes) m->attn_ws_bytes = b;
+        } else if (L.kind == VOX_MIXER_WINDOW_ATTN) {
+            const int nchunks = (hb_win_keys(L, cfg->max_seq_len) + 63) / 64;
+            const size_t b = (size_t)HB_ATTN_SEG_ROWS * L.heads * (nchunks < HB_SIG_MAX_SEG ? nchunks : HB_SIG_MAX_SEG) * (L.vdim + 2) * 4;
+            if (b > m->attn_ws_bytes) m->attn_ws_bytes = b;
         } else if (hb_is_attn(L.kind)) {
             const bool causal = L.kind == VOX_MIXER_CAUSAL_ATTN, latent = L.kind == VOX_MIXER_LATENT_ATTN;
             const int max_keys = causal || (latent && L.window < 1) ? cfg->max_seq_len
@@ -4580,7 +5222,7 @@ int vox_hybrid_create(vox_ctx* ctx, const vox_hybrid_config* cfg, const vox_hybr
 void vox_hybrid_destroy(vox_hybrid* m) {
     if (!m) return;
     (void)hipFree(m->xa); (void)hipFree(m->xb); (void)hipFree(m->h); (void)hipFree(m->h2); (void)hipFree(m->proj); (void)hipFree(m->mix);
-    (void)hipFree(m->ff); (void)hipFree(m->ff_act); (void)hipFree(m->u); (void)hipFree(m->ones); (void)hipFree(m->rgate); (void)hipFree(m->hout); (void)hipFree(m->logits16); (void)hipFree(m->attn_ws); (void)hipFree(m->shift); (void)hipFree(m->scan_ws);
+    (void)hipFree(m->ff); (void)hipFree(m->ff_act); (void)hipFree(m->u); (void)hipFree(m->y); (void)hipFree(m->ones); (void)hipFree(m->rgate); (void)hipFree(m->hout); (void)hipFree(m->logits16); (void)hipFree(m->attn_ws); (void)hipFree(m->shift); (void)hipFree(m->scan_ws);
     (void)hipFree(m->moe_wgt); (void)hipFree(m->moe_sel); (void)hipFree(m->moe_act); (void)hipFree(m->moe_out);
     (void)hipFree(m->moe_list); (void)hipFree(m->moe_count);
     delete m;

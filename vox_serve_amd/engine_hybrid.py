@@ -2,9 +2,9 @@
 diagonal unit behind a short convolution, a matrix state with token shift and per-channel decay, retention with a fixed decay
 per head, the gated delta rule behind short convolutions) and with attention over a paged cache (a sliding window with pooled
 history, plain causal attention with normed q / k / v -- optionally behind a short convolution, rotated, with a softmax sink --, or
-attention whose keys and values are expanded from a cached low-rank latent, or attention with independent sigmoid weights inside
-position chunks), optionally two mixers side by side, sequential or parallel layers with an optional layer scale or a residual gate, one
-residual stream or several mixed at every sublayer, a dense or a routed feed-forward, and a range of layers looped over shared weights.
+attention whose keys and values are expanded from a cached low-rank latent, attention with independent sigmoid weights inside
+position chunks, or softmax attention over a window and the first tokens, optionally on an earlier layer's keys and values), optionally two
+mixers side by side, sequential, parallel or post-normed layers with an optional layer scale or a residual gate, one residual stream or several mixed at every sublayer, a dense or a routed feed-forward, and a range of layers looped over shared weights.
 
 It reuses the plan / stream / hipGraph machinery of the other LM engines (`Qwen3Engine`): one pinned int32 plan block per
 step, decode steps captured per batch size.  Beyond the K / V pages that the worker hands out, every request holds one
@@ -24,13 +24,13 @@ from . import _native as N
 from .engine import Qwen3Engine
 
 MIXER_HGRN2, MIXER_POOLED_WINDOW_ATTN, MIXER_MLSTM, MIXER_RGLRU, MIXER_CAUSAL_ATTN, MIXER_SHIFT_DECAY = 0, 1, 2, 3, 4, 5
-MIXER_LATENT_ATTN, MIXER_RETENTION, MIXER_DELTA, MIXER_SIGMOID_ATTN = 6, 7, 8, 9
+MIXER_LATENT_ATTN, MIXER_RETENTION, MIXER_DELTA, MIXER_SIGMOID_ATTN, MIXER_WINDOW_ATTN = 6, 7, 8, 9, 10
 MIXER_KINDS = {"hgrn2": MIXER_HGRN2, "attention": MIXER_POOLED_WINDOW_ATTN, "mlstm": MIXER_MLSTM, "rglru": MIXER_RGLRU,
                "causal_attention": MIXER_CAUSAL_ATTN, "shift_decay": MIXER_SHIFT_DECAY, "latent_attention": MIXER_LATENT_ATTN,
-               "retention": MIXER_RETENTION, "delta": MIXER_DELTA, "sigmoid_attention": MIXER_SIGMOID_ATTN}
-ATTENTION_KINDS = ("attention", "causal_attention", "latent_attention", "sigmoid_attention")
+               "retention": MIXER_RETENTION, "delta": MIXER_DELTA, "sigmoid_attention": MIXER_SIGMOID_ATTN, "window_attention": MIXER_WINDOW_ATTN}
+ATTENTION_KINDS = ("attention", "causal_attention", "latent_attention", "sigmoid_attention", "window_attention")
 NORM_KINDS = {"layer": 0, "rms_groups": 1}
-BLOCK_FORMS = {"sequential": 0, "parallel": 1, "parallel_one_norm": 2}
+BLOCK_FORMS = {"sequential": 0, "parallel": 1, "parallel_one_norm": 2, "post_norm": 3}
 FF_KINDS = {"up_down": 0, "gated": 1}
 ACT_KINDS = {"gelu_tanh": 0, "swish": 1, "relu2": 2}
 ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
@@ -59,6 +59,7 @@ class MoECfg:
     groups: int = 0                 # > 1: equal groups of neighbouring experts, of which the `keep` best (by their best score) can be chosen from
     keep: int = 0
     weight_scale: float = 1.0       # multiplies the weights
+    group_best_two: bool = False    # a group's score is the sum of its two largest choice values (else its largest)
 
 
 @dataclass
@@ -68,7 +69,7 @@ class MixerCfg:
     dim: int                        # rglru: channels per block
     vdim: int                       # rglru, shift_decay: = dim
     kv_heads: int = 0               # attention
-    window: int = 0                 # attention: tokens a position sees, itself included
+    window: int = 0                 # attention: tokens a position sees, itself included (window attention: 0 for all)
     pool: int = 0                   # attention: tokens per pooled block
     rot_dims: int = 0
     rot_base: float = 10000.0
@@ -86,6 +87,7 @@ class MixerCfg:
     out_scale: float = 1.0          # the mixer's output is multiplied by this before it joins the residual sum
     block: str = "sequential"       # "sequential": x += mixer(norm1 x); x += ff(norm2 x) | "parallel": x += mixer(norm1 x) + ff(norm2 x)
                                     # | "parallel_one_norm": x += mixer(n) + ff(n), n = norm1 x
+                                    # | "post_norm": x += norm1 mixer(x); x += norm2 ff(x)
     ff_kind: str = "up_down"        # dense feed-forward: "up_down" down(gelu(up h)) | "gated" down(act(gate h + b) * (up h + b)) + b
     ff_act: str = "gelu_tanh"       # activation of the gated form ("gelu_tanh" | "swish"); "relu2": the up_down form with the square of relu
     q_rank: int = 0                 # latent attention: width of the query latent (0: none, the query is projected from the normed row)
@@ -102,7 +104,12 @@ class MixerCfg:
     chunk: int = 0                  # sigmoid attention: tokens per position chunk (0: every earlier token is seen)
     score_cap: float = 0.0          # sigmoid attention: soft cap of the scaled scores (0: none)
     dist_max: int = 0               # sigmoid attention: distance from which the last row of the bias table applies (0: no distance bias)
-    out_gate: bool = False          # sigmoid attention: a sigmoid gate per output column
+    out_gate: bool = False          # sigmoid, window attention: a sigmoid gate per output column
+    keep_first: int = 0             # window attention: first tokens of the sequence that stay visible behind the window
+    kv_from: Optional[int] = None   # window attention: the layer whose keys and values are used instead of own ones
+    ff_limit: float = 0.0           # gated dense form: min(gate, limit), clamp(up, -limit, limit) (0: not clamped)
+    ff_alpha: float = 1.0           # gated dense form with "swish": g * sigmoid(alpha g)
+    ff_up_offset: float = 0.0       # gated dense form: the activation is multiplied by up + offset
     res_gate: bool = False          # sublayer results are multiplied by sigmoid(W n + b) before they join the residual sum
     side: Optional["MixerCfg"] = None   # a second mixer on the same normed input, added to the same sum
     moe: Optional[MoECfg] = None    # routed feed-forward (instead of the dense one)
@@ -113,6 +120,8 @@ class MixerCfg:
         h, d, v = self.heads, self.dim, self.vdim
         if self.kind == "sigmoid_attention":
             return h * d + self.kv_heads * (d + v) + (h * v if self.out_gate else 0)
+        if self.kind == "window_attention":
+            return h * d + (0 if self.kv_from is not None else self.kv_heads * (d + v)) + (h * v if self.out_gate else 0)
         if self.kind == "hgrn2":
             return 2 * h * d + h * v
         if self.kind == "attention":
@@ -136,6 +145,8 @@ class MixerCfg:
         """Values one token leaves in the paged cache of an attention mixer."""
         if self.kind == "latent_attention":
             return self.kv_rank + self.rot_dim
+        if self.kv_from is not None:
+            return 0
         return self.kv_heads * (self.dim + self.vdim) if self.kind in ATTENTION_KINDS else 0
 
     def state_floats(self, width: int) -> int:
@@ -183,7 +194,7 @@ class HybridMoEC(ctypes.Structure):
                [(n, ctypes.c_void_p) for n in ("router", "correction", "w_gate_up", "w_down", "shared_gate_up", "shared_down")] + \
                [(n, ctypes.c_int32) for n in ("score_kind", "renorm", "scale_input")] + [("up_offset", ctypes.c_float)] + \
                [("expert_form", ctypes.c_int32), ("expert_act", ctypes.c_int32), ("router_bias", ctypes.c_void_p),
-                ("groups", ctypes.c_int32), ("keep", ctypes.c_int32), ("weight_scale", ctypes.c_float)]
+                ("groups", ctypes.c_int32), ("keep", ctypes.c_int32), ("weight_scale", ctypes.c_float), ("group_best_two", ctypes.c_int32)]
 
 
 class HybridLayerC(ctypes.Structure):
@@ -209,7 +220,9 @@ class HybridLayerC(ctypes.Structure):
                 ("head_temp", ctypes.c_void_p), ("dist_bias", ctypes.c_void_p), ("weight_bias", ctypes.c_void_p),
                 ("no_head_gate", ctypes.c_int32), ("rot_mag", ctypes.c_float), ("sinks", ctypes.c_void_p),
                 ("res_gate", ctypes.c_int32), ("w_gate_ff", ctypes.c_void_p), ("b_gate_ff", ctypes.c_void_p),
-                ("hc_in", ctypes.c_void_p * 2), ("hc_out", ctypes.c_void_p * 2), ("hc_mix", ctypes.c_void_p * 2)]
+                ("hc_in", ctypes.c_void_p * 2), ("hc_out", ctypes.c_void_p * 2), ("hc_mix", ctypes.c_void_p * 2),
+                ("keep_first", ctypes.c_int32), ("kv_shared", ctypes.c_int32), ("norm1_b", ctypes.c_void_p), ("norm2_b", ctypes.c_void_p),
+                ("ff_limit", ctypes.c_float), ("ff_alpha", ctypes.c_float), ("ff_up_offset", ctypes.c_float)]
 
 
 class HybridRunC(ctypes.Structure):
@@ -228,7 +241,7 @@ class HybridConfigC(ctypes.Structure):
 
 class HybridWeightsC(ctypes.Structure):
     _fields_ = [("layers", ctypes.POINTER(HybridLayerC)), ("runs", ctypes.POINTER(HybridRunC))] + \
-               [(n, ctypes.c_void_p) for n in ("embedding", "loop_in", "head", "final_norm", "bigram", "prev_token")]
+               [(n, ctypes.c_void_p) for n in ("embedding", "loop_in", "head", "final_norm", "bigram", "prev_token", "final_norm_b")]
 
 
 class HybridIO(ctypes.Structure):
@@ -273,7 +286,7 @@ def distance_bias(table: torch.Tensor, dist_max: int, longest: int) -> torch.Ten
     return table.float()[torch.tensor([bucket(d) for d in range(n)])].t().contiguous()
 
 
-ROTARY_KINDS = ("attention", "latent_attention", "retention", "causal_attention")
+ROTARY_KINDS = ("attention", "latent_attention", "retention", "causal_attention", "window_attention")
 
 
 def reduced_bigram(bigram) -> tuple:
@@ -291,7 +304,7 @@ class HybridEngine(Qwen3Engine):
     """`weights`: {"embedding", "head", "final_norm", "loop_in" (or None), "layers": [per layer dict with norm1, norm2, w_in,
     b_in, w_out, lower, head_norm, w_up, w_down, b_up, b_down; per mixer kind also q_norm, k_norm | conv_w, conv_b, w_gates, b_gates,
     lam | shift_mu, w_decay2, decay0, bonus | w_uq, w_ukT, w_uv, q_lat_norm, kv_lat_norm | conv_w, w_decay2, w_gate2, a_log, dt_bias
-    (delta rule) | q_norm, k_norm, head_temp, dist_table, weight_bias (sigmoid attention) | sinks (latent attention); ls1, ls2 (layer scale);
+    (delta rule) | q_norm, k_norm, head_temp, dist_table, weight_bias (sigmoid attention) | sinks (latent, window attention); norm1_b, norm2_b and beside final_norm final_norm_b (biases of layer norms); ls1, ls2 (layer scale);
     w_gate_in, b_gate_in, w_gate_ff, b_gate_ff (residual gates of the mixer and of the feed-forward); hc_in, hc_out, hc_mix (several streams:
     [mixer's, feed-forward's]); "moe": {router, router_bias, correction, w_gate_up (up rows only in the up / down form),
     w_down, shared_gate_up, shared_down}; "side": the same mixer keys for a sibling mixer], "bigram" (or None)} — matrices in any
@@ -365,6 +378,9 @@ class HybridEngine(Qwen3Engine):
             c.kind, c.heads, c.kv_heads, c.dim, c.vdim = MIXER_KINDS[m.kind], m.heads, m.kv_heads, m.dim, m.vdim
             c.window, c.pool, c.rot_dims, c.scale, c.gate_cap, c.ff = m.window, m.pool, m.rot_dims, m.scale, m.gate_cap, m.ff
             c.norm1, c.norm2 = norm_w(lw["norm1"]), norm_w(lw.get("norm2"))
+            c.norm1_b, c.norm2_b = vec(lw.get("norm1_b")), vec(lw.get("norm2_b"))
+            c.keep_first, c.kv_shared = m.keep_first, int(m.kv_from is not None)
+            c.ff_limit, c.ff_alpha, c.ff_up_offset = m.ff_limit, m.ff_alpha, m.ff_up_offset
             c.ls1, c.ls2 = vec(lw.get("ls1")), vec(lw.get("ls2"))
             c.qk_norm_whole, c.sink = int(m.qk_norm_whole), int(m.sink)
             c.decay_channels, c.gate_rank, c.gate_act = int(m.decay_channels), m.gate_rank, GATE_KINDS[m.gate_act]
@@ -399,7 +415,7 @@ class HybridEngine(Qwen3Engine):
                                 vec(ew["router"]), vec(ew.get("correction")), mat(ew.get("w_gate_up")), mat(ew.get("w_down")),
                                 mat(ew.get("shared_gate_up")), mat(ew.get("shared_down")), ROUTER_SCORES[e.score], int(e.renorm),
                                 int(e.scale_input), e.up_offset, EXPERT_FORMS[e.expert_form], ACT_KINDS[e.expert_act],
-                                vec(ew.get("router_bias")) if e.router_bias else None, e.groups, e.keep, e.weight_scale)
+                                vec(ew.get("router_bias")) if e.router_bias else None, e.groups, e.keep, e.weight_scale, int(e.group_best_two))
                 self._moes.append(mc)
                 c.moe = ctypes.pointer(mc)
 
@@ -432,11 +448,21 @@ class HybridEngine(Qwen3Engine):
             self.states.append(st)
             return None, None, st.data_ptr()
 
+        latest = {}                 # layer index -> its last run so far
         for j, (li, loop_in) in enumerate(runs):
             m = cfg.layers[li]
+            if m.kv_from is not None:
+                src = cfg.layers[m.kv_from] if 0 <= m.kv_from < len(cfg.layers) else None
+                if m.kv_from not in latest or m.kind != "window_attention" or src.kind != m.kind or src.kv_from is not None or \
+                        (src.kv_heads, src.dim, src.vdim) != (m.kv_heads, m.dim, m.vdim):
+                    raise ValueError(f"layer {li}: cannot use the keys and values of layer {m.kv_from}")
             # a loop without an input matrix just runs the range again: nothing happens between the passes
             rarr[j].layer, rarr[j].loop_in = li, int(loop_in and weights.get("loop_in") is not None)
-            rarr[j].cache, rarr[j].pool, rarr[j].state = storage(m)
+            if m.kv_from is not None:
+                rarr[j].cache = rarr[latest[m.kv_from]].cache
+            else:
+                rarr[j].cache, rarr[j].pool, rarr[j].state = storage(m)
+            latest[li] = j
             if m.side is not None:
                 rarr[j].side_cache, rarr[j].side_pool, rarr[j].side_state = storage(m.side)
         self.n_runs = len(runs)
@@ -452,7 +478,7 @@ class HybridEngine(Qwen3Engine):
         head = emb if weights["head"] is weights["embedding"] else mat(weights["head"])      # a tied head shares the table
         cw = HybridWeightsC(ctypes.cast(larr, ctypes.POINTER(HybridLayerC)), ctypes.cast(rarr, ctypes.POINTER(HybridRunC)),
                             emb, mat(weights.get("loop_in")), head, norm_w(weights["final_norm"]),
-                            mat(weights.get("bigram")) if cfg.bigram else None, self.prev_token.data_ptr())
+                            mat(weights.get("bigram")) if cfg.bigram else None, self.prev_token.data_ptr(), vec(weights.get("final_norm_b")))
         self._larr, self._rarr = larr, rarr
         h = ctypes.c_void_p()
         N.check(L.vox_hybrid_create(self.ctx, ctypes.byref(cc), ctypes.byref(cw), ctypes.byref(h)))

@@ -210,6 +210,13 @@ def _gaparax(model_name, device="cuda:0", weights=None, checkpoint_dir=None, syn
     return _hybrid_lm(".gaparax", "GaparaxModel", model_name, device, weights, checkpoint_dir, synthetic, config, kw)
 
 
+@register_model("kazozen")
+def _kazozen(model_name, device="cuda:0", weights=None, checkpoint_dir=None, synthetic=False, config=None, **kw):
+    """Post-normed LM of window attention with kept first tokens, keys and values shared between layers, clamped gated units and
+    group-limited sigmoid routing."""
+    return _hybrid_lm(".kazozen", "KazozenModel", model_name, device, weights, checkpoint_dir, synthetic, config, kw)
+
+
 def load_checkpoint_dir(path: str, device: str = "cuda:0", **kw):
     """A local checkpoint folder whose config.json names its architecture: the registry entry of that name loads it."""
     import json

@@ -755,8 +755,15 @@ def main():
     ap.add_argument("--gaparax", action="store_true", help="instead of the default workload: prefill / decode throughput of the Gaparax "
                     "design (random weights) beside Dipivik, the closest existing model, on the same engine at equal width and depth "
                     "(tools/bench_gaparax.py); prints that comparison as one JSON line")
+    ap.add_argument("--kazozen", action="store_true", help="instead of the default workload: prefill / decode throughput of the Kazozen "
+                    "design (random weights) beside Gaparax, the closest existing model, on the same engine at equal width and depth "
+                    "(tools/bench_kazozen.py); prints that comparison as one JSON line")
     args = ap.parse_args()
 
+    if args.kazozen:
+        from tools.bench_kazozen import run as run_kazozen
+        print(json.dumps(run_kazozen(steps=min(args.steps, 50), warmup=min(args.warmup, 10))))
+        return
     if args.gaparax:
         from tools.bench_gaparax import run as run_gaparax
         print(json.dumps(run_gaparax(steps=min(args.steps, 50), warmup=min(args.warmup, 10))))

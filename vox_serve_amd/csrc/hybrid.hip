@@ -98,6 +98,11 @@ template <int EPI> __device__ __forceinline__ void hb_epilogue(float* c, float a
 __device__ __forceinline__ float hb_gelu_tanh(float z) {
     return 0.5f * z * (1.0f + tanhf(0.79788456080286535588f * (z + 0.044715f * z * z * z)));
 }
+// act(g) * (u + up_offset), g = min(gate, limit), u = clamp(up, -limit, limit); act(g) = g * sigmoid(alpha g), or the tanh form of gelu
+__device__ __forceinline__ float hb_glu(float g0, float u0, float limit, float alpha, float up_offset, int gelu) {
+    const float g = fminf(g0, limit), u = fminf(fmaxf(u0, -limit), limit);
+    return (gelu ? hb_gelu_tanh(g) : g * hb_sigmoid(alpha * g)) * (u + up_offset);
+}
 // How a sublayer's result v joins the residual stream at (row, col): v is multiplied by sigmoid(gate logit) and by a layer scale where
 // they are given; then x += v, or -- several streams -- x_t <- sum_s mix[s*streams + t] x_s + out[t] v for all streams at once, and
 // u = sum_t next[t] x_t, what the next sublayer (or the head: all ones) reads, is left beside them.  Streams of a row lie `sld` apart.
@@ -308,7 +313,7 @@ static void hb_layernorm(hipStream_t st, int n, const float* x, long ldx, const 
 }
 
 // ---- norm of a sublayer's output, added to the residual row: x += norm(y) * w + b ------------------------------------------------
-// The layer norm above, or (rms) the RMS norm over the row; 256 threads per row.  NV > 0: the row (width <= 256 * NV) stays in registers.
+// The layer norm, or (rms) the RMS norm over the row; 256 threads per row.
 struct hb_post {
     const float* y;         // [rows][ldy] the sublayer's output (NULL: nothing to do)
     long ldy;
@@ -316,63 +321,91 @@ struct hb_post {
     float eps;
     int rms;
 };
-template <int NV> __device__ __forceinline__ void hb_post_norm_row(const hb_post& p, int row, float* xr, int W, float (*red)[4]) {
+// NC > 0: rows of at most 1024 * NC columns whose operands lie on 16-byte boundaries; thread t owns the columns 4t .. 4t+3 of every 1024,
+// everything is requested at the start and the new row stays in its registers (out) as well as in xo (NULL: not written)
+template <int NC> __device__ __forceinline__ void hb_post_row(const hb_post& p, int row, const float* xr, float* xo, int W, float (*red)[4], float4 (&out)[NC]) {
     const float* yr = p.y + (size_t)row * p.ldy;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
-    float yv[NV > 0 ? NV : 1];
-    float s = 0.f, q = 0.f;
-    if (NV > 0) {
+    float4 y[NC], g[NC], b[NC];
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int k = threadIdx.x + i * 256;
-            yv[i] = k < W ? yr[k] : 0.f;
-        }
-#pragma unroll
-        for (int i = 0; i < NV; ++i) s += yv[i];
-    } else {
-        for (int i = threadIdx.x; i < W; i += 256) s += yr[i];
+    for (int i = 0; i < NC; ++i) {
+        const int k = threadIdx.x * 4 + 1024 * i, kc = k < W ? k : 0;
+        y[i] = *(const float4*)(yr + kc);
+        out[i] = *(const float4*)(xr + kc);
+        g[i] = *(const float4*)(p.w + kc);
+        b[i] = p.b ? *(const float4*)(p.b + kc) : make_float4(0.f, 0.f, 0.f, 0.f);
+        if (k >= W) y[i] = make_float4(0.f, 0.f, 0.f, 0.f);
     }
     float mean = 0.f;
     if (!p.rms) {
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) { s += y[i].x; s += y[i].y; s += y[i].z; s += y[i].w; }
         s = hb_wave_sum(s);
         if (lane == 0) red[0][wv] = s;
         __syncthreads();
         mean = (((red[0][0] + red[0][1]) + red[0][2]) + red[0][3]) / (float)W;
     }
-    if (NV > 0) {
+    float q = 0.f;
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const float d = threadIdx.x + i * 256 < W ? yv[i] - mean : 0.f;
-            q += d * d;
+    for (int i = 0; i < NC; ++i)
+        if ((int)threadIdx.x * 4 + 1024 * i < W) {
+            y[i].x -= mean; y[i].y -= mean; y[i].z -= mean; y[i].w -= mean;
+            q += y[i].x * y[i].x; q += y[i].y * y[i].y; q += y[i].z * y[i].z; q += y[i].w * y[i].w;
         }
-    } else {
-        for (int i = threadIdx.x; i < W; i += 256) {
-            const float d = yr[i] - mean;
-            q += d * d;
-        }
+    q = hb_wave_sum(q);
+    if (lane == 0) red[1][wv] = q;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((((red[1][0] + red[1][1]) + red[1][2]) + red[1][3]) / (float)W + p.eps);
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+        const int k = threadIdx.x * 4 + 1024 * i;
+        out[i].x += y[i].x * inv * g[i].x + b[i].x;
+        out[i].y += y[i].y * inv * g[i].y + b[i].y;
+        out[i].z += y[i].z * inv * g[i].z + b[i].z;
+        out[i].w += y[i].w * inv * g[i].w + b[i].w;
+        if (xo && k < W) *(float4*)(xo + k) = out[i];
+    }
+}
+// any width and alignment, in place
+__device__ __forceinline__ void hb_post_row_any(const hb_post& p, int row, float* xr, int W, float (*red)[4]) {
+    const float* yr = p.y + (size_t)row * p.ldy;
+    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    float s = 0.f, q = 0.f, mean = 0.f;
+    if (!p.rms) {
+        for (int i = threadIdx.x; i < W; i += 256) s += yr[i];
+        s = hb_wave_sum(s);
+        if (lane == 0) red[0][wv] = s;
+        __syncthreads();
+        mean = (((red[0][0] + red[0][1]) + red[0][2]) + red[0][3]) / (float)W;
+    }
+    for (int i = threadIdx.x; i < W; i += 256) {
+        const float d = yr[i] - mean;
+        q += d * d;
     }
     q = hb_wave_sum(q);
     if (lane == 0) red[1][wv] = q;
     __syncthreads();
     const float inv = 1.0f / sqrtf((((red[1][0] + red[1][1]) + red[1][2]) + red[1][3]) / (float)W + p.eps);
-    if (NV > 0) {
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int k = threadIdx.x + i * 256;
-            if (k < W) xr[k] += (yv[i] - mean) * inv * p.w[k] + (p.b ? p.b[k] : 0.f);
-        }
-    } else {
-        for (int i = threadIdx.x; i < W; i += 256) xr[i] += (yr[i] - mean) * inv * p.w[i] + (p.b ? p.b[i] : 0.f);
-    }
+    for (int i = threadIdx.x; i < W; i += 256) xr[i] += (yr[i] - mean) * inv * p.w[i] + (p.b ? p.b[i] : 0.f);
 }
-template <int NV> __global__ __launch_bounds__(256) void k_hb_post_norm(hb_post p, float* x, long ldx, int W) {
+// 1024-column pieces of the register form (1, 2, 4), or 0: the general form
+static int hb_post_pieces(const hb_post& p, const float* x, long ldx, int W) {
+    if ((W & 3) || (ldx & 3) || (p.ldy & 3) || W > 4096 || (((size_t)p.y | (size_t)x | (size_t)p.w | (size_t)p.b) & 15)) return 0;
+    return W <= 1024 ? 1 : (W <= 2048 ? 2 : 4);
+}
+template <int NC> __global__ __launch_bounds__(256) void k_hb_post_norm(hb_post p, float* x, long ldx, int W) {
     __shared__ float red[2][4];
-    hb_post_norm_row<NV>(p, blockIdx.x, x + (size_t)blockIdx.x * ldx, W, red);
+    float* xr = x + (size_t)blockIdx.x * ldx;
+    if constexpr (NC > 0) {
+        float4 out[NC];
+        hb_post_row<NC>(p, blockIdx.x, xr, xr, W, red, out);
+    } else hb_post_row_any(p, blockIdx.x, xr, W, red);
 }
 static void hb_post_norm(hipStream_t st, int n, const hb_post& p, float* x, long ldx, int W) {
-    if (W <= 1024) hipLaunchKernelGGL(k_hb_post_norm<4>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
-    else if (W <= 4096) hipLaunchKernelGGL(k_hb_post_norm<16>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
-    else hipLaunchKernelGGL(k_hb_post_norm<0>, dim3(n), dim3(256), 0, st, p, x, ldx, W);
+    const int nc = hb_post_pieces(p, x, ldx, W);
+    auto kern = nc == 1 ? k_hb_post_norm<1> : nc == 2 ? k_hb_post_norm<2> : nc == 4 ? k_hb_post_norm<4> : k_hb_post_norm<0>;
+    hipLaunchKernelGGL(kern, dim3(n), dim3(256), 0, st, p, x, ldx, W);
 }
 
 // ---- RMS norm over `groups` equal consecutive slices of the row, fp32; optional row gather; one or two weights --------------
@@ -874,6 +907,99 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
 #undef HB_LN
 #undef HB_LN2
     return true;
+}
+
+// One-row steps of post-normed layers: the row is completed (x_out = x + norm(y), hb_post_row) in front of the product that reads it.  Every
+// block takes the row itself -- 256 threads, each requesting its columns and the wave its two weight rows at the start --, keeps it in LDS as the
+// product's operand, and block 0 also stores it.  x_out must not be x: other blocks still read it.  GLU: the wave's rows are gate row n
+// and up row N + n, the result is their activated product (hb_glu); else rows 2n and 2n + 1.
+template <typename T, int GLU, int NC>
+__global__ __launch_bounds__(256) void k_hb_post_gemv(hb_post p, const float* x, float* x_out, const T* Wt, const float* bias, float* C, int N, int K,
+                                                      float limit, float alpha, float up_offset, int gelu) {
+    constexpr int CH = sizeof(T) == 2 ? 8 : 4, NK = 1024 * NC / (64 * CH);
+    __shared__ float red[2][4];
+    __shared__ __attribute__((aligned(16))) float xs[1024 * NC];
+    const int lane = threadIdx.x & 63, n = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int r0 = GLU ? n : 2 * n, r1 = GLU ? N + n : 2 * n + 1, rows = GLU ? 2 * N : N;
+    const bool ok0 = GLU ? n < N : r0 < N, ok1 = GLU ? n < N : r1 < N;
+    const T *w0 = Wt + (size_t)(ok0 ? r0 : rows - 1) * K, *w1 = Wt + (size_t)(ok1 ? r1 : rows - 1) * K;
+    uint4 wr0[NK], wr1[NK];
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+        const int k = (lane + 64 * i) * CH, kc = k < K ? k : 0;
+        wr0[i] = *(const uint4*)(w0 + kc);
+        wr1[i] = *(const uint4*)(w1 + kc);
+    }
+    float4 out[NC];
+    hb_post_row<NC>(p, 0, x, blockIdx.x == 0 ? x_out : nullptr, K, red, out);
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+        *(float4*)(xs + threadIdx.x * 4 + 1024 * i) = make_float4(hb_operand<T>(out[i].x), hb_operand<T>(out[i].y), hb_operand<T>(out[i].z), hb_operand<T>(out[i].w));
+    __syncthreads();
+    float a0 = 0.f, a1 = 0.f;
+    auto unpack = [](const uint4& u, float (&w)[CH]) {
+        if constexpr (sizeof(T) == 2) {
+            w[0] = bflo(u.x); w[1] = bfhi(u.x); w[2] = bflo(u.y); w[3] = bfhi(u.y);
+            w[4] = bflo(u.z); w[5] = bfhi(u.z); w[6] = bflo(u.w); w[7] = bfhi(u.w);
+        } else {
+            w[0] = __uint_as_float(u.x); w[1] = __uint_as_float(u.y); w[2] = __uint_as_float(u.z); w[3] = __uint_as_float(u.w);
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+        const int k = (lane + 64 * i) * CH;
+        if (k < K) {
+            float u[CH], v[CH];
+            unpack(wr0[i], u);
+            unpack(wr1[i], v);
+#pragma unroll
+            for (int e = 0; e < CH; e += 4) {
+                const float4 x4 = *(const float4*)(xs + k + e);
+                a0 = fmaf(u[e], x4.x, a0); a0 = fmaf(u[e + 1], x4.y, a0); a0 = fmaf(u[e + 2], x4.z, a0); a0 = fmaf(u[e + 3], x4.w, a0);
+                a1 = fmaf(v[e], x4.x, a1); a1 = fmaf(v[e + 1], x4.y, a1); a1 = fmaf(v[e + 2], x4.z, a1); a1 = fmaf(v[e + 3], x4.w, a1);
+            }
+        }
+    }
+    a0 = hb_wave_sum(a0);
+    a1 = hb_wave_sum(a1);
+    if (lane != 0) return;
+    if (bias) {
+        if (ok0) a0 += bias[r0];
+        if (ok1) a1 += bias[r1];
+    }
+    if (GLU) {
+        if (ok0) C[n] = hb_glu(a0, a1, limit, alpha, up_offset, gelu);
+    } else {
+        if (ok0) C[r0] = a0;
+        if (ok1) C[r1] = a1;
+    }
+}
+// A normed sublayer output that is still to join x: the next reader of a one-row step completes the row on the way (into x_next), every other
+// reader has it completed in place first.
+struct hb_pending {
+    hb_post p;          // p.y NULL: nothing pending
+    float *x, *x_next;
+    long ldx;
+};
+// true: the product was launched with the pending norm in front of it; x and x_next have changed places
+template <typename T>
+static bool hb_try_post_gemv(hipStream_t st, hb_pending& pd, bool glu, const T* Wt, const float* bias, float* C, int N, int K, float limit = INFINITY,
+                             float alpha = 1.f, float up_offset = 0.f, int gelu = 0) {
+    const int nc = hb_post_pieces(pd.p, pd.x, pd.ldx, K);
+    if (!nc || (K & 7) || ((size_t)Wt & 15) || ((size_t)pd.x_next & 15)) return false;
+    const dim3 g(glu ? (N + 3) / 4 : (N + 7) / 8), b(256);
+#define HB_PG(G_, NC_) \
+    hipLaunchKernelGGL((k_hb_post_gemv<T, G_, NC_>), g, b, 0, st, pd.p, pd.x, pd.x_next, Wt, bias, C, N, K, limit, alpha, up_offset, gelu)
+    if (glu) { if (nc == 1) HB_PG(1, 1); else if (nc == 2) HB_PG(1, 2); else HB_PG(1, 4); }
+    else { if (nc == 1) HB_PG(0, 1); else if (nc == 2) HB_PG(0, 2); else HB_PG(0, 4); }
+#undef HB_PG
+    float* t = pd.x; pd.x = pd.x_next; pd.x_next = t;
+    pd.p.y = nullptr;
+    return true;
+}
+static void hb_settle(hipStream_t st, hb_pending& pd, int n, int W) {
+    if (pd.p.y) hb_post_norm(st, n, pd.p, pd.x, pd.ldx, W);
+    pd.p.y = nullptr;
 }
 
 // 2..16 rows, bf16: one MFMA row tile; a block owns 16 output columns and its eight waves take the 32-wide k-steps w, w + 8, ...
@@ -2558,10 +2684,12 @@ __global__ __launch_bounds__(1024) __attribute__((amdgpu_waves_per_eu(1, 4))) vo
 }
 
 // few-row steps: the segments' partial results of a (row, head), merged in segment order; output gate (one per head, or gate_cols: one per
-// output column) applied here.  keep: the first tokens of the sequence that stay visible before the window
+// output column) applied here.  VPL: value columns per lane at most.  keep: the first tokens of the sequence that stay visible before the window
+template <int VPL>
 __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nseg_grid, float* out, long ldo, const int* pos, int H, int vdim,
                                                       int window, int P, int seg_chunks, const float* gate, long ldg, float out_scale, int chunk,
-                                                      hb_sink sink, int keep = 0, int gate_cols = 0) {
+                                                      hb_sink sink, int keep, int gate_cols) {
+    constexpr int U = 32 / VPL;
     const int row = blockIdx.x, hq = blockIdx.y, lane = threadIdx.x;
     const int p = pos[row];
     const int first = p - window + 1;
@@ -2576,39 +2704,39 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
     mm = hb_wave_max(mm);
     const float gmul = (gate && !gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
     float lt = 0.f;
-    float acc[HB_MAX_VPL];
+    float acc[VPL];
 #pragma unroll
-    for (int e = 0; e < HB_MAX_VPL; ++e) acc[e] = 0.f;
+    for (int e = 0; e < VPL; ++e) acc[e] = 0.f;
     for (int s0 = 0; s0 < nseg; s0 += 64) {
         const bool mine = s0 + lane < nseg;
         const float wmine = mine ? expf(src[(size_t)(s0 + lane) * (vdim + 2) + vdim] - mm) : 0.f;
         const float lmine = mine ? src[(size_t)(s0 + lane) * (vdim + 2) + vdim + 1] * wmine : 0.f;
         const int ns = nseg - s0 < 64 ? nseg - s0 : 64;
-        for (int s2 = 0; s2 < ns; s2 += 4) {
-            // four segments' values on their way before the first is used
-            float v[4][HB_MAX_VPL];
+        for (int s2 = 0; s2 < ns; s2 += U) {
+            // several segments' values on their way before the first is used
+            float v[U][VPL];
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
+            for (int u = 0; u < U; ++u) {
                 const float* sp = src + (size_t)(s0 + (s2 + u < ns ? s2 + u : ns - 1)) * (vdim + 2);
 #pragma unroll
-                for (int e = 0; e < HB_MAX_VPL; ++e) {
+                for (int e = 0; e < VPL; ++e) {
                     const int j = lane + e * 64;
                     v[u][e] = j < vdim ? sp[j] : 0.f;
                 }
             }
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
+            for (int u = 0; u < U; ++u) {
                 if (s2 + u >= ns) break;
                 const float w = __shfl(wmine, s2 + u, 64);
                 lt += __shfl(lmine, s2 + u, 64);
 #pragma unroll
-                for (int e = 0; e < HB_MAX_VPL; ++e) acc[e] += v[u][e] * w;
+                for (int e = 0; e < VPL; ++e) acc[e] += v[u][e] * w;
             }
         }
     }
     if (sink.on) lt += expf(sk - mm);
 #pragma unroll
-    for (int e = 0; e < HB_MAX_VPL; ++e) {
+    for (int e = 0; e < VPL; ++e) {
         const int j = lane + e * 64;
         if (j < vdim) out[(size_t)row * ldo + hq * vdim + j] = acc[e] / lt * gmul * (gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq * vdim + j]) : 1.0f);
     }
@@ -3411,6 +3539,7 @@ struct hb_win {
 };
 __device__ __forceinline__ int hb_win_start(const hb_win& w, int p) { return w.window > 0 && p >= w.window ? p - w.window + 1 : 0; }
 
+#define HB_WIN_PAIRS 8
 // What a row leaves in the cache, and its query: q and k RMS-normed over their whole projection (all heads at once, weights q_norm
 // [H*dim], k_norm [G*dim]), then the first `rot` dims of every head rotated (interleaved pairs, cos and sin times `mag`).  proj row =
 // [q | k | v | ...]; the query stays in place, k and v go into the cache.  Block (row, part 0 q / 1 k / 2 v); a thread owns whole pairs.
@@ -3432,20 +3561,45 @@ __global__ __launch_bounds__(256) void k_hb_win_prep(float* proj, long ldp, T* c
     const int n = part == 0 ? nq : nk, heads = part == 0 ? H : G;
     const float* nw = part == 0 ? q_norm : k_norm;
     const float pf = (float)pos[row];
+    const int pph = (dim + 1) >> 1, pairs = heads * pph;
+    // (the first HB_WIN_PAIRS * 256 pairs stay in registers)
+    float2 x[HB_WIN_PAIRS], w[HB_WIN_PAIRS];
+    auto at = [&](int i) { const int h = i / pph; return h * dim + 2 * (i - h * pph); };
+    auto load = [&](int i, float2& xv, float2& wv2) {
+        const int j = i % pph, c = at(i);
+        const bool two = 2 * j + 1 < dim;
+        xv = make_float2(src[c], two ? src[c + 1] : 0.f);
+        wv2 = make_float2(nw[c], two ? nw[c + 1] : 0.f);
+    };
+    const bool even = (dim & 1) == 0 && ((((size_t)src) | ((size_t)nw)) & 7) == 0;
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < HB_WIN_PAIRS; ++e) {
+        const int i = tid + e * 256;
+        x[e] = w[e] = make_float2(0.f, 0.f);
+        if (i < pairs) {
+            if (even) { x[e] = *(const float2*)(src + 2 * i); w[e] = *(const float2*)(nw + 2 * i); }
+            else load(i, x[e], w[e]);
+        }
+    }
     for (int i = tid; i < rot / 2; i += 256) {
         float sn, cs;
         sincosf(pf * inv_freq[i], &sn, &cs);
         turn[i] = make_float2(cs * mag, sn * mag);
     }
-    float ss = 0.f;
-    for (int i = tid; i < n; i += 256) ss = fmaf(src[i], src[i], ss);
+#pragma unroll
+    for (int e = 0; e < HB_WIN_PAIRS; ++e) { ss = fmaf(x[e].x, x[e].x, ss); ss = fmaf(x[e].y, x[e].y, ss); }
+    for (int i = tid + HB_WIN_PAIRS * 256; i < pairs; i += 256) {
+        float2 xv, wv2;
+        load(i, xv, wv2);
+        ss = fmaf(xv.x, xv.x, ss); ss = fmaf(xv.y, xv.y, ss);
+    }
     const float inv = 1.0f / sqrtf(hb_block_sum256(ss, red) / (float)n + eps);
     T* kd = part == 1 ? cache + tok * (size_t)nk : nullptr;
-    const int pph = (dim + 1) >> 1;
-    for (int i = tid; i < heads * pph; i += 256) {
+    auto finish = [&](int i, const float2& xv, const float2& wv2) {
         const int h = i / pph, j = i - h * pph, c = h * dim + 2 * j;
         const bool two = 2 * j + 1 < dim;
-        float u = src[c] * inv * nw[c], v = two ? src[c + 1] * inv * nw[c + 1] : 0.f;
+        float u = xv.x * inv * wv2.x, v = xv.y * inv * wv2.y;
         if (2 * j < rot) {
             const float2 t = turn[j];
             const float u2 = fmaf(u, t.x, -(v * t.y));
@@ -3453,12 +3607,21 @@ __global__ __launch_bounds__(256) void k_hb_win_prep(float* proj, long ldp, T* c
             u = u2;
         }
         if (part == 0) {
+            if (even) { *(float2*)(src + c) = make_float2(u, v); return; }
             src[c] = u;
             if (two) src[c + 1] = v;
         } else {
             hb_st(kd + c, u);
             if (two) hb_st(kd + c + 1, v);
         }
+    };
+#pragma unroll
+    for (int e = 0; e < HB_WIN_PAIRS; ++e)
+        if (tid + e * 256 < pairs) finish(tid + e * 256, x[e], w[e]);
+    for (int i = tid + HB_WIN_PAIRS * 256; i < pairs; i += 256) {
+        float2 xv, wv2;
+        load(i, xv, wv2);
+        finish(i, xv, wv2);
     }
 }
 
@@ -3626,22 +3789,22 @@ __global__ __launch_bounds__(256) void k_hb_win_attn_rows(const float* q, long l
         out[(size_t)row * ldo + (size_t)h * vdim + j] = a;
     }
 }
-// Steps of many rows, bf16 cache: block = 64 * RT consecutive rows of one request (RT groups of 16 per wave) and one head; tiles of 64 keys
+// Steps of many rows, bf16 cache: block = 64 consecutive rows of one request (16 per wave) and one head; tiles of 64 keys
 // in LDS, keys as cached (Kt[key][dim]), values transposed two keys at a time (Vt[column][key]); the next tile's requests are on their way
-// while a tile is multiplied.  Tiles: the kept tokens before the first row's window, then the windows of all rows.  Per tile, wave and group,
+// while a tile is multiplied.  Tiles: the kept tokens before the first row's window, then the windows of all rows.  Per tile and wave,
 // rows being the 16 columns of both products:
 //   S^T[key][row] = sum_dim Kt[key][dim] Q[row][dim]     v_mfma_f32_16x16x32_bf16, the query in registers as two bf16 parts (hi + lo)
 //   weights 2^(score - running maximum) of the lane's 16 (key, row) pairs, fp32, scores carrying scale * log2(e); masked pairs 0
 //   O^T[col][row] += sum_key Vt[col][key] P[row][key]    the weights as they sit in the lanes (k index laid out to match), hi + lo
 // Row tiles of the launch are found by walking the requests' row counts; blocks beyond the last tile leave.  KS 32-dim steps of the key
 // and CT 16-column tiles of the value at most.
-template <int KS, int CT, int RT>
+template <int KS, int CT>
 __global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long ldq, const bf16_t* cache, float* out, long ldo, const int* pos,
                                                           const int* req_rows, int n_req, const int* ptab, int pts, int H, int G, int dim, int vdim,
                                                           int ps, long v_base, hb_win w, float scale, hb_sink sink, const float* gate, long ldg,
                                                           float out_scale, int ks_n, int ct_n, int fold) {
     extern __shared__ float sm[];
-    constexpr int BR = 64 * RT, WR = 16 * RT;
+    constexpr int BR = 64, WR = 16;
     constexpr float LOG2E = 1.44269504088896340736f, LOWEST = -1e30f;
     const int DPK = ks_n * 32 + 8;
     bf16_t* Kt = (bf16_t*)sm;                            // [64][DPK]
@@ -3669,38 +3832,27 @@ __global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long l
     const int wlo_first = hb_win_start(w, wp_first), wlo_hi = active ? hb_win_start(w, wp_hi) : 0;
     const int* pt = ptab + (size_t)rq * pts;
     const float zmul = scale * LOG2E;
-    int p[RT], lo_r[RT];
-    bool rowok[RT];
-    uint4 qh[RT][KS], ql[RT][KS];
+    const bool rowok = col < wn;
+    const int row = rs + (active ? w0 + (rowok ? col : wn - 1) : 0);      // (a lane without a row follows the wave's last one)
+    const int p = pos[row], lo_r = hb_win_start(w, p);
+    uint4 qh[KS], ql[KS];
 #pragma unroll
-    for (int rt = 0; rt < RT; ++rt) {
-        rowok[rt] = rt * 16 + col < wn;
-        const int row = rs + (active ? w0 + (rowok[rt] ? rt * 16 + col : wn - 1) : 0);      // (a lane without a row follows the wave's last one)
-        p[rt] = pos[row];
-        lo_r[rt] = hb_win_start(w, p[rt]);
+    for (int ks = 0; ks < KS; ++ks) {
+        float v[8];
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks) {
-            float v[8];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) v[i] = 0.f;
-            const int d0 = ks * 32 + g4 * 8;
-            if (ks < ks_n && rowok[rt] && d0 < dim) {
-                const float* src = q + (size_t)row * ldq + (size_t)h * dim + d0;
-                const float4 a = *(const float4*)src, b = *(const float4*)(src + 4);
-                v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
-            }
-            hb_split_bf16x8(v, qh[rt][ks], ql[rt][ks]);
+        for (int i = 0; i < 8; ++i) v[i] = 0.f;
+        const int d0 = ks * 32 + g4 * 8;
+        if (ks < ks_n && rowok && d0 < dim) {
+            const float* src = q + (size_t)row * ldq + (size_t)h * dim + d0;
+            const float4 a = *(const float4*)src, b = *(const float4*)(src + 4);
+            v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
         }
+        hb_split_bf16x8(v, qh[ks], ql[ks]);
     }
-    hb_f32x4 oacc[RT][CT];
-    float m[RT], l[RT];         // running maximum of the row (log2 units), the lane's share of its sum
+    hb_f32x4 oacc[CT];
+    float m = LOWEST, l = 0.f;         // running maximum of the row (log2 units), the lane's share of its sum
 #pragma unroll
-    for (int rt = 0; rt < RT; ++rt) {
-        m[rt] = LOWEST;
-        l[rt] = 0.f;
-#pragma unroll
-        for (int ct = 0; ct < CT; ++ct) oacc[rt][ct] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
-    }
+    for (int ct = 0; ct < CT; ++ct) oacc[ct] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
     // staging: keys -- four threads per key, pieces of 8 dims (tid & 3) + 4k; values -- eight threads per pair of keys, pieces of 8
     // columns (tid & 7) + 8k of both keys
     constexpr int NV = (CT * 2 + 7) / 8;
@@ -3755,71 +3907,63 @@ __global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long l
         if (c + 1 < ntiles) fetch(c + 1);
         // (a wave whose rows see no key of the tile)
         if (!active || (!early && (base > wp_hi || (base + 63 < wlo_first && base >= w.keep)))) continue;
-        hb_f32x4 st[RT][4];
+        hb_f32x4 st[4];
 #pragma unroll
-        for (int rt = 0; rt < RT; ++rt)
-#pragma unroll
-            for (int kt = 0; kt < 4; ++kt) st[rt][kt] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int kt = 0; kt < 4; ++kt) st[kt] = hb_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
             if (ks < ks_n) {
 #pragma unroll
                 for (int kt = 0; kt < 4; ++kt) {
                     const uint4 a = *(const uint4*)(Kt + (size_t)(kt * 16 + col) * DPK + ks * 32 + g4 * 8);
-#pragma unroll
-                    for (int rt = 0; rt < RT; ++rt) {
-                        st[rt][kt] = hb_mfma_bf16(a, qh[rt][ks], st[rt][kt]);
-                        st[rt][kt] = hb_mfma_bf16(a, ql[rt][ks], st[rt][kt]);
-                    }
+                    st[kt] = hb_mfma_bf16(a, qh[ks], st[kt]);
+                    st[kt] = hb_mfma_bf16(a, ql[ks], st[kt]);
                 }
             }
         }
-        // lane (col, g4) holds the scores of row `col` of each group against keys base + kt*16 + g4*4 + i
+        // lane (col, g4) holds the scores of row `col` against keys base + kt*16 + g4*4 + i
         const bool full = early ? base + 63 < kept : (base + 63 <= wp_first && base >= wlo_hi);     // every row of the wave sees the whole tile
-        uint4 ph[RT][2], plo[RT][2];
+        float z[4][4], top = LOWEST;
 #pragma unroll
-        for (int rt = 0; rt < RT; ++rt) {
-            float z[4][4], top = LOWEST;
+        for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
-            for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    float s = st[rt][kt][i] * zmul;
-                    if (!full) {
-                        const int key = base + kt * 16 + g4 * 4 + i;
-                        const bool see = early ? key < kept : key <= p[rt] && (key >= lo_r[rt] || key < w.keep);
-                        s = see ? s : -INFINITY;
-                    }
-                    z[kt][i] = s;
-                    top = fmaxf(top, s);
+            for (int i = 0; i < 4; ++i) {
+                float s = st[kt][i] * zmul;
+                if (!full) {
+                    const int key = base + kt * 16 + g4 * 4 + i;
+                    const bool see = early ? key < kept : key <= p && (key >= lo_r || key < w.keep);
+                    s = see ? s : -INFINITY;
                 }
-            top = fmaxf(top, __shfl_xor(top, 16, 64));
-            top = fmaxf(top, __shfl_xor(top, 32, 64));
-            if (__ballot(top > m[rt])) {
-                const float mn = fmaxf(m[rt], top), alpha = __builtin_amdgcn_exp2f(m[rt] - mn);
-                m[rt] = mn;
-                l[rt] *= alpha;
-#pragma unroll
-                for (int ct = 0; ct < CT; ++ct)
-                    if (ct < ct_n)
-#pragma unroll
-                        for (int i = 0; i < 4; ++i) oacc[rt][ct][i] *= alpha;
+                z[kt][i] = s;
+                top = fmaxf(top, s);
             }
-            float sum = 0.f;
+        top = fmaxf(top, __shfl_xor(top, 16, 64));
+        top = fmaxf(top, __shfl_xor(top, 32, 64));
+        if (__ballot(top > m)) {
+            const float mn = fmaxf(m, top), alpha = __builtin_amdgcn_exp2f(m - mn);
+            m = mn;
+            l *= alpha;
 #pragma unroll
-            for (int kt = 0; kt < 4; ++kt)
+            for (int ct = 0; ct < CT; ++ct)
+                if (ct < ct_n)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    z[kt][i] = __builtin_amdgcn_exp2f(z[kt][i] - m[rt]);
-                    sum += z[kt][i];
-                }
-            l[rt] += sum;
+                    for (int i = 0; i < 4; ++i) oacc[ct][i] *= alpha;
+        }
+        float sum = 0.f;
 #pragma unroll
-            for (int kk = 0; kk < 2; ++kk) {
-                const float v[8] = {z[2 * kk][0], z[2 * kk][1], z[2 * kk][2], z[2 * kk][3], z[2 * kk + 1][0], z[2 * kk + 1][1], z[2 * kk + 1][2],
-                                    z[2 * kk + 1][3]};
-                hb_split_bf16x8(v, ph[rt][kk], plo[rt][kk]);
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                z[kt][i] = __builtin_amdgcn_exp2f(z[kt][i] - m);
+                sum += z[kt][i];
             }
+        l += sum;
+        uint4 ph[2], plo[2];
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            const float v[8] = {z[2 * kk][0], z[2 * kk][1], z[2 * kk][2], z[2 * kk][3], z[2 * kk + 1][0], z[2 * kk + 1][1], z[2 * kk + 1][2],
+                                z[2 * kk + 1][3]};
+            hb_split_bf16x8(v, ph[kk], plo[kk]);
         }
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) {
@@ -3829,41 +3973,32 @@ __global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long l
                     const bf16_t* vr = Vt + (size_t)(ct * 16 + col) * HB_SIG_VLD + kk * 32 + g4 * 4;
                     const uint2 a0 = *(const uint2*)vr, a1 = *(const uint2*)(vr + 16);
                     const uint4 a = make_uint4(a0.x, a0.y, a1.x, a1.y);
-#pragma unroll
-                    for (int rt = 0; rt < RT; ++rt) {
-                        oacc[rt][ct] = hb_mfma_bf16(a, ph[rt][kk], oacc[rt][ct]);
-                        oacc[rt][ct] = hb_mfma_bf16(a, plo[rt][kk], oacc[rt][ct]);
-                    }
+                    oacc[ct] = hb_mfma_bf16(a, ph[kk], oacc[ct]);
+                    oacc[ct] = hb_mfma_bf16(a, plo[kk], oacc[ct]);
                 }
             }
         }
     }
-    const float sk = sink.on ? hb_sink_of(sink, h) * LOG2E : 0.f;
-#pragma unroll
-    for (int rt = 0; rt < RT; ++rt) {
-        float den = l[rt];
-        den += __shfl_xor(den, 16, 64);
-        den += __shfl_xor(den, 32, 64);
-        float f = out_scale;
-        if (sink.on) {
-            const float mm = fmaxf(m[rt], sk), a = __builtin_amdgcn_exp2f(m[rt] - mm);
-            den = fmaf(den, a, __builtin_amdgcn_exp2f(sk - mm));
-            f *= a;
-        }
-        if (!rowok[rt]) continue;
-        const int row = rs + w0 + rt * 16 + col;
-        f /= den;
-        float* dst = out + (size_t)row * ldo + (size_t)h * vdim;
-        const float* gr = gate ? gate + (size_t)row * ldg + (size_t)h * vdim : nullptr;
-#pragma unroll
-        for (int ct = 0; ct < CT; ++ct)
-            if (ct < ct_n)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const int cc = ct * 16 + g4 * 4 + i;
-                    if (cc < vdim) dst[cc] = oacc[rt][ct][i] * f * (gr ? hb_sigmoid(gr[cc]) : 1.0f);
-                }
+    float den = l, f = out_scale;
+    den += __shfl_xor(den, 16, 64);
+    den += __shfl_xor(den, 32, 64);
+    if (sink.on) {
+        const float sk = hb_sink_of(sink, h) * LOG2E, mm = fmaxf(m, sk), a = __builtin_amdgcn_exp2f(m - mm);
+        den = fmaf(den, a, __builtin_amdgcn_exp2f(sk - mm));
+        f *= a;
     }
+    if (!rowok) return;
+    f /= den;
+    float* dst = out + (size_t)row * ldo + (size_t)h * vdim;
+    const float* gr = gate ? gate + (size_t)row * ldg + (size_t)h * vdim : nullptr;
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct)
+        if (ct < ct_n)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int cc = ct * 16 + g4 * 4 + i;
+                if (cc < vdim) dst[cc] = oacc[ct][i] * f * (gr ? hb_sigmoid(gr[cc]) : 1.0f);
+            }
 }
 
 // ---- routed feed-forward --------------------------------------------------------------------------------------------------
@@ -3873,7 +4008,9 @@ __global__ __launch_bounds__(256) void k_hb_win_attn_mfma(const float* q, long l
 // sigmoid != 0: s_j = sigmoid(z_j) instead of the softmax; renorm == 0: the weights are the chosen s as they are.
 // bias != NULL: added to the logits before the scores are formed.  groups > 1: only experts of the `keep` best groups can be chosen.
 // wscale multiplies the weights.  A group's score is its largest choice value, or (best_two) the sum of its two largest.
-// post.y != NULL: the row is first completed with a normed sublayer output, x_out (= h) += norm(y).
+// post.y != NULL: the row is first completed with a normed sublayer output, x_out (= h) += norm(y); NC > 0: in the register form of
+// hb_post_row, whose columns are those a thread multiplies, with the first eight router rows requested before the norm.
+template <int NC>
 __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh, const float* router, const float* corr, int W, int nE, int top,
                                                        int* sel, float* wgt, int sigmoid, int renorm, const float* bias, int groups, int keep,
                                                        float wscale, int best_two, hb_post post, float* x_out) {
@@ -3885,21 +4022,48 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
     float* gs = part + 4 * nE;         // [groups] group scores (groups > 1)
     const int row = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const float* x = h + (size_t)row * ldh;
-    if (post.y) {
-        __shared__ float red[2][4];
+    __shared__ float red[2][4];
+    constexpr int NX = NC > 0 ? NC : 1;
+    float4 mine4[NX], r4[8][NX];
+    auto router_rows = [&](int j0) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+#pragma unroll
+            for (int i = 0; i < NX; ++i) {
+                const int k = threadIdx.x * 4 + 1024 * i;
+                r4[j][i] = *(const float4*)(router + (size_t)(j0 + j < nE ? j0 + j : nE - 1) * W + (k < W ? k : 0));
+            }
+    };
+    if constexpr (NC > 0) {
+        router_rows(0);
         float* xr = x_out + (size_t)row * ldh;
-        if (W <= 1024) hb_post_norm_row<4>(post, row, xr, W, red);
-        else if (W <= 4096) hb_post_norm_row<16>(post, row, xr, W, red);
-        else hb_post_norm_row<0>(post, row, xr, W, red);
+        hb_post_row<NC>(post, row, xr, xr, W, red, mine4);
+    } else if (post.y) {
+        hb_post_row_any(post, row, x_out + (size_t)row * ldh, W, red);
         __syncthreads();
     }
     const bool vec = (W % 4 == 0) && (ldh % 4 == 0) && ((((size_t)h) & 15) == 0) && ((((size_t)router) & 15) == 0);
     // wave w sums the k-chunks w, w + 4, ... (64 lanes x 4 values, or 64 values); a logit = the four waves' sums added in wave order
     for (int j0 = 0; j0 < nE; j0 += 8) {
         float acc[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[j] = 0.f;
+        if constexpr (NC > 0) {
+            if (j0 > 0) router_rows(j0);
+#pragma unroll
+            for (int i = 0; i < NC; ++i)
+                if ((int)threadIdx.x * 4 + 1024 * i < W) {
+                    const float4 xv = mine4[i];
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        acc[j] = fmaf(r4[j][i].x, xv.x, acc[j]); acc[j] = fmaf(r4[j][i].y, xv.y, acc[j]);
+                        acc[j] = fmaf(r4[j][i].z, xv.z, acc[j]); acc[j] = fmaf(r4[j][i].w, xv.w, acc[j]);
+                    }
+                }
+        } else {
         const float* r[8];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) { acc[j] = 0.f; r[j] = router + (size_t)(j0 + j < nE ? j0 + j : nE - 1) * W; }
+        for (int j = 0; j < 8; ++j) r[j] = router + (size_t)(j0 + j < nE ? j0 + j : nE - 1) * W;
         if (vec) {
             for (int k = (wv * 64 + lane) * 4; k < W; k += 1024) {
                 const float4 xv = *(const float4*)(x + k);
@@ -3916,6 +4080,7 @@ __global__ __launch_bounds__(256) void k_hb_moe_router(const float* h, long ldh,
 #pragma unroll
                 for (int j = 0; j < 8; ++j) acc[j] = fmaf(r[j][k], xv, acc[j]);
             }
+        }
         }
         // eight sums over the wave with 10 exchanges instead of 48: each of the first three exchanges halves the values a lane
         // carries (lanes with the partner bit clear keep the lower half and receive the partner's), three more finish the one left;
@@ -4050,13 +4215,8 @@ __global__ __launch_bounds__(256) void k_hb_moe_group(const int* sel, int n_entr
     }
     if (threadIdx.x == 0) count[e] = base;
 }
-// y = act(g) * (u + up_offset), g = min(gate, limit), u = clamp(up, -limit, limit); act(g) = g * sigmoid(alpha g), or the tanh form
-// of gelu (gelu != 0); gu row = [gate (ff) | up (ff)].
-// sel != NULL: rows are routed entries, those of identity outputs (sel >= experts) are skipped.
-__device__ __forceinline__ float hb_glu(float g0, float u0, float limit, float alpha, float up_offset, int gelu) {
-    const float g = fminf(g0, limit), u = fminf(fmaxf(u0, -limit), limit);
-    return (gelu ? hb_gelu_tanh(g) : g * hb_sigmoid(alpha * g)) * (u + up_offset);
-}
+// y = hb_glu of gu row = [gate (ff) | up (ff)] (k_hb_glu_clamp below).  sel != NULL: rows are routed entries, those of identity outputs
+// (sel >= experts) are skipped.
 // the activation of an up / down unit: the square of relu, or g * sigmoid(alpha g)
 __device__ __forceinline__ float hb_unit_act(float g, int relu2, float alpha) {
     if (relu2) { const float r = fmaxf(g, 0.f); return r * r; }
@@ -4381,6 +4541,8 @@ static bool hb_try_norm_gemv(const vox_hybrid* m, hipStream_t st, int epi, const
     return (m->cfg.norm_kind == VOX_NORM_LAYER || rms) && hb_try_ln_gemv<T>(st, epi, X, ldx, rows, nw, m->cfg.eps, W, bias, C, N, K, rms ? 1 : 0, epi_arg, nb);
 }
 
+static auto hb_merge_kernel(int columns) -> decltype(&k_hb_attn_merge<2>) { return columns <= 128 ? k_hb_attn_merge<2> : k_hb_attn_merge<HB_MAX_VPL>; }
+
 // The matrix-core latent attention for steps of many rows over a bf16 cache.  false: the shapes do not fit it (rows of the cache that are
 // no multiple of 16 bytes, a latent beyond 512 values or keys beyond 576) and the caller takes the general kernel.
 static bool hb_try_latent_mfma(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, const bf16_t* cache, const float* qa,
@@ -4478,16 +4640,17 @@ static bool hb_try_win_mfma(hipStream_t st, const vox_hybrid_io* io, const vox_h
     if ((L.dim & 7) || (L.vdim & 7) || L.dim > 256 || L.vdim > 256 || (ldp & 3) || ((size_t)q & 15) || ((size_t)cache & 15)) return false;
     const int ks_n = (L.dim + 31) / 32, ct_n = (L.vdim + 15) / 16;
     const size_t lds = (size_t)64 * (ks_n * 32 + 8) * 2 + (size_t)ct_n * 16 * HB_SIG_VLD * 2;
-#define HB_WM(KS_, CT_, RT_) \
+    const dim3 grid(L.heads, (n + 63 * n_req) / 64), block(256);      // (at least the sum of the requests' tiles)
+    const int fold = grid.x * grid.y <= 2 * 256 ? 1 : 0;
+#define HB_WM(KS_, CT_) \
     do { \
-        const dim3 grid(L.heads, (n + (64 * RT_ - 1) * n_req) / (64 * RT_)), block(256);      /* (at least the sum of the requests' tiles) */ \
-        if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_win_attn_mfma<KS_, CT_, RT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
-        hipLaunchKernelGGL((k_hb_win_attn_mfma<KS_, CT_, RT_>), grid, block, lds, st, q, ldp, cache, out, ldo, io->pos, io->req_rows, n_req, io->page_table, \
+        if (lds > 64 * 1024) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k_hb_win_attn_mfma<KS_, CT_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        hipLaunchKernelGGL((k_hb_win_attn_mfma<KS_, CT_>), grid, block, lds, st, q, ldp, cache, out, ldo, io->pos, io->req_rows, n_req, io->page_table, \
                            io->pt_stride, L.heads, L.kv_heads, L.dim, L.vdim, ps, v_base, hb_win{L.window, L.keep_first}, L.scale, sink, gate, ldp, \
-                           L.out_scale, ks_n, ct_n, grid.x * grid.y <= 2 * 256 ? 1 : 0); \
+                           L.out_scale, ks_n, ct_n, fold); \
     } while (0)
-    if (ks_n <= 4 && ct_n <= 8) HB_WM(4, 8, 1);
-    else HB_WM(8, 16, 1);
+    if (ks_n <= 4 && ct_n <= 8) HB_WM(4, 8);
+    else HB_WM(8, 16);
 #undef HB_WM
     return true;
 }
@@ -4521,7 +4684,7 @@ static int hb_win_attention(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* 
     else HB_WR(1);
 #undef HB_WR
     if (nseg > 1)
-        hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim,
+        hipLaunchKernelGGL(hb_merge_kernel(L.vdim), dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim,
                            L.window > 0 ? L.window : 0x7fffffff, 0x7fffffff, cpb, gate, ldp, L.out_scale, 64, sink, L.keep_first, gate ? 1 : 0);
     return VOX_OK;
 }
@@ -4537,10 +4700,11 @@ static int hb_gemm_resid(hipStream_t st, const float* A, long lda, const T* W, c
     return hb_gemm<T>(st, epi, A, lda, W, bias, cur, ldx, n, N, K, rm);
 }
 // One mixer: reads the rows hn (!= NULL, ldh apart: normed already, or read as they are) or norms src (rows lds apart) itself with L.norm1; out_scale * mixer(.) joins cur as `jn`
-// says (the layer's residual gate, when it has one, is added to it here: its logits are the last columns of the input projection).
+// says; pd != NULL: the rows are pd->x, with whatever is pending on it (the layer's residual gate, when it has one, is added to it here: its logits are the last columns of the input projection).
 template <typename T>
 static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const vox_hybrid_layer& L, void* cache, float* pool, float* state,
-                    const float* hn, long ldh, const float* src, long lds_x, float* cur, long ldx, int n, int n_req, int max_kvlen, hb_join jn) {
+                    const float* hn, long ldh, const float* src, long lds_x, float* cur, long ldx, int n, int n_req, int max_kvlen, hb_join jn,
+                    hb_pending* pd = nullptr) {
     const vox_hybrid_config& c = m->cfg;
     const int W = c.width, ps = c.page_size;
     const int n_in = hb_layer_in(L), n_proj = hb_layer_proj(L), n_mix = L.heads * L.vdim;
@@ -4603,7 +4767,12 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
                                (int)HB_GATE_SILU, L.vdim, c.eps, L.out_scale);
         return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
     }
-    if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, src, lds_x, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W, 0.f, L.norm1_b))) {
+    if (pd) {
+        // (post-normed layer: the rows are the stream itself, a norm may still be pending on it)
+        const bool done = n == 1 && pd->p.y && hb_try_post_gemv<T>(st, *pd, false, (const T*)L.w_in, L.b_in, m->proj, n_in, W);
+        if (!done) hb_settle(st, *pd, n, W);
+        hn = done ? nullptr : pd->x;
+    } else if (!hn && !(n == 1 && hb_try_norm_gemv<T>(m, st, HB_EPI_STORE, src, lds_x, nullptr, L.norm1, (const T*)L.w_in, L.b_in, m->proj, n_in, W, 0.f, L.norm1_b))) {
         hb_norm(m, st, n, src, lds_x, nullptr, L.norm1, m->h, nullptr, nullptr, (long)W, L.norm1_b);
         hn = m->h;
         ldh = W;
@@ -4742,8 +4911,8 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
                                io->pos, io->row_req, io->page_table, io->pt_stride, H, R, r, window, ps, L.scale, cpb,
                                seg2 ? m->attn_ws : (float*)nullptr, gate, (long)n_proj, L.out_scale, DP, sink);
             if (seg2)
-                hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg2, o, (long)n_proj, io->pos, H, R, window, P, cpb,
-                                   gate, (long)n_proj, L.out_scale, KT, sink);
+                hipLaunchKernelGGL(hb_merge_kernel(R), dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg2, o, (long)n_proj, io->pos, H, R, window, P, cpb,
+                                   gate, (long)n_proj, L.out_scale, KT, sink, 0, 0);
         } else if (hb_try_latent_mfma(m, st, io, L, (const T*)cache, qa, o, (long)n_proj, gate, n, n_req, window, ps)) {
         } else {
         const int nseg = 1;
@@ -4757,8 +4926,8 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
                            0L, L.scale, split, segmented ? HB_ATTN_SEG : 0, segmented ? m->attn_ws : (float*)nullptr, gate, (long)n_proj,
                            L.out_scale, 1, (long)D, sink);
         if (segmented)
-            hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, o, (long)n_proj, io->pos, H, R, window, P,
-                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink);
+            hipLaunchKernelGGL(hb_merge_kernel(R), dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, o, (long)n_proj, io->pos, H, R, window, P,
+                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink, 0, 0);
         }
         // every head's weighted latent times its value expansion
         VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, o, n_proj, (const T*)L.w_uv, nullptr, m->mix, n_mix, n, L.vdim, R,
@@ -4841,8 +5010,8 @@ static int hb_mixer(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, cons
                            P, ps, ppp, v_base, L.scale, split, segmented ? HB_ATTN_SEG : 0, segmented ? m->attn_ws : (float*)nullptr,
                            gate, (long)n_proj, L.out_scale, G, (long)G * L.vdim, sink);
         if (segmented)
-            hipLaunchKernelGGL(k_hb_attn_merge, dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim, window, P,
-                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink);
+            hipLaunchKernelGGL(hb_merge_kernel(L.vdim), dim3(n, H), dim3(64), 0, st, m->attn_ws, nseg, m->mix, (long)n_mix, io->pos, H, L.vdim, window, P,
+                               HB_ATTN_SEG, gate, (long)n_proj, L.out_scale, 64, sink, 0, 0);
     }
     return hb_gemm_resid<T>(st, m->mix, n_mix, (const T*)L.w_out, nullptr, cur, ldx, n, W, n_mix, jn);
 }
@@ -4856,8 +5025,10 @@ static int hb_moe(vox_hybrid* m, hipStream_t st, const vox_hybrid_layer& L, cons
     if (L.res_gate) { jn.gate = m->rgate; jn.ldg = m->cfg.width; }
     const int W = m->cfg.width, nE = E.experts + E.identity, top = E.top, ne = n * top, ff = E.ff;
     const int up_down = E.expert_form == VOX_EXPERT_UP_DOWN ? 1 : 0, relu2 = E.expert_act == VOX_ACT_RELU2 ? 1 : 0, nf = up_down ? 1 : 2;
-    hipLaunchKernelGGL(k_hb_moe_router, dim3(n), dim3(256), (size_t)(6 * nE + top + (E.groups > 1 ? E.groups : 0)) * 4, st, h2, ldh, E.router, E.correction,
-                       W, nE, top, m->moe_sel, m->moe_wgt, E.score_kind == VOX_ROUTER_SIGMOID ? 1 : 0, E.renorm, E.router_bias, E.groups, E.keep,
+    const int nc = post.y && ((size_t)E.router & 15) == 0 ? hb_post_pieces(post, h2, ldh, W) : 0;
+    auto router = nc == 1 ? k_hb_moe_router<1> : nc == 2 ? k_hb_moe_router<2> : nc == 4 ? k_hb_moe_router<4> : k_hb_moe_router<0>;
+    hipLaunchKernelGGL(router, dim3(n), dim3(256), (size_t)(6 * nE + top + (E.groups > 1 ? E.groups : 0)) * 4, st, h2, ldh, E.router, E.correction, W, nE, top,
+                       m->moe_sel, m->moe_wgt, E.score_kind == VOX_ROUTER_SIGMOID ? 1 : 0, E.renorm, E.router_bias, E.groups, E.keep,
                        E.weight_scale != 0.f ? E.weight_scale : 1.0f, E.group_best_two, post, post.y ? const_cast<float*>(h2) : (float*)nullptr);
     if (n <= HB_MOE_GEMV_ROWS) {
         const int per = top + (E.shared_ff > 0 ? 1 : 0), maxf = ff > E.shared_ff ? ff : E.shared_ff;
@@ -4909,10 +5080,13 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
     if (bigram && n != n_req)
         hipLaunchKernelGGL(k_hb_store_prev, dim3((n_req + 63) / 64), dim3(64), 0, st, ids, 1, c.vocab, io->req_rows, io->req_state, m->w.prev_token, n_req);
     float *cur = m->xa, *other = m->xb;
+    hb_pending pd{};
+    pd.ldx = ldx;
     for (int ri = 0; ri < c.n_runs; ++ri) {
         const vox_hybrid_run& run = m->runs[ri];
         const vox_hybrid_layer& L = m->layers[run.layer];
         if (run.loop_in) {
+            hb_settle(st, pd, n, W);
             VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, cur, ldx, (const T*)m->w.loop_in, nullptr, other, ldx, n, W, 2 * W));
             float* t = cur; cur = other; other = t;
         }
@@ -4936,29 +5110,42 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
         const hb_post none{}, post1{m->y, W, L.norm1, L.norm1_b, c.eps, rms}, post2{m->y, W, L.norm2, L.norm2_b, c.eps, rms};
         float* dst = post ? m->y : cur;
         const long ldd = post ? W : ldx;
-        if (post) j1.store = j2.store = 1;
+        if (post) {
+            j1.store = j2.store = 1;
+            pd.x = cur;
+            pd.x_next = other;
+        } else hb_settle(st, pd, n, W);
         // a parallel layer norms x once for both branches before anything is added; a mixer with a sibling needs the normed rows twice
         const float* hn = nullptr;
         if (parallel || L.sibling >= 0) {
             hb_norm(m, st, n, cur, ldx, nullptr, L.norm1, m->h, parallel && has_ff && !one_norm ? L.norm2 : nullptr, m->h2, (long)W, L.norm1_b, L.norm2_b);
             hn = m->h;
         }
-        const float* hf = post ? cur : one_norm ? m->h : m->h2;      // what the feed-forward of a parallel or post-normed layer reads
+        const float* hf = one_norm ? m->h : m->h2;      // what the feed-forward of a parallel layer reads
         const long ldf = post ? ldx : W;
-        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, post ? cur : hn, post ? ldx : W, src, lds_x, dst, ldd, n, n_req, max_kvlen, j1));
-        if (post && !L.moe) hb_post_norm(st, n, post1, cur, ldx, W);
+        VOX_TRY(hb_mixer<T>(m, st, io, L, run.cache, run.pool, run.state, hn, post ? ldx : W, src, lds_x, dst, ldd, n, n_req, max_kvlen, j1, post ? &pd : nullptr));
+        if (post) {
+            pd.p = post1;
+            if (L.ff > 0 && !L.moe && !(n == 1 && L.ff_kind == VOX_FF_GATED)) hb_settle(st, pd, n, W);
+        }
         if (L.sibling >= 0)
             VOX_TRY(hb_mixer<T>(m, st, io, m->layers[L.sibling], run.side_cache, run.side_pool, run.side_state, hn, W, src, lds_x, cur, ldx, n, n_req,
                                 max_kvlen, j1));
         if (L.moe) {
             if (!parallel && !post) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W, L.norm2_b);
-            VOX_TRY(hb_moe<T>(m, st, L, hf, ldf, post ? post1 : none, dst, ldd, n, j2));
+            const hb_post p1 = pd.p;
+            pd.p.y = nullptr;
+            VOX_TRY(hb_moe<T>(m, st, L, post ? pd.x : hf, ldf, post ? p1 : none, dst, ldd, n, j2));
         } else if (L.ff > 0 && L.ff_kind == VOX_FF_GATED) {
             // down(act(gate h + b) * (up h + b)) + b: gate and up rows in one product, the activation in place behind it
             if (!parallel && !post) hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h2, nullptr, nullptr, (long)W, L.norm2_b);
-            const float* hd = parallel || post ? hf : m->h2;
+            const float* hd = parallel ? hf : m->h2;
             const float limit = L.ff_limit > 0.f ? L.ff_limit : INFINITY, alpha = L.ff_alpha != 0.f ? L.ff_alpha : 1.0f;
-            if (n == 1) {
+            if (post && n == 1 && hb_try_post_gemv<T>(st, pd, true, (const T*)L.w_up, L.b_up, m->ff_act, L.ff, W, limit, alpha, L.ff_up_offset,
+                                                      L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0)) {
+                // (one row of a post-normed layer: norm, both products and the activation in one launch)
+            } else if (n == 1) {
+                if (post) { hb_settle(st, pd, n, W); hd = pd.x; }
                 // one row: gate and up rows of a column by one wave, biases and activation in its epilogue (the routed feed-forward's
                 // kernel with the dense unit in the place of the shared expert and nothing routed); more rows would stream the matrix
                 // once per row
@@ -4967,6 +5154,7 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
                 hipLaunchKernelGGL((k_hb_moe_gate_up<T>), dim3((L.ff + 3) / 4, n), dim3(256), 0, st, hd, ldf, (const T*)nullptr, (const T*)L.w_up,
                                    m->ff_act, W, q);
             } else {
+                if (post) hd = pd.x;
                 VOX_TRY(hb_gemm<T>(st, HB_EPI_STORE, hd, ldf, (const T*)L.w_up, L.b_up, m->ff, 2 * L.ff, n, 2 * L.ff, W));
                 hipLaunchKernelGGL(k_hb_glu_clamp, dim3(n, (L.ff + 1023) / 1024), dim3(256), 0, st, m->ff, m->ff_act, L.ff, limit, alpha,
                                    (const int*)nullptr, 0, L.ff_up_offset, L.ff_act == VOX_ACT_GELU_TANH ? 1 : 0, 0, 0);
@@ -4978,7 +5166,7 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
             hb_rowmap rm = hb_plain();
             rm.epi_arg = (float)L.ff;
             if (parallel || post) {
-                VOX_TRY(hb_gemm<T>(st, epi, hf, ldf, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
+                VOX_TRY(hb_gemm<T>(st, epi, post ? pd.x : hf, ldf, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
             } else if (!(n == 1 && hb_try_norm_gemv<T>(m, st, epi, src, lds_x, nullptr, L.norm2, (const T*)L.w_up, L.b_up, m->ff, nf, W, rm.epi_arg, L.norm2_b))) {
                 hb_norm(m, st, n, src, lds_x, nullptr, L.norm2, m->h, nullptr, nullptr, (long)W, L.norm2_b);
                 VOX_TRY(hb_gemm<T>(st, epi, m->h, W, (const T*)L.w_up, L.b_up, m->ff, nf, n, nf, W, rm));
@@ -4986,12 +5174,18 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
             if (L.res_gate) { j2.gate = m->ff + L.ff; j2.ldg = nf; }
             VOX_TRY(hb_gemm_resid<T>(st, m->ff, nf, (const T*)L.w_down, nullptr, dst, ldd, n, W, L.ff, j2));
         }
-        if (post && has_ff) hb_post_norm(st, n, post2, cur, ldx, W);
+        if (post) {
+            if (has_ff) pd.p = post2;
+            if (io->trace) hb_settle(st, pd, n, W);
+            cur = pd.x;
+            other = pd.x_next;
+        }
         if (io->trace && S > 0)
             hipLaunchKernelGGL(k_hb_sum_streams, dim3(n), dim3(256), 0, st, cur, S, io->trace + (size_t)ri * c.max_rows * W, (long)W, W);
         else if (io->trace)
             hipLaunchKernelGGL(k_hb_copy_rows, dim3(n), dim3(256), 0, st, cur, ldx, io->trace + (size_t)ri * c.max_rows * W, (long)W, W);
     }
+    hb_settle(st, pd, n, W);
     if (n_out > 0) {
         // (several streams: the last sublayer left their sum in m->u)
         const float* last = S > 0 ? m->u : cur;
@@ -5003,8 +5197,7 @@ static int hb_step(vox_hybrid* m, hipStream_t st, const vox_hybrid_io* io, const
         if (!(n_out == 1 && hb_try_norm_gemv<T>(m, st, epi, last, ld_last, io->out_rows, m->w.final_norm, (const T*)m->w.head, nullptr, io->logits, c.vocab,
                                                 W, rm.epi_arg, m->w.final_norm_b))) {
             hb_norm(m, st, n_out, last, ld_last, io->out_rows, m->w.final_norm, m->hout, nullptr, nullptr, (long)W, m->w.final_norm_b);
-            VOX_TRY(hb_gemm<T>(st, epi, m->hout, W, (const T*)m->w.head,
-                               nullptr, io->logits, c.vocab, n_out, c.vocab, W, rm));
+            VOX_TRY(hb_gemm<T>(st, epi, m->hout, W, (const T*)m->w.head, nullptr, io->logits, c.vocab, n_out, c.vocab, W, rm));
         }
     }
     VOX_HIP(hipGetLastError());

@@ -2691,16 +2691,36 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
                                                       hb_sink sink, int keep, int gate_cols) {
     constexpr int U = 32 / VPL;
     const int row = blockIdx.x, hq = blockIdx.y, lane = threadIdx.x;
+    const float* src = part + (size_t)(row * H + hq) * nseg_grid * (vdim + 2);
+    // several segments' values on their way before the first is used; those of the first segments before it is known how many there are
+    // (the places of segments that do not exist are never used)
+    float v[U][VPL];
+    auto fetch = [&](int s0, int last) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const float* sp = src + (size_t)(s0 + u < last ? s0 + u : last) * (vdim + 2);
+#pragma unroll
+            for (int e = 0; e < VPL; ++e) {
+                const int j = lane + e * 64;
+                v[u][e] = j < vdim ? sp[j] : 0.f;
+            }
+        }
+    };
+    // lane s of each 64 segments fetches segment s's maximum and sum; the total is added in segment order
+    auto stat = [&](int s, int what) { return src[(size_t)(s < nseg_grid ? s : nseg_grid - 1) * (vdim + 2) + vdim + what]; };
+    float m0 = stat(lane, 0), l0 = stat(lane, 1);
+    fetch(0, nseg_grid - 1);
+    float gcol[VPL];
+#pragma unroll
+    for (int e = 0; e < VPL; ++e) gcol[e] = gate_cols && lane + e * 64 < vdim ? gate[(size_t)row * ldg + hq * vdim + lane + e * 64] : 0.f;
     const int p = pos[row];
     const int first = p - window + 1;
     const int lo = first > 0 ? first : 0;
     const int total = lo / P + (keep < lo ? keep : lo) + (p - lo + 1);
     const int nseg = ((total + chunk - 1) / chunk + seg_chunks - 1) / seg_chunks;
-    const float* src = part + (size_t)(row * H + hq) * nseg_grid * (vdim + 2);
-    // lane s of each 64 segments fetches segment s's maximum and sum; the total is added in segment order
     const float sk = sink.on ? hb_sink_of(sink, hq) : -INFINITY;      // sink: a key without a value
-    float mm = sk;
-    for (int s0 = 0; s0 < nseg; s0 += 64) mm = fmaxf(mm, s0 + lane < nseg ? src[(size_t)(s0 + lane) * (vdim + 2) + vdim] : -INFINITY);
+    float mm = fmaxf(sk, lane < nseg ? m0 : -INFINITY);
+    for (int s0 = 64; s0 < nseg; s0 += 64) mm = fmaxf(mm, s0 + lane < nseg ? stat(s0 + lane, 0) : -INFINITY);
     mm = hb_wave_max(mm);
     const float gmul = (gate && !gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq]) : 1.0f) * out_scale;
     float lt = 0.f;
@@ -2708,22 +2728,13 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
 #pragma unroll
     for (int e = 0; e < VPL; ++e) acc[e] = 0.f;
     for (int s0 = 0; s0 < nseg; s0 += 64) {
+        if (s0 > 0) { m0 = stat(s0 + lane, 0); l0 = stat(s0 + lane, 1); }
         const bool mine = s0 + lane < nseg;
-        const float wmine = mine ? expf(src[(size_t)(s0 + lane) * (vdim + 2) + vdim] - mm) : 0.f;
-        const float lmine = mine ? src[(size_t)(s0 + lane) * (vdim + 2) + vdim + 1] * wmine : 0.f;
+        const float wmine = mine ? expf(m0 - mm) : 0.f;
+        const float lmine = mine ? l0 * wmine : 0.f;
         const int ns = nseg - s0 < 64 ? nseg - s0 : 64;
         for (int s2 = 0; s2 < ns; s2 += U) {
-            // several segments' values on their way before the first is used
-            float v[U][VPL];
-#pragma unroll
-            for (int u = 0; u < U; ++u) {
-                const float* sp = src + (size_t)(s0 + (s2 + u < ns ? s2 + u : ns - 1)) * (vdim + 2);
-#pragma unroll
-                for (int e = 0; e < VPL; ++e) {
-                    const int j = lane + e * 64;
-                    v[u][e] = j < vdim ? sp[j] : 0.f;
-                }
-            }
+            if (s0 + s2 > 0) fetch(s0 + s2, nseg - 1);
 #pragma unroll
             for (int u = 0; u < U; ++u) {
                 if (s2 + u >= ns) break;
@@ -2738,7 +2749,7 @@ __global__ __launch_bounds__(64) void k_hb_attn_merge(const float* part, int nse
 #pragma unroll
     for (int e = 0; e < VPL; ++e) {
         const int j = lane + e * 64;
-        if (j < vdim) out[(size_t)row * ldo + hq * vdim + j] = acc[e] / lt * gmul * (gate_cols ? hb_sigmoid(gate[(size_t)row * ldg + hq * vdim + j]) : 1.0f);
+        if (j < vdim) out[(size_t)row * ldo + hq * vdim + j] = acc[e] / lt * gmul * (gate_cols ? hb_sigmoid(gcol[e]) : 1.0f);
     }
 }
 

@@ -2,11 +2,11 @@
 // unit behind a short convolution, a matrix state with token shift and per-channel decay, retention, the gated delta rule behind
 // short convolutions) or with attention over a paged cache (a sliding window that also keeps one mean key / value per block of
 // older tokens, plain causal attention with normed q / k / v -- optionally behind a short convolution, rotated, with a softmax
-// sink --, attention over a cached low-rank latent, or attention with independent sigmoid weights inside position chunks).  Two mixers
-// may run side by side on one input; a layer is sequential or parallel, with an optional layer scale or a gate on what joins the
-// residual sum, over one residual stream or several that are mixed at every sublayer; its feed-forward is dense or a routed mixture of
-// experts.  A contiguous range of layers
-// may run several times with the same weights; every run owns its cache or recurrent state.
+// sink --, attention over a cached low-rank latent, attention with independent sigmoid weights inside position chunks, or softmax
+// attention over a window and the first tokens).  Two mixers may run side by side on one input; a layer is sequential, parallel or
+// post-normed, with an optional layer scale or a gate on what joins the residual sum, over one residual stream or several that are mixed
+// at every sublayer; its feed-forward is dense or a routed mixture of experts.  A contiguous range of layers may run several times with the
+// same weights; every run owns its cache or recurrent state, or (window attention) reads the cache of an earlier run.
 //
 // Numeric rule of this engine: the residual stream, norms, rotary angles, attention scores / softmax, gates, decays and every
 // recurrent state are fp32.  The engine's dtype (bf16 or fp32) is the storage of the large matrices, of the K / V cache and of
@@ -768,13 +768,13 @@ __global__ __launch_bounds__(256) void k_hb_gemv(const float* A, long lda, const
         }
 }
 
-// One-row steps: the norm of the row (LayerNorm with a weight and, lnb != NULL, a bias; rms != 0: the RMS norm over the whole row) fused in front of the GEMV.
+// One-row steps: the norm of the row (LayerNorm with a weight and, BIASED, a bias; rms != 0: the RMS norm over the whole row) fused in front of the GEMV.
 // Every wave takes the row's statistics itself (mean, then the mean of the squared deviations; lane-chunked sums and a butterfly, an
 // order fixed by K), so the row is read from cache instead of from a normalised copy, and a dependent launch is saved.  NK > 0: a
 // lane's share of the row and of its weight rows (K <= 64 * CH * NK) is requested at the start and kept in registers, so the weights
 // are on their way while the statistics are taken; NK = 0: any K, several reads.  Same sums in the same order either way.  Needs
 // K % 8 == 0 (4 for fp32).
-template <typename T, int EPI, int CPW, int NK>
+template <typename T, int EPI, int CPW, int NK, bool BIASED>
 __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, const int* rows, const float* lnw, const float* lnb, float eps,
                                                     const T* Wt, const float* bias, float* C, int N, int K, int rms, float epi_arg) {
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CPW;
@@ -830,9 +830,12 @@ __global__ __launch_bounds__(256) void k_hb_ln_gemv(const float* X, long ldx, co
 #pragma unroll
         for (int e = 0; e < CH; e += 4) {
             const float4 x4 = xv[e / 4], g4 = *(const float4*)(lnw + k + e);
-            const float4 b4 = lnb ? *(const float4*)(lnb + k + e) : make_float4(0.f, 0.f, 0.f, 0.f);
-            const float x[4] = {hb_operand<T>((x4.x - mean) * inv * g4.x + b4.x), hb_operand<T>((x4.y - mean) * inv * g4.y + b4.y),
-                                hb_operand<T>((x4.z - mean) * inv * g4.z + b4.z), hb_operand<T>((x4.w - mean) * inv * g4.w + b4.w)};
+            float n[4] = {(x4.x - mean) * inv * g4.x, (x4.y - mean) * inv * g4.y, (x4.z - mean) * inv * g4.z, (x4.w - mean) * inv * g4.w};
+            if constexpr (BIASED) {
+                const float4 b4 = *(const float4*)(lnb + k + e);
+                n[0] += b4.x; n[1] += b4.y; n[2] += b4.z; n[3] += b4.w;
+            }
+            const float x[4] = {hb_operand<T>(n[0]), hb_operand<T>(n[1]), hb_operand<T>(n[2]), hb_operand<T>(n[3])};
 #pragma unroll
             for (int j = 0; j < CPW; ++j) {
                 const uint4 v = u[j];
@@ -886,19 +889,24 @@ bool hb_try_ln_gemv(hipStream_t st, int epi, const float* X, long ldx, const int
     const bool wide = N >= 16 * 1024;
     const dim3 g(wide ? (N + 15) / 16 : (N + 3) / 4), b(256);
     const int nk = (K + 64 * CH - 1) / (64 * CH);
-#define HB_LN2(EPI_, CPW_) \
+#define HB_LN2(EPI_, CPW_, B_) \
     do { \
-        if (nk <= 2) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 2>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
-        else if (nk <= 4) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 4>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
-        else if (nk <= 8) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 8>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
-        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 0>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        if (nk <= 2) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 2, B_>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 4) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 4, B_>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else if (nk <= 8) hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 8, B_>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
+        else hipLaunchKernelGGL((k_hb_ln_gemv<T, EPI_, CPW_, 0, B_>), g, b, 0, st, X, ldx, rows, lnw, lnb, eps, W, bias, C, N, K, rms, epi_arg); \
     } while (0)
 #define HB_LN(EPI_) \
     do { \
-        if (wide) HB_LN2(EPI_, 4); \
-        else HB_LN2(EPI_, 1); \
+        if (wide) HB_LN2(EPI_, 4, false); \
+        else HB_LN2(EPI_, 1, false); \
     } while (0)
-    if (epi == HB_EPI_GELU) HB_LN(HB_EPI_GELU);
+    if (lnb) {
+        // (biased norms: the plain product and the capped head)
+        if (epi == HB_EPI_SOFTCAP) { if (wide) HB_LN2(HB_EPI_SOFTCAP, 4, true); else HB_LN2(HB_EPI_SOFTCAP, 1, true); }
+        else if (epi == HB_EPI_STORE) { if (wide) HB_LN2(HB_EPI_STORE, 4, true); else HB_LN2(HB_EPI_STORE, 1, true); }
+        else return false;
+    } else if (epi == HB_EPI_GELU) HB_LN(HB_EPI_GELU);
     else if (epi == HB_EPI_SCALE) HB_LN(HB_EPI_SCALE);
     else if (epi == HB_EPI_RELU2) HB_LN(HB_EPI_RELU2);
     else if (epi == HB_EPI_SOFTCAP) HB_LN(HB_EPI_SOFTCAP);
